@@ -101,6 +101,8 @@ __device__ __forceinline__ float activate(float x, int act) {
   if (act == MS_ACT_GELU_TANH) return 0.5f * x * (1.f + tanhf(0.7978845608028654f * (x + 0.044715f * x * x * x)));
   return x / (1.f + expf(-x));
 }
+// log(1 + exp(z)) without overflow.
+__device__ __forceinline__ float softplus(float z) { return fmaxf(z, 0.f) + log1pf(expf(-fabsf(z))); }
 // What a gated feed-forward makes of one gate and one up value, float32.
 __device__ __forceinline__ float gated_value(float gate, float up, int act, float limit) {
   if (act == MS_ACT_SWIGLU_CLAMPED) {

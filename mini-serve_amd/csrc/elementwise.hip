@@ -47,20 +47,22 @@ extern "C" int ms_feed_tokens(int* ids, const int* row_start, const int* feed, c
 // y[r, :] = w * x[row(r), :] * rsqrt(mean(x^2) + eps), float32 throughout, rounded once.
 // With `parts` (float [splits, rows_total, width], the partial sums of a matrix product that still
 // has to be added to the residual stream) the row is first brought up to date: x[row] + sum over
-// splits in ascending order. Without a row list x is updated in place; with one x is left unchanged
-// (a list may name a row twice).
+// splits in ascending order, times `scale` [width] element by element where it is given. Without a row
+// list x is updated in place; with one x is left unchanged (a list may name a row twice).
 // One block of NT threads per row; each thread keeps up to KEEP of its elements in registers between
 // the two passes (wider rows are read again). Few rows (a decode step) run with 1024 threads so that
 // all loads of a row are in flight at once.
 template <typename TW, typename TO, int NT, int KEEP>
 __global__ __launch_bounds__(NT) void rmsnorm_kernel(float* __restrict__ x, const TW* __restrict__ w, TO* __restrict__ y,
                                                      const int* __restrict__ rows, int width, float eps,
-                                                     const float* __restrict__ parts, int splits, size_t split_stride) {
+                                                     const float* __restrict__ parts, int splits, size_t split_stride,
+                                                     const float* __restrict__ scale) {
   __shared__ float red[NT / WAVE];
   const int r = blockIdx.x;
   const size_t row = rows ? rows[r] : r;
   float* src = x + row * width;
   const bool in_place = parts != nullptr && rows == nullptr;
+  auto pending = [&](int i) { return sum_splits(parts + row * width + i, splits, split_stride) * (scale ? scale[i] : 1.f); };
   float kept[KEEP];
   float ss = 0.f;
 #pragma unroll
@@ -70,7 +72,7 @@ __global__ __launch_bounds__(NT) void rmsnorm_kernel(float* __restrict__ x, cons
     if (i < width) {
       v = src[i];
       if (parts != nullptr) {
-        v += sum_splits(parts + row * width + i, splits, split_stride);
+        v += pending(i);
         if (in_place) src[i] = v;
       }
     }
@@ -80,7 +82,7 @@ __global__ __launch_bounds__(NT) void rmsnorm_kernel(float* __restrict__ x, cons
   for (int i = threadIdx.x + KEEP * NT; i < width; i += NT) {  // rows wider than NT * KEEP
     float v = src[i];
     if (parts != nullptr) {
-      v += sum_splits(parts + row * width + i, splits, split_stride);
+      v += pending(i);
       if (in_place) src[i] = v;
     }
     ss += v * v;
@@ -95,7 +97,7 @@ __global__ __launch_bounds__(NT) void rmsnorm_kernel(float* __restrict__ x, cons
   }
   for (int i = threadIdx.x + KEEP * NT; i < width; i += NT) {
     float v = src[i];  // in place: this thread's own update; otherwise the sum is formed again
-    if (parts != nullptr && !in_place) v += sum_splits(parts + row * width + i, splits, split_stride);
+    if (parts != nullptr && !in_place) v += pending(i);
     dst[i] = from_f32<TO>(v * rstd * to_f32(w[i]));
   }
 }
@@ -139,7 +141,7 @@ template <typename TW, int NT>
 __global__ __launch_bounds__(NT) void rmsnorm_vec4_kernel(float* __restrict__ x, const TW* __restrict__ w,
                                                             bf16* __restrict__ y, const int* __restrict__ rows, int width,
                                                             float eps, const float* __restrict__ parts, int splits,
-                                                            size_t split_stride) {
+                                                            size_t split_stride, const float* __restrict__ scale) {
   __shared__ float red[NT / WAVE];
   const int r = blockIdx.x;
   const size_t row = rows ? rows[r] : r;
@@ -160,7 +162,9 @@ __global__ __launch_bounds__(NT) void rmsnorm_vec4_kernel(float* __restrict__ x,
         float4 acc = make_float4(0.f, 0.f, 0.f, 0.f);
         // The loads of a batch of splits go out together; few splits (a tile product's two to four) take
         // a batch of their own size, so that no load is issued for nothing. Ascending split order always.
-        if (splits <= 2) {
+        if (splits == 1) {
+          add_splits<1>(acc, p, 0, splits, split_stride);
+        } else if (splits <= 2) {
           add_splits<2>(acc, p, 0, splits, split_stride);
         } else if (splits <= 4) {
           add_splits<4>(acc, p, 0, splits, split_stride);
@@ -168,6 +172,10 @@ __global__ __launch_bounds__(NT) void rmsnorm_vec4_kernel(float* __restrict__ x,
           add_splits<8>(acc, p, 0, splits, split_stride);
         } else {  // the products of a decode step leave 12 to 16: one round trip, not two
           for (int s0 = 0; s0 < splits; s0 += 16) add_splits<16>(acc, p, s0, splits, split_stride);
+        }
+        if (scale != nullptr) {
+          const float4 s = *reinterpret_cast<const float4*>(scale + i);
+          acc.x *= s.x; acc.y *= s.y; acc.z *= s.z; acc.w *= s.w;
         }
         v.x += acc.x; v.y += acc.y; v.z += acc.z; v.w += acc.w;
         if (in_place) *reinterpret_cast<float4*>(src + i) = v;
@@ -194,7 +202,8 @@ __global__ __launch_bounds__(NT) void rmsnorm_vec4_kernel(float* __restrict__ x,
 }
 
 extern "C" int ms_rmsnorm(float* x, const void* w, int w_is_bf16, void* y, int y_is_bf16, const int* rows, int n_rows,
-                          int width, float eps, const float* parts, int splits, long long split_stride, hipStream_t st) {
+                          int width, float eps, const float* parts, int splits, long long split_stride, const float* scale,
+                          hipStream_t st) {
   if (n_rows <= 0) return MS_OK;
   if (width <= 0 || (parts != nullptr && splits < 1)) return MS_BAD_ARG;
   // float32 output keeps one block shape for every batch, so that its sums are formed in one order
@@ -204,10 +213,10 @@ extern "C" int ms_rmsnorm(float* x, const void* w, int w_is_bf16, void* y, int y
 #define LAUNCH_VEC(TW)                                                                                                  \
   if (width <= 2048)                                                                                                    \
     rmsnorm_vec4_kernel<TW, 256><<<n_rows, 256, 0, st>>>(x, (const TW*)w, (bf16*)y, rows, width, eps, parts, splits,    \
-                                                          (size_t)split_stride);                                        \
+                                                          (size_t)split_stride, scale);                                 \
   else                                                                                                                  \
     rmsnorm_vec4_kernel<TW, 1024><<<n_rows, 1024, 0, st>>>(x, (const TW*)w, (bf16*)y, rows, width, eps, parts, splits,  \
-                                                            (size_t)split_stride)
+                                                            (size_t)split_stride, scale)
     if (w_is_bf16) { LAUNCH_VEC(bf16); } else { LAUNCH_VEC(float); }
 #undef LAUNCH_VEC
     return launch_status();
@@ -215,10 +224,10 @@ extern "C" int ms_rmsnorm(float* x, const void* w, int w_is_bf16, void* y, int y
 #define LAUNCH(TW, TO)                                                                                                  \
   if (wide)                                                                                                             \
     rmsnorm_kernel<TW, TO, 1024, 4><<<n_rows, 1024, 0, st>>>(x, (const TW*)w, (TO*)y, rows, width, eps, parts, splits,  \
-                                                              (size_t)split_stride);                                    \
+                                                              (size_t)split_stride, scale);                             \
   else                                                                                                                  \
     rmsnorm_kernel<TW, TO, 256, 8><<<n_rows, 256, 0, st>>>(x, (const TW*)w, (TO*)y, rows, width, eps, parts, splits,    \
-                                                            (size_t)split_stride)
+                                                            (size_t)split_stride, scale)
   if (w_is_bf16 && y_is_bf16) { LAUNCH(bf16, bf16); }
   else if (w_is_bf16) { LAUNCH(bf16, float); }
   else if (y_is_bf16) { LAUNCH(float, bf16); }

@@ -995,22 +995,24 @@ __global__ __launch_bounds__(256) void gemm_bf16_small_kernel(const bf16* __rest
   for (int i = 0; i < MB; ++i) store4(dst, 1, i * 16 + r, nb + g * 4, M, N, N, acc[i], N % 4 == 0);
 }
 
-// C (mode 0 bf16 / 1 float / 2 float +=) from the partial sums, in ascending split order.
+// C (mode 0 bf16 / 1 float / 2 float +=) from the partial sums, in ascending split order, times `scale` [N] element by
+// element where it is given.
 __global__ void splitk_reduce_kernel(const float* __restrict__ P, void* __restrict__ C, int mode, int splits, int M,
-                                     int N, int ldc) {
+                                     int N, int ldc, const float* __restrict__ scale) {
   const int n = blockIdx.x * blockDim.x + threadIdx.x, m = blockIdx.y;
   if (n >= N) return;
-  const float v = sum_splits(P + (size_t)m * N + n, splits, (size_t)M * N);
+  const float v = sum_splits(P + (size_t)m * N + n, splits, (size_t)M * N) * (scale ? scale[n] : 1.f);
   const size_t at = (size_t)m * ldc + n;
   if (mode == 0) ((bf16*)C)[at] = static_cast<bf16>(v);
   else if (mode == 1) ((float*)C)[at] = v;
   else ((float*)C)[at] += v;
 }
 
-extern "C" int ms_splitk_reduce(const float* P, void* C, int mode, int splits, int M, int N, int ldc, hipStream_t st) {
+extern "C" int ms_splitk_reduce(const float* P, void* C, int mode, int splits, int M, int N, int ldc, const float* scale,
+                                hipStream_t st) {
   if (M <= 0 || N <= 0) return MS_OK;
   if (splits < 1 || ldc < N || mode < 0 || mode > 2 || M > 65535) return MS_BAD_ARG;
-  splitk_reduce_kernel<<<dim3((N + 255) / 256, M), 256, 0, st>>>(P, C, mode, splits, M, N, ldc);
+  splitk_reduce_kernel<<<dim3((N + 255) / 256, M), 256, 0, st>>>(P, C, mode, splits, M, N, ldc, scale);
   return launch_status();
 }
 
@@ -1272,7 +1274,7 @@ extern "C" int ms_gemm_bf16_small(const void* X, const void* W, float* partials,
     if (rc != MS_OK) return rc;
     if (reduce) {
       if (C == nullptr || ldc < N || mode < 0 || mode > 2) return MS_BAD_ARG;
-      splitk_reduce_kernel<<<dim3((N + 255) / 256, M), 256, 0, st>>>(partials, C, mode, splits, M, N, ldc);
+      splitk_reduce_kernel<<<dim3((N + 255) / 256, M), 256, 0, st>>>(partials, C, mode, splits, M, N, ldc, nullptr);
     }
     return launch_status();
   }
@@ -1291,7 +1293,7 @@ extern "C" int ms_gemm_bf16_small(const void* X, const void* W, float* partials,
   else gemm_bf16_small_kernel<4, true><<<(unsigned)wide_blocks, 256, 0, st>>>(x, w, partials, M, N, K, ldx, per, splits);
   if (reduce) {
     if (C == nullptr || ldc < N || mode < 0 || mode > 2) return MS_BAD_ARG;
-    splitk_reduce_kernel<<<dim3((N + 255) / 256, M), 256, 0, st>>>(partials, C, mode, splits, M, N, ldc);
+    splitk_reduce_kernel<<<dim3((N + 255) / 256, M), 256, 0, st>>>(partials, C, mode, splits, M, N, ldc, nullptr);
   }
   return launch_status();
 }

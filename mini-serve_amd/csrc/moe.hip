@@ -76,15 +76,16 @@ extern "C" int ms_moe_route(const float* logits, int ld, int splits, long long s
 }
 
 // ---------------------------------------------------------------------------------------------
-// Routing by scores: s = softmax(logits[t]) over all E outputs; the choice is made by c = s + correction (correction may
-// be absent), the weights are the chosen outputs' s as they stand (not renormalised). With groups > 1 the E outputs form
+// Routing by scores: s = softmax(logits[t]) over all E outputs, or, `sigmoid`, s = 1 / (1 + exp(-logits[t])) each on its own;
+// the choice is made by c = s + correction (correction may be absent; sigmoid scores without one are chosen by their logits,
+// which are in the same order and do not saturate), the weights are the chosen outputs' s as they stand (not renormalised). With groups > 1 the E outputs form
 // `groups` equal groups of neighbours, a group's score is its largest c, and only outputs of the `keep` best groups
 // (ties: the lower group) can be chosen: the others' c counts as minus infinity. The `top` largest c are chosen, largest
 // first (ties: the lower index). One wave per token; s and c of a token pass through the wave's own rows of LDS.
 template <typename TB>
 __global__ __launch_bounds__(256) void moe_route_scored_kernel(const float* __restrict__ logits, int ld, int splits, size_t stride,
                                                                const TB* __restrict__ correction, int T, int E, int top,
-                                                               int groups, int keep, int* __restrict__ ids,
+                                                               int groups, int keep, int sigmoid, int* __restrict__ ids,
                                                                float* __restrict__ weights) {
   __shared__ float ss[4][MOE_MAX_EXPERTS], cs[4][MOE_MAX_EXPERTS];
   const int wave = threadIdx.x / WAVE, lane = threadIdx.x % WAVE;
@@ -102,7 +103,7 @@ __global__ __launch_bounds__(256) void moe_route_scored_kernel(const float* __re
   float sum = 0.f;
 #pragma unroll
   for (int i = 0; i < MOE_MAX_EXPERTS / WAVE; ++i) {
-    c[i] = lane + i * WAVE < E ? expf(c[i] - m) : 0.f;
+    if (!sigmoid) c[i] = lane + i * WAVE < E ? expf(c[i] - m) : 0.f;
     sum += c[i];
   }
   sum = wave_sum(sum);
@@ -110,9 +111,9 @@ __global__ __launch_bounds__(256) void moe_route_scored_kernel(const float* __re
   for (int i = 0; i < MOE_MAX_EXPERTS / WAVE; ++i) {
     const int e = lane + i * WAVE;
     if (e < E) {
-      const float sc = c[i] / sum;
+      const float sc = sigmoid ? 1.f / (1.f + expf(-c[i])) : c[i] / sum;
       ss[wave][e] = sc;
-      c[i] = sc + (correction ? to_f32(correction[e]) : 0.f);
+      if (correction || !sigmoid) c[i] = sc + (correction ? to_f32(correction[e]) : 0.f);
       cs[wave][e] = c[i];
     } else {
       c[i] = -INFINITY;
@@ -185,16 +186,16 @@ __global__ __launch_bounds__(256) void moe_route_scored_kernel(const float* __re
 }
 
 extern "C" int ms_moe_route_scored(const float* logits, int ld, int splits, long long stride, const void* correction,
-                                   int correction_is_bf16, int T, int E, int top, int groups, int keep, int* ids, float* weights,
-                                   hipStream_t st) {
+                                   int correction_is_bf16, int T, int E, int top, int groups, int keep, int sigmoid, int* ids,
+                                   float* weights, hipStream_t st) {
   if (T <= 0) return MS_OK;
   if (logits == nullptr || ids == nullptr || weights == nullptr || E < 1 || top < 1 || top > E || ld < E || splits < 1 ||
       (splits > 1 && stride < (long long)T * ld) || groups < 1 || E % groups || keep < 1 || keep > groups)
     return MS_BAD_ARG;
   if (E > MOE_MAX_EXPERTS || top > MOE_MAX_TOP) return MS_UNSUPPORTED;
   const unsigned blocks = (unsigned)((T + 3) / 4);
-  if (correction_is_bf16) moe_route_scored_kernel<bf16><<<blocks, 256, 0, st>>>(logits, ld, splits, (size_t)stride, (const bf16*)correction, T, E, top, groups, keep, ids, weights);
-  else moe_route_scored_kernel<float><<<blocks, 256, 0, st>>>(logits, ld, splits, (size_t)stride, (const float*)correction, T, E, top, groups, keep, ids, weights);
+  if (correction_is_bf16) moe_route_scored_kernel<bf16><<<blocks, 256, 0, st>>>(logits, ld, splits, (size_t)stride, (const bf16*)correction, T, E, top, groups, keep, sigmoid, ids, weights);
+  else moe_route_scored_kernel<float><<<blocks, 256, 0, st>>>(logits, ld, splits, (size_t)stride, (const float*)correction, T, E, top, groups, keep, sigmoid, ids, weights);
   return launch_status();
 }
 
@@ -268,6 +269,8 @@ extern "C" int ms_moe_plan(const int* ids, int P, int E, int tile_rows, int max_
 //   MODE 2 (plain first product): the same rows, one weight per expert; act(up) goes to h[sorted place][N].
 //   MODE 0: rows are h[sorted place] (K = the experts' width), one weight per expert [E, N, K]; the result times the pair's
 //          routing weight goes to y[pair][N] in float32.
+// The routing weights may belong in front of the expert instead: given to a first product they multiply its float32
+// results, W (w x) = w (W x), before the activation; the second product is then given none.
 typedef __attribute__((__vector_size__(8 * sizeof(__bf16)))) __bf16 moe_bf16x8;
 typedef __attribute__((__vector_size__(4 * sizeof(float)))) float moe_floatx4;
 
@@ -372,19 +375,19 @@ __global__ __launch_bounds__(256) void moe_gemm_bf16_kernel(
   for (int r = 0; r < 4; ++r) {
     const int m = m0 + grp * 4 + r;
     if (m >= count) continue;
+    const int pair = order[start + m];
+    const float pw = pair_weight ? pair_weight[pair] : 1.f;
     if (GATED) {
       bf16* o = (bf16*)out + (size_t)(start + m) * N + n0 + l16;
 #pragma unroll
       for (int nt = 0; nt < NT; ++nt)
-        if (col_ok[nt]) o[nt * 16] = static_cast<bf16>(gated_value(acc1[nt][r], acc2[nt][r], act, 0.f));
+        if (col_ok[nt]) o[nt * 16] = static_cast<bf16>(gated_value(acc1[nt][r] * pw, acc2[nt][r] * pw, act, 0.f));
     } else if (FIRST) {
       bf16* o = (bf16*)out + (size_t)(start + m) * N + n0 + l16;
 #pragma unroll
       for (int nt = 0; nt < NT; ++nt)
-        if (col_ok[nt]) o[nt * 16] = static_cast<bf16>(activate(acc1[nt][r], act));
+        if (col_ok[nt]) o[nt * 16] = static_cast<bf16>(activate(acc1[nt][r] * pw, act));
     } else {
-      const int pair = order[start + m];
-      const float pw = pair_weight[pair];
       float* o = (float*)out + (size_t)pair * N + n0 + l16;
 #pragma unroll
       for (int nt = 0; nt < NT; ++nt)
@@ -504,6 +507,8 @@ __global__ __launch_bounds__(256, 2) void moe_gemm_bf16_lds_kernel(
   for (int j = 0; j < FM; ++j) {
     const int m = wm + j * 16 + r;
     if (m >= count) continue;
+    const int pair = order[start + m];
+    const float pw = pair_weight ? pair_weight[pair] : 1.f;
     if (GATED) {
       bf16* o = (bf16*)out + (size_t)(start + m) * N;
 #pragma unroll
@@ -511,7 +516,7 @@ __global__ __launch_bounds__(256, 2) void moe_gemm_bf16_lds_kernel(
         const int col = n0 + wn / 2 + (i / 2) * 16 + g * 4;
         union { uint2 u; bf16 v[4]; } q;
 #pragma unroll
-        for (int c = 0; c < 4; ++c) q.v[c] = static_cast<bf16>(gated_value(acc[i][j][c], acc[i + 1][j][c], act, 0.f));
+        for (int c = 0; c < 4; ++c) q.v[c] = static_cast<bf16>(gated_value(acc[i][j][c] * pw, acc[i + 1][j][c] * pw, act, 0.f));
         if (vec && col + 3 < N) *reinterpret_cast<uint2*>(o + col) = q.u;
         else
 #pragma unroll
@@ -525,7 +530,7 @@ __global__ __launch_bounds__(256, 2) void moe_gemm_bf16_lds_kernel(
         const int col = n0 + wn + i * 16 + g * 4;
         union { uint2 u; bf16 v[4]; } q;
 #pragma unroll
-        for (int c = 0; c < 4; ++c) q.v[c] = static_cast<bf16>(activate(acc[i][j][c], act));
+        for (int c = 0; c < 4; ++c) q.v[c] = static_cast<bf16>(activate(acc[i][j][c] * pw, act));
         if (vec && col + 3 < N) *reinterpret_cast<uint2*>(o + col) = q.u;
         else
 #pragma unroll
@@ -533,8 +538,6 @@ __global__ __launch_bounds__(256, 2) void moe_gemm_bf16_lds_kernel(
             if (col + c < N) o[col + c] = q.v[c];
       }
     } else {
-      const int pair = order[start + m];
-      const float pw = pair_weight[pair];
       float* o = (float*)out + (size_t)pair * N;
 #pragma unroll
       for (int i = 0; i < FN; ++i) {
@@ -636,14 +639,14 @@ __global__ __launch_bounds__(256) void moe_gemm_f32_kernel(
   for (int i = 0; i < 4; ++i) {
     const int m = ty * 4 + i;
     if (m >= count) continue;
-    const int pair = FIRST ? 0 : order[start + m];
-    const float pw = FIRST ? 1.f : pair_weight[pair];
+    const int pair = order[start + m];
+    const float pw = pair_weight ? pair_weight[pair] : 1.f;
 #pragma unroll
     for (int j = 0; j < 4; ++j) {
       const int n = n0 + tx * 4 + j;
       if (n >= N) continue;
-      if (GATED) out[(size_t)(start + m) * N + n] = gated_value(acc1[i][j], acc2[i][j], act, 0.f);
-      else if (FIRST) out[(size_t)(start + m) * N + n] = activate(acc1[i][j], act);
+      if (GATED) out[(size_t)(start + m) * N + n] = gated_value(acc1[i][j] * pw, acc2[i][j] * pw, act, 0.f);
+      else if (FIRST) out[(size_t)(start + m) * N + n] = activate(acc1[i][j] * pw, act);
       else out[(size_t)pair * N + n] = acc1[i][j] * pw;
     }
   }
@@ -659,7 +662,7 @@ extern "C" int ms_moe_gemm(const void* a, int lda, const void* w1, const void* w
   if (max_tiles <= 0 || N <= 0) return MS_OK;
   const bool gated = mode == 1;
   if (mode < 0 || mode > 2 || a == nullptr || w1 == nullptr || (gated && w2 == nullptr) || out == nullptr || order == nullptr ||
-      tile_expert == nullptr || tile_start == nullptr || tile_count == nullptr || (mode == 0 && pair_weight == nullptr) || top < 1 ||
+      tile_expert == nullptr || tile_start == nullptr || tile_count == nullptr || top < 1 ||
       K <= 0 || lda < K || (gated && (act < 0 || act >= MS_ACT_COUNT)) || (mode == 2 && !ms_act_ungated_ok(act)))
     return MS_BAD_ARG;
   if (is_bf16) {
@@ -716,12 +719,12 @@ extern "C" int ms_moe_gemm(const void* a, int lda, const void* w1, const void* w
 }
 
 // ---------------------------------------------------------------------------------------------
-// stream[t][n] += sum over j < top of y[t * top + j][n], in ascending j. With ids: a choice whose id is `real` or more is
+// stream[t][n] += scale[n] (where it is given) times the sum over j < top of y[t * top + j][n], in ascending j. With ids: a choice whose id is `real` or more is
 // an identity expert, and its term is weights[t * top + j] * x[t][n] (y holds nothing for it).
 template <typename TX>
 __global__ void moe_combine_kernel(float* __restrict__ stream, const float* __restrict__ y, int top, int N,
                                    const int* __restrict__ ids, const float* __restrict__ weights, const TX* __restrict__ x,
-                                   int ldx, int real) {
+                                   int ldx, int real, const float* __restrict__ scale) {
   const int n = blockIdx.x * blockDim.x + threadIdx.x;
   if (n >= N) return;
   const size_t t = blockIdx.y;
@@ -730,16 +733,16 @@ __global__ void moe_combine_kernel(float* __restrict__ stream, const float* __re
     if (ids != nullptr && ids[t * top + j] >= real) acc += weights[t * top + j] * to_f32(x[t * ldx + n]);
     else acc += y[(t * top + j) * N + n];
   }
-  stream[t * N + n] += acc;
+  stream[t * N + n] += scale ? acc * scale[n] : acc;
 }
 
 extern "C" int ms_moe_combine(float* stream, const float* y, int T, int top, int N, const int* ids, const float* weights,
-                              const void* x, int x_is_bf16, int ldx, int real, hipStream_t st) {
+                              const void* x, int x_is_bf16, int ldx, int real, const float* scale, hipStream_t st) {
   if (T <= 0 || N <= 0) return MS_OK;
   if (stream == nullptr || y == nullptr || top < 1 || T > 65535 || (ids != nullptr && (weights == nullptr || x == nullptr || ldx < N)))
     return MS_BAD_ARG;
   const dim3 grid((N + 255) / 256, T);
-  if (x_is_bf16) moe_combine_kernel<bf16><<<grid, 256, 0, st>>>(stream, y, top, N, ids, weights, (const bf16*)x, ldx, real);
-  else moe_combine_kernel<float><<<grid, 256, 0, st>>>(stream, y, top, N, ids, weights, (const float*)x, ldx, real);
+  if (x_is_bf16) moe_combine_kernel<bf16><<<grid, 256, 0, st>>>(stream, y, top, N, ids, weights, (const bf16*)x, ldx, real, scale);
+  else moe_combine_kernel<float><<<grid, 256, 0, st>>>(stream, y, top, N, ids, weights, (const float*)x, ldx, real, scale);
   return launch_status();
 }

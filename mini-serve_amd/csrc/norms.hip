@@ -72,13 +72,14 @@ extern "C" int ms_layernorm(const float* x, const void* w, const void* b, int w_
 // ---------------------------------------------------------------------------------------------
 // y[t, g * group + e] = x[t, g * group + e] * rsqrt(mean over the group of x^2 + eps) * w[g * group + e]
 //                       * sigmoid(gate[t * gate_stride + g * group + e])     (gate_act = 1: SiLU instead of the sigmoid)
+// gate_first: the gate multiplies x before the group's mean of squares is taken instead of the normed result.
 // w == nullptr: no weight; gate == nullptr: no gate. One wave per (token, group) when the group is at
 // most 256 wide (four groups per block), else one block per (token, group).
 template <typename TW, typename TO>
 __global__ __launch_bounds__(256) void group_rmsnorm_gate_kernel(const float* __restrict__ x, const TW* __restrict__ w,
                                                                  const float* __restrict__ gate, int gate_stride,
                                                                  TO* __restrict__ y, int groups, int group, float eps,
-                                                                 int per_wave, int gate_act) {
+                                                                 int per_wave, int gate_act, int gate_first) {
   __shared__ float red[256 / WAVE];
   const int t = blockIdx.x;
   const int width = groups * group;
@@ -94,34 +95,53 @@ __global__ __launch_bounds__(256) void group_rmsnorm_gate_kernel(const float* __
   }
   const bool live = g < groups;
   const float* xr = x + (size_t)t * width + (size_t)(live ? g : 0) * group;
+  const float* gr = gate != nullptr ? gate + (size_t)t * gate_stride + (size_t)(live ? g : 0) * group : nullptr;
+  auto gated = [&](float v, int e) {
+    const float z = gr[e];
+    return v * ((gate_act ? z : 1.f) / (1.f + expf(-z)));  // times sigmoid(z), or z sigmoid(z)
+  };
+  const bool before = gate_first && gr != nullptr, after = !gate_first && gr != nullptr;
+  constexpr int KEEP = 16;  // elements a thread keeps between the two passes (wider groups are formed again)
+  float kept[KEEP];
   float s = 0.f;
+#pragma unroll
+  for (int i = 0; i < KEEP; ++i) {
+    const int e = first + i * step;
+    kept[i] = 0.f;
+    if (live && e < group) kept[i] = before ? gated(xr[e], e) : xr[e];
+    s += kept[i] * kept[i];
+  }
   if (live)
-    for (int e = first; e < group; e += step) s += xr[e] * xr[e];
+    for (int e = first + KEEP * step; e < group; e += step) {
+      const float v = before ? gated(xr[e], e) : xr[e];
+      s += v * v;
+    }
   s = per_wave ? wave_sum(s) : block_sum<256>(s, red);
   if (!live) return;
   const float rstd = 1.f / sqrtf(s / (float)group + eps);
-  for (int e = first; e < group; e += step) {
+  auto store = [&](float v, int e) {
     const int c = g * group + e;
-    float o = xr[e] * rstd;
+    float o = v * rstd;
     if (w != nullptr) o *= to_f32(w[c]);
-    if (gate != nullptr) {
-      const float z = gate[(size_t)t * gate_stride + c];
-      o *= (gate_act ? z : 1.f) / (1.f + expf(-z));  // sigmoid(z), or z sigmoid(z)
-    }
+    if (after) o = gated(o, e);
     y[(size_t)t * width + c] = from_f32<TO>(o);
-  }
+  };
+#pragma unroll
+  for (int i = 0; i < KEEP; ++i)
+    if (first + i * step < group) store(kept[i], first + i * step);
+  for (int e = first + KEEP * step; e < group; e += step) store(before ? gated(xr[e], e) : xr[e], e);
 }
 
 extern "C" int ms_group_rmsnorm_gate(const float* x, const void* w, int w_is_bf16, const float* gate, int gate_stride,
                                      void* y, int y_is_bf16, int tokens, int groups, int group, float eps, int gate_act,
-                                     hipStream_t st) {
+                                     int gate_first, hipStream_t st) {
   if (tokens <= 0) return MS_OK;
-  if ((gate_act != 0 && gate_act != 1) || groups <= 0 || group <= 0 || tokens > 65535 * 32 || !(eps >= 0.f) || (gate != nullptr && gate_stride < groups * group))
+  if ((gate_act != 0 && gate_act != 1) || (gate_first && gate == nullptr) || groups <= 0 || group <= 0 || tokens > 65535 * 32 || !(eps >= 0.f) || (gate != nullptr && gate_stride < groups * group))
     return MS_BAD_ARG;
   const int per_wave = group <= 256;
   const dim3 grid(tokens, per_wave ? (groups + 3) / 4 : groups);
   if (grid.y > 65535) return MS_UNSUPPORTED;
-#define GN(TW, TO) group_rmsnorm_gate_kernel<TW, TO><<<grid, 256, 0, st>>>(x, (const TW*)w, gate, gate_stride, (TO*)y, groups, group, eps, per_wave, gate_act)
+#define GN(TW, TO) group_rmsnorm_gate_kernel<TW, TO><<<grid, 256, 0, st>>>(x, (const TW*)w, gate, gate_stride, (TO*)y, groups, group, eps, per_wave, gate_act, gate_first)
   if (w_is_bf16) { if (y_is_bf16) GN(bf16, bf16); else GN(bf16, float); }
   else { if (y_is_bf16) GN(float, bf16); else GN(float, float); }
 #undef GN

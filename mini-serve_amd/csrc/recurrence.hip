@@ -1,6 +1,6 @@
 // Linear recurrences over a matrix state per (request, head), token by token:
 //     S_t = a_t S_(t-1) + b_t k_t v_t^T,   o_t = S_t^T q_t          (S: [D, E], k, q: [D], v: [E])
-// in two forms that differ in where a_t and b_t come from:
+// in forms that differ in where a_t and b_t come from:
 //   MS_REC_DECAY: a_t = decay[head] (a constant per head), b_t = 1; o_t as above.
 //   MS_REC_EXP_GATES: a log input gate i_t and a log forget gate f_t per head and token, made bounded by a soft cap,
 //       i = cap tanh((x_i + bias_i) / cap), f = logsigmoid(cap tanh((x_f + bias_f) / cap)), and a running maximum
@@ -10,6 +10,9 @@
 //   MS_REC_WKV: a decay per key channel and token, w_t [D] (its logarithm is row t of the float32 matrix `w`, columns h D ..), and a bonus
 //       u [H, D] that only the current token gets: o_t = (S_(t-1) + diag(u) k_t v_t^T)^T q_t, and only then
 //       S_t = diag(w_t) S_(t-1) + k_t v_t^T.
+//   MS_REC_STEP: both from one step size per head and token, d_t = softplus(w_t + bias) (column h of the matrix `w`):
+//       a_t = exp(decay[head] d_t), b_t = d_t; a share of the value joins the output, o_t = S_t^T q_t + u[head] v_t. `share`
+//       consecutive heads read the same q and k.
 // q, k, v (and the gates' inputs) are columns of one float32 matrix x [tokens, ld] (the layer's projections);
 // an activation (none or SiLU) is applied to q, k and v on the way in, q is then scaled by q_scale. Everything
 // is float32. The state lives in S [slots, H, D, E] (and n [slots, H, D], m [slots, H]); a row whose
@@ -27,6 +30,7 @@
 #define MS_REC_DECAY 0
 #define MS_REC_EXP_GATES 1
 #define MS_REC_WKV 2
+#define MS_REC_STEP 3
 
 struct RecurrenceArgs {
   const float* x;
@@ -44,9 +48,10 @@ struct RecurrenceArgs {
   const int* starts;
   const int* state_slots;
   float* out;
-  const float* w;  // MS_REC_WKV: the decays' logarithms [tokens, ld_w], head h's D channels from column h D on
+  const float* w;  // MS_REC_WKV: the decays' logarithms [tokens, ld_w], head h's D channels from column h D on; MS_REC_STEP: the steps [tokens, ld_w]
   int ld_w;
-  const float* u;  // MS_REC_WKV: the bonus [H, D]
+  const float* u;  // MS_REC_WKV: the bonus [H, D]; MS_REC_STEP: the value's share of the output [H]
+  int share;       // heads that read the same q and k (1 but for MS_REC_STEP)
 };
 
 __device__ __forceinline__ float rec_act(float v, int act) { return act ? v / (1.f + expf(-v)) : v; }
@@ -71,7 +76,8 @@ __global__ __launch_bounds__(256) void gated_recurrence_kernel(RecurrenceArgs a,
   const bool fresh = a.starts[b] == 0;
   const size_t slot = (size_t)a.state_slots[b];
   float* Sg = a.S + (slot * a.H + h) * (size_t)D * E;
-  const bool gates = a.mode == MS_REC_EXP_GATES, wkv = a.mode == MS_REC_WKV;
+  const bool gates = a.mode == MS_REC_EXP_GATES, wkv = a.mode == MS_REC_WKV, steps = a.mode == MS_REC_STEP;
+  const int hq = steps ? h / a.share : h;
   if (wkv && tid < D) us[tid] = a.u[h * D + tid];  // read behind the first token's barrier
   float S[PM];
 #pragma unroll
@@ -85,7 +91,7 @@ __global__ __launch_bounds__(256) void gated_recurrence_kernel(RecurrenceArgs a,
     m = a.m[slot * a.H + h];
   }
   const float decay = (gates || wkv) ? 0.f : a.decay[h];
-  const float bi = gates ? rec_bias(a.i_bias, a.bias_is_bf16, h) : 0.f;
+  const float bi = (gates || steps) ? rec_bias(a.i_bias, a.bias_is_bf16, h) : 0.f;
   const float bf = gates ? rec_bias(a.f_bias, a.bias_is_bf16, h) : 0.f;
   for (int t = t0; t < t1; ++t) {
     const float* xr = a.x + (size_t)t * a.ld;
@@ -99,10 +105,14 @@ __global__ __launch_bounds__(256) void gated_recurrence_kernel(RecurrenceArgs a,
       is = expf(gi - m_new);
       m = m_new;
     }
+    if (steps) {
+      is = softplus(a.w[(size_t)t * a.ld_w + h] + bi);
+      fs = expf(decay * is);
+    }
     float kd = 0.f, qd = 0.f;
     if (tid < D) {
-      qd = rec_act(xr[a.q_off + h * D + tid], a.act) * a.q_scale;
-      kd = rec_act(xr[a.k_off + h * D + tid], a.act);
+      qd = rec_act(xr[a.q_off + hq * D + tid], a.act) * a.q_scale;
+      kd = rec_act(xr[a.k_off + hq * D + tid], a.act);
       qs[buf][tid] = qd;
       ks[buf][tid] = kd;
       if (wkv) ws[buf][tid] = expf(a.w[(size_t)t * a.ld_w + h * D + tid]);
@@ -143,6 +153,7 @@ __global__ __launch_bounds__(256) void gated_recurrence_kernel(RecurrenceArgs a,
         const float nq = (wred[buf][0] + wred[buf][1]) + (wred[buf][2] + wred[buf][3]);
         acc = acc / (fmaxf(fabsf(nq), expf(-m)) + 1e-6f);
       }
+      if (steps) acc += a.u[h] * v;
       a.out[(size_t)t * (a.H * E) + h * E + e] = acc;
     }
   }
@@ -161,7 +172,7 @@ extern "C" int ms_gated_recurrence(const float* x, int ld, int q_off, int k_off,
                                    int E, int act, int mode, float q_scale, float cap, const float* decay, const void* i_bias,
                                    const void* f_bias, int bias_is_bf16, float* S, float* n, float* m, const int* row_start,
                                    const int* starts, const int* state_slots, float* out, int rows, const float* w, int ld_w,
-                                   const float* u, hipStream_t st) {
+                                   const float* u, int share, hipStream_t st) {
   if (rows <= 0) return MS_OK;
   if (H <= 0 || D <= 0 || E <= 0 || x == nullptr || S == nullptr || out == nullptr || row_start == nullptr || starts == nullptr ||
       state_slots == nullptr || (act != 0 && act != 1) || q_off < 0 || k_off < 0 || v_off < 0)
@@ -174,6 +185,8 @@ extern "C" int ms_gated_recurrence(const float* x, int ld, int q_off, int k_off,
     if (n == nullptr || m == nullptr || !(cap > 0.f) || i_off < 0 || f_off < 0 || i_off + H > ld || f_off + H > ld) return MS_BAD_ARG;
   } else if (mode == MS_REC_WKV) {
     if (w == nullptr || u == nullptr || ld_w < H * D) return MS_BAD_ARG;
+  } else if (mode == MS_REC_STEP) {
+    if (decay == nullptr || w == nullptr || u == nullptr || ld_w < H || share < 1 || H % share) return MS_BAD_ARG;
   } else {
     return MS_BAD_ARG;
   }
@@ -182,7 +195,7 @@ extern "C" int ms_gated_recurrence(const float* x, int ld, int q_off, int k_off,
   const int EB = E < 32 ? E : 32, EP = 32;
   const int per = (D + 256 / EP - 1) / (256 / EP);
   RecurrenceArgs a{x, ld, q_off, k_off, v_off, i_off, f_off, H, D, E, act, mode, q_scale, cap, decay, i_bias, f_bias, bias_is_bf16,
-                   S, n, m, row_start, starts, state_slots, out, w, ld_w, u};
+                   S, n, m, row_start, starts, state_slots, out, w, ld_w, u, share};
   const dim3 grid(rows, H, (E + EB - 1) / EB);
   if (per <= 4) gated_recurrence_kernel<4><<<grid, 256, 0, st>>>(a, EP, EB);
   else if (per <= 16) gated_recurrence_kernel<16><<<grid, 256, 0, st>>>(a, EP, EB);

@@ -238,24 +238,25 @@ extern "C" int ms_latent_prepare(const float* x, int ld, int q_col, int kv_col, 
 }
 
 // ---------------------------------------------------------------------------------------------
-// A gate per head: o[t][h][:] *= sigmoid(x[t][col + h]), in place; x float32 with row stride ld, o [tokens, H * E].
+// A gate: o[t][h][:] *= sigmoid(x[t][col + h]), in place, or, `each`, a gate per element, o[t][h][e] *= sigmoid(x[t][col + h E + e]);
+// x float32 with row stride ld, o [tokens, H * E].
 template <typename T>
-__global__ void head_gate_kernel(T* __restrict__ o, const float* __restrict__ x, int ld, int col, int H, int E, size_t n) {
+__global__ void head_gate_kernel(T* __restrict__ o, const float* __restrict__ x, int ld, int col, int H, int E, int each, size_t n) {
   const size_t i = (size_t)blockIdx.x * blockDim.x + threadIdx.x;
   if (i >= n) return;
   const size_t t = i / ((size_t)H * E);
-  const int h = (int)((i / E) % H);
-  const float g = 1.f / (1.f + expf(-x[t * ld + col + h]));
+  const int c = each ? (int)(i % ((size_t)H * E)) : (int)((i / E) % H);
+  const float g = 1.f / (1.f + expf(-x[t * ld + col + c]));
   o[i] = from_f32<T>(to_f32(o[i]) * g);
 }
 
-extern "C" int ms_head_gate(void* o, int is_bf16, const float* x, int ld, int col, int tokens, int H, int E, hipStream_t st) {
+extern "C" int ms_head_gate(void* o, int is_bf16, const float* x, int ld, int col, int tokens, int H, int E, int each, hipStream_t st) {
   if (tokens <= 0) return MS_OK;
-  if (H <= 0 || E <= 0 || col < 0 || ld < col + H) return MS_BAD_ARG;
+  if (H <= 0 || E <= 0 || col < 0 || ld < col + (each ? H * E : H)) return MS_BAD_ARG;
   const size_t n = (size_t)tokens * H * E;
   const unsigned blocks = (unsigned)((n + 255) / 256);
-  if (is_bf16) head_gate_kernel<bf16><<<blocks, 256, 0, st>>>((bf16*)o, x, ld, col, H, E, n);
-  else head_gate_kernel<float><<<blocks, 256, 0, st>>>((float*)o, x, ld, col, H, E, n);
+  if (is_bf16) head_gate_kernel<bf16><<<blocks, 256, 0, st>>>((bf16*)o, x, ld, col, H, E, each, n);
+  else head_gate_kernel<float><<<blocks, 256, 0, st>>>((float*)o, x, ld, col, H, E, each, n);
   return launch_status();
 }
 
@@ -281,7 +282,8 @@ extern "C" int ms_activate(const float* x, void* out, int out_is_bf16, long long
 // w[h][n][k], x [M, ld >= H K] and w [H, N, K] bfloat16, float32 sums (v_mfma_f32_16x16x32_bf16), the result bfloat16 or
 // float32. A block owns 64 rows x 64 columns of one head, a wave 16 of the rows; both operands come straight from
 // memory, 16 bytes a lane (the weights of a head are small and stay in the cache). K a multiple of 8.
-// gate (optional): float32 rows of stride gate_ld; head h's results of row m are multiplied by sigmoid(gate[m][gate_col + h]).
+// gate (optional): float32 rows of stride gate_ld; head h's results of row m are multiplied by sigmoid(gate[m][gate_col + h]), or,
+// gate_each, result n of head h by sigmoid(gate[m][gate_col + h N + n]).
 typedef __attribute__((__vector_size__(8 * sizeof(__bf16)))) __bf16 hg_bf16x8;
 typedef __attribute__((__vector_size__(4 * sizeof(float)))) float hg_floatx4;
 
@@ -294,7 +296,7 @@ __device__ __forceinline__ hg_bf16x8 hg_load(const bf16* p, bool ok) {
 __global__ __launch_bounds__(256) void head_gemm_bf16_kernel(const bf16* __restrict__ x, int ldx, const bf16* __restrict__ w,
                                                              void* __restrict__ out, int ldc, int out_stride, int col0, int M, int N,
                                                              int K, int out_f32, const float* __restrict__ gate, int gate_ld,
-                                                             int gate_col) {
+                                                             int gate_col, int gate_each) {
   const int lane = threadIdx.x % WAVE, wave = threadIdx.x / WAVE, l16 = lane % 16, grp = lane / 16;
   const int h = blockIdx.z, m0 = blockIdx.x * 64 + wave * 16, n0 = blockIdx.y * 64;
   if (m0 >= M) return;
@@ -330,24 +332,27 @@ __global__ __launch_bounds__(256) void head_gemm_bf16_kernel(const bf16* __restr
     const int m = m0 + grp * 4 + r;
     if (m >= M) continue;
     const size_t at = (size_t)m * ldc + (size_t)h * out_stride + col0 + n0 + l16;
-    const float gm = gate ? 1.f / (1.f + expf(-gate[(size_t)m * gate_ld + gate_col + h])) : 1.f;
+    const float* gr = gate ? gate + (size_t)m * gate_ld + gate_col + (gate_each ? (size_t)h * N + n0 + l16 : (size_t)h) : nullptr;
+    const float gm = gate && !gate_each ? 1.f / (1.f + expf(-gr[0])) : 1.f;
 #pragma unroll
     for (int nt = 0; nt < 4; ++nt) {
       if (!col_ok[nt]) continue;
-      if (out_f32) ((float*)out)[at + nt * 16] = acc[nt][r] * gm;
-      else ((bf16*)out)[at + nt * 16] = static_cast<bf16>(acc[nt][r] * gm);
+      const float v = acc[nt][r] * (gate && gate_each ? 1.f / (1.f + expf(-gr[nt * 16])) : gm);
+      if (out_f32) ((float*)out)[at + nt * 16] = v;
+      else ((bf16*)out)[at + nt * 16] = static_cast<bf16>(v);
     }
   }
 }
 
 extern "C" int ms_head_gemm_bf16(const void* x, int ldx, const void* w, void* out, int ldc, int out_stride, int col0, int out_f32,
-                                 int M, int H, int N, int K, const float* gate, int gate_ld, int gate_col, hipStream_t st) {
+                                 int M, int H, int N, int K, const float* gate, int gate_ld, int gate_col, int gate_each,
+                                 hipStream_t st) {
   if (M <= 0 || H <= 0 || N <= 0) return MS_OK;
   if (K <= 0 || ldx < H * K || out_stride < col0 + N || ldc < H * out_stride || col0 < 0 || H > 65535 || (N + 63) / 64 > 65535)
     return MS_BAD_ARG;
-  if (gate && (gate_col < 0 || gate_ld < gate_col + H)) return MS_BAD_ARG;
+  if (gate && (gate_col < 0 || gate_ld < gate_col + (gate_each ? H * N : H))) return MS_BAD_ARG;
   if (K % 8 || ldx % 8 || ((size_t)x % 16) || ((size_t)w % 16)) return MS_UNSUPPORTED;
   head_gemm_bf16_kernel<<<dim3((M + 63) / 64, (N + 63) / 64, H), 256, 0, st>>>((const bf16*)x, ldx, (const bf16*)w, out, ldc, out_stride,
-                                                                             col0, M, N, K, out_f32, gate, gate_ld, gate_col);
+                                                                             col0, M, N, K, out_f32, gate, gate_ld, gate_col, gate_each);
   return launch_status();
 }

@@ -23,11 +23,12 @@ _ERRORS = {1: "bad argument", 2: "unsupported size", 3: "kernel launch failed"}
 _SIGNATURES = {
     "ms_embed": [_c_void, _c_void, _c_int, _c_void, _c_int, _c_int, _c_void],
     "ms_feed_tokens": [_c_void, _c_void, _c_void, _c_void, _c_int, _c_int, _c_void],
-    "ms_rmsnorm": [_c_void, _c_void, _c_int, _c_void, _c_int, _c_void, _c_int, _c_int, _c_float, _c_void, _c_int, _c_ll, _c_void],
+    "ms_rmsnorm": [_c_void, _c_void, _c_int, _c_void, _c_int, _c_void, _c_int, _c_int, _c_float, _c_void, _c_int, _c_ll, _c_void, _c_void],
     "ms_act_mul": [_c_void, _c_void, _c_int, _c_int, _c_int, _c_int, _c_int, _c_float, _c_void],
     "ms_act_mul_parts": [_c_void, _c_int, _c_ll, _c_void, _c_int, _c_int, _c_int, _c_int, _c_int, _c_float, _c_void],
     "ms_layernorm": [_c_void, _c_void, _c_void, _c_int, _c_void, _c_int, _c_void, _c_int, _c_int, _c_float, _c_void],
-    "ms_group_rmsnorm_gate": [_c_void, _c_void, _c_int, _c_void, _c_int, _c_void, _c_int, _c_int, _c_int, _c_int, _c_float, _c_int, _c_void],
+    "ms_group_rmsnorm_gate": [_c_void, _c_void, _c_int, _c_void, _c_int, _c_void, _c_int, _c_int, _c_int, _c_int, _c_float, _c_int, _c_int,
+                              _c_void],
     "ms_normed_mean_add": [_c_void, _c_void, _c_void, _c_int, _c_int, _c_int, _c_int, _c_float, _c_float, _c_void],
     "ms_normed_add_pending": [_c_void, _c_void, _c_void, _c_int, _c_ll, _c_void, _c_int, _c_int, _c_int, _c_float, _c_void, _c_int,
                               _c_void],
@@ -36,7 +37,16 @@ _SIGNATURES = {
                                _c_int, _c_int, _c_void, _c_void, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_void],
     "ms_gated_recurrence": [_c_void, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_float,
                             _c_float, _c_void, _c_void, _c_void, _c_int, _c_void, _c_void, _c_void, _c_void, _c_void, _c_void, _c_void,
-                            _c_int, _c_void, _c_int, _c_void, _c_void],
+                            _c_int, _c_void, _c_int, _c_void, _c_int, _c_void],
+    "ms_time_conv": [_c_void, _c_int, _c_int, _c_int, _c_void, _c_void, _c_void, _c_void, _c_void, _c_void, _c_void, _c_void, _c_void, _c_int,
+                     _c_int, _c_int, _c_void],
+    "ms_ssd_chunked": [_c_void, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_void, _c_int, _c_void, _c_void, _c_void,
+                       _c_void, _c_void, _c_void, _c_void, _c_void, _c_int, _c_int, _c_void, _c_void, _c_void],
+    "ms_ssd_chunk_tokens": [],
+    "ms_ssd_max_dim": [],
+    "ms_rglru": [_c_void, _c_int, _c_int, _c_int, _c_void, _c_void, _c_int, _c_void, _c_void, _c_void, _c_void, _c_void, _c_void, _c_int,
+                 _c_void, _c_void, _c_int, _c_void, _c_void, _c_void, _c_void, _c_int, _c_int, _c_int, _c_void, _c_void],
+    "ms_rglru_chunk_tokens": [],
     "ms_rotate_columns": [_c_void, _c_int, _c_int, _c_int, _c_int, _c_int, _c_void, _c_int, _c_int, _c_float, _c_void],
     "ms_token_shift_mix": [_c_void, _c_void, _c_void, _c_int, _c_void, _c_void, _c_void, _c_void, _c_void, _c_int, _c_int, _c_int, _c_void],
     "ms_neg_exp_bias": [_c_void, _c_void, _c_int, _c_int, _c_int, _c_int, _c_void],
@@ -62,7 +72,7 @@ _SIGNATURES = {
     "ms_gemm_bf16_small": [_c_void, _c_void, _c_void, _c_void, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_void],
     "ms_gemm_bf16_small_splits": [_c_int, _c_int, _c_int],
     "ms_gemm_bf16_small_tile_cols": [_c_int, _c_int],
-    "ms_splitk_reduce": [_c_void, _c_void, _c_int, _c_int, _c_int, _c_int, _c_int, _c_void],
+    "ms_splitk_reduce": [_c_void, _c_void, _c_int, _c_int, _c_int, _c_int, _c_int, _c_void, _c_void],
     "ms_paged_attention_generic": [_c_void, _c_int, _c_void, _c_void, _c_int, _c_void, _c_int, _c_void, _c_void, _c_void,
                                    _c_void, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_float, _c_int, _c_int, _c_int,
                                    _c_float, _c_void, _c_int, _c_int, _c_int, _c_void],
@@ -77,8 +87,8 @@ _SIGNATURES = {
                                            _c_void, _c_int, _c_int, _c_void, _c_void, _c_void],
     "ms_paged_attention_tiled_mfma_wide_chunk": [_c_int, _c_int, _c_int, _c_int, _c_int],
     "ms_head_gemm_bf16": [_c_void, _c_int, _c_void, _c_void, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_void, _c_int,
-                          _c_int, _c_void],
-    "ms_head_gate": [_c_void, _c_int, _c_void, _c_int, _c_int, _c_int, _c_int, _c_int, _c_void],
+                          _c_int, _c_int, _c_void],
+    "ms_head_gate": [_c_void, _c_int, _c_void, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_void],
     "ms_activate": [_c_void, _c_void, _c_int, _c_ll, _c_int, _c_void],
     "ms_paged_attention_tiled": [_c_void, _c_int, _c_void, _c_void, _c_int, _c_void, _c_int, _c_void, _c_void, _c_int, _c_void, _c_void,
                                  _c_void, _c_int, _c_int, _c_int, _c_int, _c_int, _c_float, _c_int, _c_int, _c_void],
@@ -107,11 +117,12 @@ _SIGNATURES = {
                               _c_int, _c_void, _c_int, _c_float, _c_void, _c_void, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int,
                               _c_void],
     "ms_moe_route": [_c_void, _c_int, _c_int, _c_ll, _c_void, _c_int, _c_int, _c_int, _c_int, _c_void, _c_void, _c_void],
-    "ms_moe_route_scored": [_c_void, _c_int, _c_int, _c_ll, _c_void, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_void, _c_void, _c_void],
+    "ms_moe_route_scored": [_c_void, _c_int, _c_int, _c_ll, _c_void, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_void, _c_void,
+                            _c_void],
     "ms_moe_plan": [_c_void, _c_int, _c_int, _c_int, _c_int, _c_void, _c_void, _c_void, _c_void, _c_void],
     "ms_moe_gemm": [_c_void, _c_int, _c_void, _c_void, _c_void, _c_int, _c_int, _c_void, _c_void, _c_void, _c_void, _c_void,
                     _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_void],
-    "ms_moe_combine": [_c_void, _c_void, _c_int, _c_int, _c_int, _c_void, _c_void, _c_void, _c_int, _c_int, _c_int, _c_void],
+    "ms_moe_combine": [_c_void, _c_void, _c_int, _c_int, _c_int, _c_void, _c_void, _c_void, _c_int, _c_int, _c_int, _c_void, _c_void],
     "ms_measure_read": [_c_void, _c_ll, _c_int, _c_void, _c_void],
     "ms_measure_copy": [_c_void, _c_void, _c_ll, _c_int, _c_void],
 }
@@ -200,12 +211,14 @@ class SplitSum:
     """A matrix that exists only as partial sums: its value is ``parts.sum(0)`` (float32
     ``[splits, M, N]``, to be added in ascending split order). The small-M matrix product leaves its
     result in this form so that the kernel that consumes it does the summing and no kernel of its own
-    is spent on it. ``accumulate`` marks a sum that still has to be added to the residual stream."""
+    is spent on it. ``scale`` (float32 ``[N]``, optional): the value is ``parts.sum(0) * scale``, column by column (a sum
+    that is to be added to the residual stream behind a layer scale)."""
 
-    __slots__ = ("parts",)
+    __slots__ = ("parts", "scale")
 
-    def __init__(self, parts: torch.Tensor):
+    def __init__(self, parts: torch.Tensor, scale: torch.Tensor | None = None):
         self.parts = parts
+        self.scale = scale
 
     @property
     def shape(self):
@@ -224,6 +237,16 @@ def _check_split(v: SplitSum, name: str, shape) -> None:
     _dev(v.parts, name, F32, 3)
     if v.shape != tuple(shape):
         raise ValueError(f"{name} holds partial sums of a {v.shape} matrix, expected {tuple(shape)}")
+    if v.scale is not None:
+        _dev(v.scale, f"{name}'s scale", F32, 1)
+        if v.scale.shape[0] != v.parts.shape[2]:
+            raise ValueError(f"{name} has a scale of {v.scale.shape[0]} elements for {v.parts.shape[2]} columns")
+
+
+def _no_scale(v, what: str) -> None:
+    """Refuses a ``SplitSum`` with a scale where the kernel that adds the parts takes none."""
+    if isinstance(v, SplitSum) and v.scale is not None:
+        raise NotImplementedError(f"{what} takes no partial sums that carry a scale")
 
 
 # ------------------------------------------------------------------------------------- elementwise
@@ -273,14 +296,14 @@ def rmsnorm(x: torch.Tensor, weight: torch.Tensor, eps: float, out_dtype, rows: 
     if rows is not None:
         _dev(rows, "rows", I32, 1)
         n = rows.shape[0]
-    parts, splits, stride = None, 0, 0
+    parts, splits, stride, scale = None, 0, 0, None
     if add is not None:
         _check_split(add, "add", x.shape)
-        parts, splits, stride = add.parts.data_ptr(), add.splits, add.stride
+        parts, splits, stride, scale = add.parts.data_ptr(), add.splits, add.stride, _ptr(add.scale)
     out = torch.empty((n, x.shape[1]), dtype=out_dtype, device=x.device)
     _check(library().ms_rmsnorm(x.data_ptr(), weight.data_ptr(), int(weight.dtype == BF16), out.data_ptr(),
                                 int(out_dtype == BF16), _ptr(rows), n, x.shape[1], float(eps), parts, splits, stride,
-                                _stream()), "rmsnorm")
+                                scale, _stream()), "rmsnorm")
     return out
 
 
@@ -327,6 +350,7 @@ def act_mul(gu, activation: str = "silu", out_dtype=None, block: int = 0, limit:
     act = _activation(activation, limit)
     limit = float(limit or 0.0)
     if isinstance(gu, SplitSum):
+        _no_scale(gu, "act_mul")
         _dev(gu.parts, "gu", F32, 3)
         t, width = gu.shape
         if width % 2 or out_dtype not in (F32, BF16) or (block and (width // 2) % block):
@@ -394,7 +418,7 @@ MAX_STEP_TOKENS = 65535  # rows one launch of the matrix and elementwise kernels
 
 
 def linear(x: torch.Tensor, weight: torch.Tensor, out_dtype=None, accumulate_into: torch.Tensor | None = None,
-           defer: bool = False, out: torch.Tensor | None = None):
+           defer: bool = False, out: torch.Tensor | None = None, scale: torch.Tensor | None = None):
     """``x [M, K] @ weight [N, K]^T``. Either returns a new ``[M, N]`` tensor of ``out_dtype``, or adds
     the product into the float32 tensor ``accumulate_into`` (the residual stream) and returns None.
     The weight's dtype picks the arithmetic: float32 weights run the true 32-bit kernel (``x`` is
@@ -406,7 +430,15 @@ def linear(x: torch.Tensor, weight: torch.Tensor, out_dtype=None, accumulate_int
 
     ``out``: a float32 ``[M, N]`` view of a wider matrix (unit column stride, rows a multiple of four floats apart and
     the first element 16-byte aligned) that receives the product; it is returned. Several products then share one
-    matrix whose columns a later kernel reads side by side."""
+    matrix whose columns a later kernel reads side by side.
+
+    ``scale`` (float32 ``[N]``, with ``accumulate_into``): what is added is the product times ``scale``, column by column.
+    The product then always comes as partial sums (one of them, where the kernels leave no more) that carry the scale:
+    the returned ``SplitSum``, or, without ``defer``, added here."""
+    if scale is not None:
+        if accumulate_into is None:
+            raise ValueError("linear: a scale goes with accumulate_into")
+        return _linear_scaled(x, weight, accumulate_into, scale, defer)
     _dev(x, "x", (F32, BF16), 2)
     _dev(weight, "weight", (F32, BF16), 2)
     m, k = x.shape
@@ -473,6 +505,19 @@ def linear(x: torch.Tensor, weight: torch.Tensor, out_dtype=None, accumulate_int
     return None if accumulate_into is not None else res
 
 
+def _linear_scaled(x, weight, residual, scale, defer: bool) -> SplitSum | None:
+    m, n = x.shape[0], weight.shape[0]
+    _dev(residual, "accumulate_into", F32, 2)
+    if tuple(residual.shape) != (m, n):
+        raise ValueError(f"linear: accumulator is {tuple(residual.shape)}, expected {(m, n)}")
+    res = linear(x, weight, out_dtype=F32, defer=True)
+    pending = SplitSum(res.parts if isinstance(res, SplitSum) else res.view(1, m, n), scale)
+    if defer:
+        return pending
+    add_pending(residual, pending)
+    return None
+
+
 def tile_shape(m: int, n: int, k: int, splits: int = 1, gated: bool = False) -> tuple[int, int] | None:
     """``(rows, columns)`` of the tile that ``linear`` (or, with ``gated``, ``gated_linear`` with ``n = 2 I``)
     runs a bfloat16 product of more than ``SMALL_M`` contiguous rows with; None where the shape takes the
@@ -482,20 +527,21 @@ def tile_shape(m: int, n: int, k: int, splits: int = 1, gated: bool = False) -> 
 
 
 def add_pending(residual: torch.Tensor, pending: SplitSum | None) -> None:
-    """``residual += pending`` for callers whose next kernel cannot take a pending sum itself."""
+    """``residual += pending`` (its scale applied) for callers whose next kernel cannot take a pending sum itself."""
     if pending is None:
         return
     _dev(residual, "residual", F32, 2)
     _check_split(pending, "pending", residual.shape)
     m, n = residual.shape
-    _check(library().ms_splitk_reduce(pending.parts.data_ptr(), residual.data_ptr(), 2, pending.splits, m, n, n, _stream()),
-           "splitk_reduce")
+    _check(library().ms_splitk_reduce(pending.parts.data_ptr(), residual.data_ptr(), 2, pending.splits, m, n, n, _ptr(pending.scale),
+                                      _stream()), "splitk_reduce")
 
 
 # ------------------------------------------------------------------------------------- mixture of experts
 
 MOE_MAX_EXPERTS = 512  # MOE_MAX_EXPERTS in csrc/moe.hip
 MOE_MAX_TOP = 64
+MOE_SCORINGS = ("chosen_softmax", "softmax", "sigmoid")
 MOE_SMALL_TILE_PAIRS = 16  # (token, expert) pairs per expert, on average, up to which a step runs 16-pair tiles
 MOE_LARGE_TILE_PAIRS = 128  # ... and from which it runs 128-pair tiles (widths that are multiples of 64)
 
@@ -509,8 +555,9 @@ def moe_route(logits, bias: torch.Tensor | None, top: int, scoring: str = "chose
     alone. ``scoring="softmax"``: ``s = softmax(logits)`` over all ``E`` outputs; the choice goes by ``s + bias`` (a
     correction that only the choice sees), the weights are the chosen outputs' ``s`` as they stand; with ``groups > 1``
     the outputs form that many equal groups of neighbours, a group's score is the largest ``s + bias`` in it, and only
-    outputs of the ``keep`` best groups can be chosen."""
+    outputs of the ``keep`` best groups can be chosen. ``scoring="sigmoid"``: the same with ``s = sigmoid(logits)``."""
     if isinstance(logits, SplitSum):
+        _no_scale(logits, "the routing")
         parts, splits, stride = logits.parts, logits.splits, logits.stride
         _dev(parts, "logits", F32, 3)
         t, e = logits.shape
@@ -522,33 +569,36 @@ def moe_route(logits, bias: torch.Tensor | None, top: int, scoring: str = "chose
         raise ValueError(f"top {top} of {e} experts")
     if e > MOE_MAX_EXPERTS or top > MOE_MAX_TOP:
         raise ValueError(f"{e} experts / top {top}: the routing kernel takes up to {MOE_MAX_EXPERTS} experts and {MOE_MAX_TOP} choices")
-    if scoring not in ("chosen_softmax", "softmax"):
-        raise NotImplementedError(f"router scoring {scoring!r}: 'chosen_softmax' or 'softmax'")
+    if scoring not in MOE_SCORINGS:
+        raise NotImplementedError(f"router scoring {scoring!r}: one of {MOE_SCORINGS}")
     if bias is not None:
         _dev(bias, "bias", (F32, BF16), 1)
         if bias.shape[0] != e:
             raise ValueError(f"the router's bias has {bias.shape[0]} elements for {e} experts")
     ids = torch.empty((t, top), dtype=I32, device=parts.device)
     weights = torch.empty((t, top), dtype=F32, device=parts.device)
-    if scoring == "softmax":
+    if scoring != "chosen_softmax":
         if groups < 1 or e % groups or not 1 <= keep <= groups:
             raise ValueError(f"{e} router outputs in {groups} groups of which {keep} are kept")
         if top > (e // groups) * keep:
             raise ValueError(f"top {top} of the {(e // groups) * keep} outputs in the kept groups")
         _check(library().ms_moe_route_scored(parts.data_ptr(), e, splits, stride, _ptr(bias), int(bias is not None and bias.dtype == BF16),
-                                             t, e, top, int(groups), int(keep), ids.data_ptr(), weights.data_ptr(), _stream()),
+                                             t, e, top, int(groups), int(keep), int(scoring == "sigmoid"), ids.data_ptr(), weights.data_ptr(), _stream()),
                "moe_route_scored")
         return ids, weights
     if groups != 1:
-        raise NotImplementedError("groups of experts go with scoring='softmax'")
+        raise NotImplementedError("groups of experts go with scores over all outputs")
     _check(library().ms_moe_route(parts.data_ptr(), e, splits, stride, _ptr(bias), int(bias is not None and bias.dtype == BF16), t, e,
                                   top, ids.data_ptr(), weights.data_ptr(), _stream()), "moe_route")
     return ids, weights
 
 
 def moe_experts(x: torch.Tensor, ids: torch.Tensor, weights: torch.Tensor, gate: torch.Tensor | None, up: torch.Tensor,
-                down: torch.Tensor, activation: str, stream: torch.Tensor) -> None:
-    """``stream[t] += sum_j weights[t, j] * expert_e(x[t])`` with ``e = ids[t, j]``, the sum in ascending ``j``. A gated
+                down: torch.Tensor, activation: str, stream: torch.Tensor, weigh_input: bool = False,
+                scale: torch.Tensor | None = None) -> None:
+    """``stream[t] += sum_j weights[t, j] * expert_e(x[t])`` with ``e = ids[t, j]``, the sum in ascending ``j``; with
+    ``weigh_input`` ``stream[t] += sum_j expert_e(weights[t, j] * x[t])`` (the weight multiplies the first products' float32
+    results, which is the same); ``scale`` (float32 ``[W]``) multiplies the sum element by element. A gated
     expert is ``down[e] (act(gate[e] x) * (up[e] x))``; with ``gate=None`` it is ``down[e] act(up[e] x)``. An id of
     ``E`` (the number of experts that have weights) or more names an identity expert: its term is ``weights[t, j] * x[t]``.
     ``x [T, W]`` in the compute dtype, ``gate`` / ``up`` ``[E, F, W]`` and ``down [E, W, F]`` in the same, ``stream`` float32
@@ -573,6 +623,10 @@ def moe_experts(x: torch.Tensor, ids: torch.Tensor, weights: torch.Tensor, gate:
         raise ValueError(f"expert weights {tuple(up.shape)} / {tuple(down.shape)} do not fit x {tuple(x.shape)}")
     if ids.shape[0] != t or tuple(weights.shape) != tuple(ids.shape) or tuple(stream.shape) != (t, width):
         raise ValueError("ids, weights and stream must have one row per row of x")
+    if scale is not None:
+        _dev(scale, "scale", F32, 1)
+        if scale.shape[0] != width:
+            raise ValueError(f"a scale of {scale.shape[0]} elements for width {width}")
     if e > MOE_MAX_EXPERTS:
         raise ValueError(f"{e} experts: the kernels take up to {MOE_MAX_EXPERTS}")
     if t == 0:
@@ -595,12 +649,12 @@ def moe_experts(x: torch.Tensor, ids: torch.Tensor, weights: torch.Tensor, gate:
     plan = (order.data_ptr(), tiles[0].data_ptr(), tiles[1].data_ptr(), tiles[2].data_ptr())
     h = torch.empty((pairs, f), dtype=x.dtype, device=dev)
     _check(lib.ms_moe_gemm(x.data_ptr(), width, (gate if gated else up).data_ptr(), up.data_ptr() if gated else None, h.data_ptr(), int(bf),
-                           1 if gated else 2, *plan, None, max_tiles, top, f, width, tile_rows, act, _stream()), "moe_gemm")
+                           1 if gated else 2, *plan, weights.data_ptr() if weigh_input else None, max_tiles, top, f, width, tile_rows, act, _stream()), "moe_gemm")
     y = torch.empty((pairs, width), dtype=F32, device=dev)
-    _check(lib.ms_moe_gemm(h.data_ptr(), f, down.data_ptr(), None, y.data_ptr(), int(bf), 0, *plan, weights.data_ptr(), max_tiles, top,
+    _check(lib.ms_moe_gemm(h.data_ptr(), f, down.data_ptr(), None, y.data_ptr(), int(bf), 0, *plan, None if weigh_input else weights.data_ptr(), max_tiles, top,
                            width, f, tile_rows, act, _stream()), "moe_gemm")
     _check(lib.ms_moe_combine(stream.data_ptr(), y.data_ptr(), t, top, width, ids.data_ptr(), weights.data_ptr(), x.data_ptr(), int(bf),
-                              width, e, _stream()), "moe_combine")
+                              width, e, _ptr(scale), _stream()), "moe_combine")
 
 
 # ------------------------------------------------------------------------------------- attention
@@ -773,6 +827,7 @@ def decode_attention_fused(qkv, q_weight, k_weight, eps, rope, store, k_cache, v
     output never goes to memory."""
     if not decode_attention_fusable(qkv, batch, q_weight, k_weight, rope, k_cache, v_cache, num_heads, num_kv_heads, head_dim):
         raise ValueError("this step cannot run the fused decode attention")
+    _no_scale(qkv, "the fused decode attention")
     _dev(qkv.parts, "qkv", F32, 3)
     t = qkv.shape[0]
     if qkv.shape[1] != (num_heads + 2 * num_kv_heads) * head_dim:
@@ -827,7 +882,7 @@ def decode_attention_fused(qkv, q_weight, k_weight, eps, rope, store, k_cache, v
 def paged_attention(qkv, k_cache, v_cache, block_table, batch, num_heads, num_kv_heads, head_dim, scale, window,
                     value_dim: int | None = None, keep_first: int = 0, exact_weights: bool = False, softcap: float = 0.0,
                     sinks: torch.Tensor | None = None, value_share: int = 1, values_in_keys: bool = False,
-                    out_dtype=None):
+                    out_dtype=None, wide_heads: bool = False):
     """Attention of the batch's new tokens over the cache. ``qkv [T, >= Hq D]`` holds the queries
     in its first ``Hq * D`` columns. Returns ``[T, Hq * Dv]`` (``Dv = D`` unless ``value_dim`` is given).
     A query at position p sees keys ``max(0, p - window + 1) .. p`` (``window == 0``: all up to p) and, with a
@@ -846,14 +901,15 @@ def paged_attention(qkv, k_cache, v_cache, block_table, batch, num_heads, num_kv
     ``exp(sinks[h])`` to head ``h``'s softmax denominator; ``value_share = n`` lets ``n`` consecutive key heads weigh
     the same value head (``v_cache`` then has ``Hkv / n`` heads); ``values_in_keys`` takes the first ``Dv`` elements
     of each key row as that token's value (``v_cache`` is None); ``out_dtype=torch.float32`` returns the result
-    unrounded whatever the cache's dtype."""
+    unrounded whatever the cache's dtype. ``wide_heads`` asks for these kernels where none of the options does (heads of
+    more than 256 elements, softmax weights unrounded)."""
     _dev(qkv, "qkv", (F32, BF16), 2)
     t = qkv.shape[0]
     dv = head_dim if value_dim is None else int(value_dim)
     out_f32 = out_dtype == F32 and qkv.dtype != F32
     if out_dtype not in (None, F32, qkv.dtype):
         raise TypeError(f"the result comes in the queries' dtype or in float32, not {out_dtype}")
-    special = bool(softcap) or sinks is not None or value_share != 1 or values_in_keys or out_f32
+    special = wide_heads or bool(softcap) or sinks is not None or value_share != 1 or values_in_keys or out_f32
     if special:
         page = _check_special_caches(k_cache, v_cache, qkv.dtype, num_kv_heads, head_dim, dv, value_share, values_in_keys)
         if sinks is not None:
@@ -1157,10 +1213,13 @@ GATE_ACTIVATIONS = {"sigmoid": 0, "silu": 1}  # what a gate goes through before 
 
 
 def group_rmsnorm_gate(x: torch.Tensor, group: int, weight: torch.Tensor | None, gate: torch.Tensor | None, eps: float,
-                       out_dtype, gate_activation: str = "sigmoid") -> torch.Tensor:
+                       out_dtype, gate_activation: str = "sigmoid", gate_first: bool = False) -> torch.Tensor:
     """``x / rms(group of x) * weight * act(gate)`` for float32 ``x [T, N]`` cut into groups of ``group``
     consecutive elements (``group == N``: one norm over the row). ``weight [N]`` and ``gate`` (float32 ``[T, N]``,
-    may be a column slice of a wider matrix) are optional; ``gate_activation``: ``"sigmoid"`` or ``"silu"``."""
+    may be a column slice of a wider matrix) are optional; ``gate_activation``: ``"sigmoid"`` or ``"silu"``. ``gate_first``: the
+    gate multiplies ``x`` in front of the norm instead, ``(x act(gate)) / rms(group of x act(gate)) * weight``."""
+    if gate_first and gate is None:
+        raise ValueError("gate_first without a gate")
     if gate_activation not in GATE_ACTIVATIONS:
         raise NotImplementedError(f"gate activation {gate_activation!r}: the kernel knows {sorted(GATE_ACTIVATIONS)}")
     _dev(x, "x", F32, 2)
@@ -1181,7 +1240,7 @@ def group_rmsnorm_gate(x: torch.Tensor, group: int, weight: torch.Tensor | None,
     out = torch.empty((t, n), dtype=out_dtype, device=x.device)
     _check(library().ms_group_rmsnorm_gate(x.data_ptr(), _ptr(weight), int(weight is not None and weight.dtype == BF16), _ptr(gate),
                                            gate_stride, out.data_ptr(), int(out_dtype == BF16), t, n // group, group, float(eps),
-                                           GATE_ACTIVATIONS[gate_activation], _stream()), "group_rmsnorm_gate")
+                                           GATE_ACTIVATIONS[gate_activation], int(gate_first), _stream()), "group_rmsnorm_gate")
     return out
 
 
@@ -1212,6 +1271,7 @@ def normed_add(residual: torch.Tensor, stream: torch.Tensor | None, weight: torc
     16 bits; with ``clear`` the stream is left zero."""
     if pending is None and stream is None:
         raise ValueError("neither a stream nor a pending sum")
+    _no_scale(pending, "the norm of a sublayer's output")
     if pending is None and next_out is None and not clear:
         return normed_mean_add(residual, [stream], [weight], eps, 1.0)
     _dev(residual, "residual", F32, 2)
@@ -1476,14 +1536,15 @@ def latent_prepare(x, q_col: int, kv_col: int | None, rope, rot: int, pairing: s
     return q_plain, q_full
 
 
-def head_gate_(o: torch.Tensor, x: torch.Tensor, col: int, heads: int) -> torch.Tensor:
-    """``o[t, h, :] *= sigmoid(x[t, col + h])`` in place: ``o [T, heads * E]``, ``x`` float32."""
+def head_gate_(o: torch.Tensor, x: torch.Tensor, col: int, heads: int, each: bool = False) -> torch.Tensor:
+    """``o[t, h, :] *= sigmoid(x[t, col + h])`` in place: ``o [T, heads * E]``, ``x`` float32. ``each``: a gate per element,
+    ``o[t, i] *= sigmoid(x[t, col + i])``."""
     _dev(o, "o", (F32, BF16), 2)
     _dev(x, "x", F32, 2)
-    if o.shape[0] != x.shape[0] or o.shape[1] % heads or x.shape[1] < col + heads:
-        raise ValueError("o and x must have the same rows, and x one gate column per head")
+    if o.shape[0] != x.shape[0] or o.shape[1] % heads or x.shape[1] < col + (o.shape[1] if each else heads):
+        raise ValueError("o and x must have the same rows, and x one gate column per head (or per element)")
     _check(library().ms_head_gate(o.data_ptr(), int(o.dtype == BF16), x.data_ptr(), x.shape[1], int(col), o.shape[0], heads,
-                                  o.shape[1] // heads, _stream()), "head_gate")
+                                  o.shape[1] // heads, int(each), _stream()), "head_gate")
     return o
 
 
@@ -1500,14 +1561,16 @@ def activate(x: torch.Tensor, activation: str, out_dtype) -> torch.Tensor:
     return out
 
 
-def head_linear(x: torch.Tensor, weights: torch.Tensor, out: torch.Tensor, out_col: int = 0, gate=None) -> torch.Tensor:
+def head_linear(x: torch.Tensor, weights: torch.Tensor, out: torch.Tensor, out_col: int = 0, gate=None,
+                gate_each: bool = False) -> torch.Tensor:
     """A matrix product per head: ``out[:, h * stride + out_col : ... + N] = x[:, h * K : (h + 1) * K] @ weights[h]^T`` with
     ``x [M, H K]``, ``weights [H, N, K]`` and ``out [M, H stride]`` (``stride = out.shape[1] / H >= out_col + N``; the other
     columns of ``out`` stay). bfloat16 weights with ``K`` a multiple of 8: one launch of a matrix-core kernel for all
     heads. float32 weights: the true 32-bit product, one launch per head over strided rows. Other sizes: head by head
     through contiguous copies. ``gate = (g, col)``: head ``h``'s results of row ``m`` are multiplied by
     ``sigmoid(g[m, col + h])`` (``g`` float32; ``out_col`` 0 and ``N`` the head's whole stride): in the matrix-core
-    kernel's epilogue, else by ``head_gate_`` behind the products."""
+    kernel's epilogue, else by ``head_gate_`` behind the products. ``gate_each``: result ``i`` of the row by
+    ``sigmoid(g[m, col + i])`` instead."""
     _dev(x, "x", (F32, BF16), 2)
     _dev(weights, "weights", (F32, BF16), 3)
     _dev(out, "out", (F32, BF16), 2)
@@ -1522,11 +1585,11 @@ def head_linear(x: torch.Tensor, weights: torch.Tensor, out: torch.Tensor, out_c
     if gate is not None:
         g, g_col = gate
         _dev(g, "gate", F32, 2)
-        if g.shape[0] != m or g.shape[1] < g_col + h or out_col != 0 or stride != n:
-            raise ValueError("a gate needs one float32 column per head and products that fill their heads' columns")
+        if g.shape[0] != m or g.shape[1] < g_col + (h * n if gate_each else h) or out_col != 0 or stride != n:
+            raise ValueError("a gate needs one float32 column per head (or element) and products that fill their heads' columns")
         if not (weights.dtype == BF16 and k % 8 == 0):
             head_linear(x, weights, out, out_col)
-            return head_gate_(out, g, g_col, h)
+            return head_gate_(out, g, g_col, h, gate_each)
     if weights.dtype == F32:
         xa = cast(x, F32)
         for i in range(h):
@@ -1538,8 +1601,8 @@ def head_linear(x: torch.Tensor, weights: torch.Tensor, out: torch.Tensor, out_c
     if k % 8 == 0:
         _check(lib.ms_head_gemm_bf16(xa.data_ptr(), h * k, weights.data_ptr(), out.data_ptr(), out.shape[1], stride, int(out_col),
                                      int(out.dtype == F32), m, h, n, k, gate[0].data_ptr() if gate is not None else None,
-                                     gate[0].shape[1] if gate is not None else 0, int(gate[1]) if gate is not None else 0, _stream()),
-               "head_gemm_bf16")
+                                     gate[0].shape[1] if gate is not None else 0, int(gate[1]) if gate is not None else 0,
+                                     int(gate_each), _stream()), "head_gemm_bf16")
         return out
     for i in range(h):
         y = linear(xa[:, i * k : (i + 1) * k].contiguous(), weights[i], out_dtype=out.dtype)
@@ -1551,10 +1614,13 @@ def head_linear(x: torch.Tensor, weights: torch.Tensor, out: torch.Tensor, out_c
 
 DECODE_GENERIC_WAVES = 16  # waves that share a (token, head) in the float32 attention of single-token rows (8 or 16)
 
-RECURRENCE_MODES = {"decay": 0, "exp_gates": 1, "wkv": 2}
+RECURRENCE_MODES = {"decay": 0, "exp_gates": 1, "wkv": 2}  # of ``gated_recurrence``
+RECURRENCE_STEP_MODE = 3  # ``step_recurrence``
 RECURRENCE_MAX_DIM = 256
 RECURRENCE_CHUNKED_FROM = 16  # tokens of the longest row from which a step runs the chunked kernels
 WKV_CHUNKED_FROM = 16  # ... and from which the recurrence with a decay per channel does
+SSD_CHUNKED_FROM = 16  # ... the one with a step size
+RGLRU_CHUNKED_FROM = 16  # ... and the one per channel
 
 
 def gated_recurrence(x: torch.Tensor, columns: dict, heads: int, dim: int, value_dim: int, batch, state: dict, *,
@@ -1678,7 +1744,156 @@ def gated_recurrence(x: torch.Tensor, columns: dict, heads: int, dim: int, value
         int(activation == "silu"), RECURRENCE_MODES[mode], float(q_scale), float(cap), _ptr(decay), _ptr(i_bias), _ptr(f_bias),
         int(bias is not None and bias.dtype == BF16), S.data_ptr(), _ptr(n), _ptr(m), batch.row_start.data_ptr(),
         batch.starts.data_ptr(), batch.state_slots.data_ptr(), out.data_ptr(), rows, _ptr(channel_decay), heads * dim, _ptr(bonus),
-        _stream()), "gated_recurrence")
+        1, _stream()), "gated_recurrence")
+    return out
+
+
+def _check_rows(batch, t: int) -> None:
+    """The rows of a step as the kernels over time read them: one row of the input per token."""
+    for name in ("token_row", "row_start", "starts", "state_slots"):
+        _dev(getattr(batch, name), name, I32, 1)
+    rows = batch.num_rows
+    if (batch.num_tokens != t or batch.token_row.shape[0] != t or batch.row_start.shape[0] < rows + 1 or batch.starts.shape[0] < rows
+            or batch.state_slots.shape[0] < rows):
+        raise ValueError("batch metadata does not match the number of tokens or rows")
+
+
+def time_conv(x: torch.Tensor, col: int, weight: torch.Tensor, bias: torch.Tensor | None, state: torch.Tensor | None, batch,
+              activation: str | None = None, in_bias: torch.Tensor | None = None) -> torch.Tensor:
+    """A short causal convolution over time on the ``C`` columns of the float32 ``x [T, ld]`` from ``col`` on:
+    ``act(bias[c] + sum_j weight[j, c] u_(t - taps + 1 + j)[c])`` with ``u = x[:, col:] + in_bias``, zero before a sequence's
+    start; float32 ``[T, C]``. ``weight`` is float32 ``[taps, C]`` (one row per tap, the current token's last), ``bias`` and
+    ``in_bias`` float32 ``[C]`` or None, ``activation`` None or ``"silu"``. ``state`` (float32 ``[slots, taps - 1, C]``; None with one
+    tap) holds each request's last ``taps - 1`` inputs ``u`` and is brought up to date; a request that starts at position 0
+    reads nothing of it."""
+    _dev(x, "x", F32, 2)
+    _dev(weight, "weight", F32, 2)
+    t, ld = x.shape
+    taps, c = weight.shape
+    if activation not in (None, "silu"):
+        raise NotImplementedError(f"activation {activation!r} behind a convolution: None or 'silu'")
+    if col < 0 or col + c > ld:
+        raise ValueError(f"columns {col} .. {col + c} lie outside the matrix of width {ld}")
+    for v, nm in ((bias, "bias"), (in_bias, "in_bias")):
+        if v is not None:
+            _dev(v, nm, F32, 1)
+            if v.shape[0] != c:
+                raise ValueError(f"{nm} has {v.shape[0]} elements for {c} channels")
+    if taps > 1:
+        _dev(state, "state", F32, 3)
+        if tuple(state.shape[1:]) != (taps - 1, c):
+            raise ValueError(f"state is {tuple(state.shape)}, expected [slots, {taps - 1}, {c}]")
+    _check_rows(batch, t)
+    out = torch.empty((t, c), dtype=F32, device=x.device)
+    _check(library().ms_time_conv(x.data_ptr() + 4 * col, ld, c, taps, weight.data_ptr(), _ptr(bias), _ptr(in_bias), out.data_ptr(),
+                                  _ptr(state) if taps > 1 else None, batch.state_slots.data_ptr(), batch.token_row.data_ptr(),
+                                  batch.row_start.data_ptr(), batch.starts.data_ptr(), t, batch.num_rows, int(activation == "silu"),
+                                  _stream()), "time_conv")
+    return out
+
+
+def step_recurrence(x: torch.Tensor, columns: dict, heads: int, dim: int, value_dim: int, groups: int, steps: torch.Tensor,
+                    step_col: int, step_bias: torch.Tensor | None, decay: torch.Tensor, skip: torch.Tensor, batch,
+                    S: torch.Tensor) -> torch.Tensor:
+    """A linear recurrence over a matrix state per (request, head) whose decay and input weight both come from one step size:
+    ``d = softplus(steps[t, step_col + h] + step_bias[h])``, ``S_t = exp(decay[h] d) S_(t-1) + d k_t v_t^T``,
+    ``o_t = S_t^T q_t + skip[h] v_t``; float32 ``[T, heads * value_dim]``.
+
+    ``x``: float32 ``[T, ld]`` whose columns hold ``q`` and ``k`` (``groups * dim`` wide each; head ``h`` reads group
+    ``h // (heads / groups)``) and ``v`` (``heads * value_dim``), from ``columns`` on. ``steps``: float32 ``[T, >= step_col + heads]``.
+    ``step_bias``, ``decay`` (negative) and ``skip``: float32 ``[heads]``. ``S``: float32 ``[slots, heads, dim, value_dim]``; rows with
+    ``starts == 0`` begin from zero. Steps whose longest row has ``SSD_CHUNKED_FROM`` tokens or more run in chunks of 64 tokens
+    (matrix products in true float32), others token by token; they differ by the order of float32 sums only."""
+    _dev(x, "x", F32, 2)
+    _dev(steps, "steps", F32, 2)
+    _dev(S, "S", F32, 4)
+    t, ld = x.shape
+    if max(dim, value_dim) > RECURRENCE_MAX_DIM or min(dim, value_dim, heads, groups) < 1 or heads % groups:
+        raise ValueError(f"{heads} heads in {groups} groups, sizes {dim} / {value_dim}: the recurrence kernels take sizes 1..{RECURRENCE_MAX_DIM}")
+    if tuple(S.shape[1:]) != (heads, dim, value_dim):
+        raise ValueError(f"state S is {tuple(S.shape)}, expected [slots, {heads}, {dim}, {value_dim}]")
+    for name, w in (("q", groups * dim), ("k", groups * dim), ("v", heads * value_dim)):
+        if columns[name] < 0 or columns[name] + w > ld:
+            raise ValueError(f"columns of {name!r} ({columns[name]} .. {columns[name] + w}) lie outside the matrix of width {ld}")
+    if steps.shape[0] != t or step_col < 0 or step_col + heads > steps.shape[1]:
+        raise ValueError(f"steps is {tuple(steps.shape)}: {t} rows and {heads} columns from {step_col} on are needed")
+    for v, nm in ((step_bias, "step_bias"), (decay, "decay"), (skip, "skip")):
+        if v is not None:
+            _dev(v, nm, F32, 1)
+            if v.shape[0] != heads:
+                raise ValueError(f"{nm} has {v.shape[0]} elements for {heads} heads")
+    _check_rows(batch, t)
+    out = torch.empty((t, heads * value_dim), dtype=F32, device=x.device)
+    lib = library()
+    lens = getattr(batch, "row_lens", None)
+    share = heads // groups
+    d = steps.data_ptr() + 4 * step_col
+    if lens is not None and max(lens) >= SSD_CHUNKED_FROM and max(dim, value_dim) <= lib.ms_ssd_max_dim():
+        per = lib.ms_ssd_chunk_tokens()
+        chunks = sum(-(-n // per) for n in lens)
+        U = torch.empty((chunks, heads, dim * value_dim), dtype=F32, device=x.device)
+        total = torch.empty((chunks, heads), dtype=F32, device=x.device)
+        _check(lib.ms_ssd_chunked(x.data_ptr(), ld, columns["q"], columns["k"], columns["v"], heads, dim, value_dim, share, d, steps.shape[1],
+                                  _ptr(step_bias), decay.data_ptr(), skip.data_ptr(), S.data_ptr(), batch.row_start.data_ptr(),
+                                  batch.starts.data_ptr(), batch.state_slots.data_ptr(), out.data_ptr(), batch.num_rows, chunks,
+                                  U.data_ptr(), total.data_ptr(), _stream()), "ssd_chunked")
+        return out
+    _check(lib.ms_gated_recurrence(
+        x.data_ptr(), ld, columns["q"], columns["k"], columns["v"], 0, 0, heads, dim, value_dim, 0, RECURRENCE_STEP_MODE, 1.0, 0.0,
+        decay.data_ptr(), _ptr(step_bias), None, 0, S.data_ptr(), None, None, batch.row_start.data_ptr(), batch.starts.data_ptr(),
+        batch.state_slots.data_ptr(), out.data_ptr(), batch.num_rows, d, steps.shape[1], skip.data_ptr(), share, _stream()),
+        "gated_recurrence")
+    return out
+
+
+def rglru(u: torch.Tensor, blocks: int, r_weight: torch.Tensor, i_weight: torch.Tensor, r_bias: torch.Tensor, i_bias: torch.Tensor,
+          coef: torch.Tensor, y: torch.Tensor, y_col: int, y_bias: torch.Tensor, batch, S: torch.Tensor, out_dtype) -> torch.Tensor:
+    """A gated linear recurrence per channel over the float32 ``u [T, W]``, times a GELU of another branch: in each of ``blocks``
+    equal parts ``r = sigmoid(r_weight u + r_bias)`` and ``i = sigmoid(i_weight u + i_bias)`` (weights ``[blocks, W / blocks,
+    W / blocks]``, out by in), ``a = exp(coef r)``, ``S_t = a S_(t-1) + sqrt(1 - a^2) i u``, result
+    ``S_t gelu_tanh(y[t, y_col + c] + y_bias[c])`` in ``out_dtype``, ``[T, W]``. Everything up to the store is float32, the products
+    with bfloat16 weights included (``u`` meets them in three pieces). Biases and ``coef`` (at most zero) are float32 ``[W]``,
+    ``y`` float32 ``[T, >= y_col + W]``; ``S``: float32 ``[slots, W]``; rows with ``starts == 0`` begin from zero. A step of single
+    tokens is one kernel; steps whose longest row has ``RGLRU_CHUNKED_FROM`` tokens or more run the recurrence in chunks."""
+    _dev(u, "u", F32, 2)
+    _dev(y, "y", F32, 2)
+    _dev(S, "S", F32, 2)
+    t, w = u.shape
+    if blocks < 1 or w % blocks:
+        raise ValueError(f"{w} channels cannot be cut into {blocks} equal blocks")
+    bs = w // blocks
+    for v, nm in ((r_weight, "r_weight"), (i_weight, "i_weight")):
+        _dev(v, nm, (F32, BF16), 3)
+        if tuple(v.shape) != (blocks, bs, bs):
+            raise ValueError(f"{nm} is {tuple(v.shape)}, expected {(blocks, bs, bs)}")
+    if r_weight.dtype != i_weight.dtype:
+        raise TypeError("the gates' weights differ in dtype")
+    for v, nm in ((r_bias, "r_bias"), (i_bias, "i_bias"), (coef, "coef"), (y_bias, "y_bias")):
+        _dev(v, nm, F32, 1)
+        if v.shape[0] != w:
+            raise ValueError(f"{nm} has {v.shape[0]} elements for {w} channels")
+    if y.shape[0] != t or y_col < 0 or y_col + w > y.shape[1] or S.shape[1] != w or out_dtype not in (F32, BF16):
+        raise ValueError(f"y {tuple(y.shape)} from column {y_col}, S {tuple(S.shape)} or out_dtype {out_dtype} do not fit {t} tokens of {w} channels")
+    _check_rows(batch, t)
+    lib = library()
+    lens = getattr(batch, "row_lens", None)
+    out = torch.empty((t, w), dtype=out_dtype, device=u.device)
+    a = x = total = None
+    chunks = 0
+    if batch.is_decode and batch.num_rows == t:
+        form = 0
+    else:
+        a, x = (torch.empty((t, w), dtype=F32, device=u.device) for _ in range(2))
+        form = 1
+        if lens is not None and max(lens) >= RGLRU_CHUNKED_FROM:
+            form = 2
+            per = lib.ms_rglru_chunk_tokens()
+            chunks = sum(-(-n // per) for n in lens)
+            total = torch.empty((chunks, 2, w), dtype=F32, device=u.device)
+    _check(lib.ms_rglru(u.data_ptr(), t, w, blocks, r_weight.data_ptr(), i_weight.data_ptr(), int(r_weight.dtype == BF16), r_bias.data_ptr(),
+                        i_bias.data_ptr(), coef.data_ptr(), _ptr(a), _ptr(x), y.data_ptr() + 4 * y_col, y.shape[1], y_bias.data_ptr(),
+                        out.data_ptr(), int(out_dtype == BF16), S.data_ptr(), batch.row_start.data_ptr(), batch.starts.data_ptr(),
+                        batch.state_slots.data_ptr(), batch.num_rows, form, chunks, _ptr(total), _stream()), "rglru")
     return out
 
 

@@ -57,6 +57,8 @@ def _names(spec: PartSpec) -> dict[str, str]:
 
 @register("mixer", "gqa_attention")
 class GQAttention(Mixer):
+    scales_output = True
+
     def __init__(self, spec: PartSpec, rt):
         super().__init__(spec, rt)
         self.prefix = spec.get("prefix", "")
@@ -197,7 +199,7 @@ class GQAttention(Mixer):
                                       self.scale, self.window, self.value_dim, self.keep_first, self.exact_weights)
             if self.head_gate:
                 ops.head_gate_(out, qkv, self.gate_col, self.heads)
-            return ops.linear(out, self.o, accumulate_into=residual, defer=True)
+            return ops.linear(out, self.o, accumulate_into=residual, defer=True, scale=self.out_scale)
         qkv = ops.linear(x, self.qkv, out_dtype=self.rt.dtype, defer=True)
         if not (self.exact_weights or self.keep_first) and ops.decode_attention_fusable(qkv, batch, self.q_norm, self.k_norm, table, cache.k, cache.v,
                                         self.heads, self.kv_heads, self.head_dim, pairing):
@@ -209,8 +211,9 @@ class GQAttention(Mixer):
                 self.scale, self.window, project=self.o if self.o.dtype == torch.bfloat16 else None,
             )
             if isinstance(out, ops.SplitSum):
+                out.scale = self.out_scale
                 return out  # the projection's partial sums: pending, for the next reader of the stream
-            return ops.linear(out, self.o, accumulate_into=residual, defer=True)
+            return ops.linear(out, self.o, accumulate_into=residual, defer=True, scale=self.out_scale)
         q = ops.qk_norm_rope_store(
             qkv, cache.slots if cache.writes else None,
             self.q_norm, self.k_norm, 0.0 if self.qk_norm_eps is None else float(self.qk_norm_eps),
@@ -221,7 +224,7 @@ class GQAttention(Mixer):
             q, cache.k, cache.v, cache.block_table, batch, self.heads, self.kv_heads, self.head_dim,
             self.scale, self.window, None, self.keep_first, self.exact_weights,
         )
-        return ops.linear(out, self.o, accumulate_into=residual, defer=True)
+        return ops.linear(out, self.o, accumulate_into=residual, defer=True, scale=self.out_scale)
 
     def _forward_prepared(self, x, batch, cache, residual, table, pairing, eps):
         ops = self.rt.ops
@@ -246,7 +249,7 @@ class GQAttention(Mixer):
                                    v_first, self.blend)
         out = ops.paged_attention(q, cache.k, cache.v, cache.block_table, batch, self.heads, self.kv_heads, self.head_dim,
                                   self.scale, self.window, self.value_dim, sinks=self.sink)
-        return ops.linear(out, self.o, accumulate_into=residual, defer=True)
+        return ops.linear(out, self.o, accumulate_into=residual, defer=True, scale=self.out_scale)
 
     def parameters_bytes(self) -> int:
         ts = [self.qkv, self.o] + ([self.q_norm, self.k_norm] if self.q_norm is not None else []) + [

@@ -18,7 +18,8 @@ and ``sum_j p_j W_uv c_j = W_uv sum_j p_j c_j``. The attention kernel then sees 
 elements over one key head whose rows are ``[c, rotated part]`` and whose values are ``c`` again. The cache holds
 those rows and, as the values, ``c`` once more with the tokens of one element side by side (the order in which the
 matrix cores take the second product's operand). Options: a sliding ``window``, a learned sink per head in the softmax's
-denominator (``sinks``), a sigmoid gate per head read off the mixer's input (``gate``), and ``shares_cache``: the
+denominator (``sinks``), a sigmoid gate read off the mixer's input (``gate``: ``"head"`` or True, one per head;
+``"element"``, one per element of the concatenated heads), and ``shares_cache``: the
 layer has no projection of its own for the latent and reads the cache rows another layer wrote (its run-order entry
 names that layer's cache slot), with query, up-projections, window and the rest of its own.
 """
@@ -40,6 +41,7 @@ def _named(spec: PartSpec, default: dict) -> dict[str, str]:
 
 @register("mixer", "differential_attention")
 class DifferentialAttention(Mixer):
+    scales_output = True
     NAMES = {"q": "q", "k": "k", "v": "v", "o": "o", "q_conv": "q.conv", "k_conv": "k.conv", "v_conv": "v.conv",
              "q_norm": "q.norm", "k_norm": "k.norm", "lq1": "lq1", "lk1": "lk1", "lq2": "lq2", "lk2": "lk2"}
 
@@ -133,7 +135,7 @@ class DifferentialAttention(Mixer):
                                 self.scale, 0, self.value_dim, softcap=self.softcap, value_share=2, out_dtype=torch.float32)
         o = ops.map_difference_norm(a, self.kv_heads, self.group, self.value_dim, self.lam, self.eps, 1.0 - self.lambda_offset,
                                     self.rt.dtype)
-        return ops.linear(o, self.o, accumulate_into=residual, defer=True)
+        return ops.linear(o, self.o, accumulate_into=residual, defer=True, scale=self.out_scale)
 
     def parameters_bytes(self) -> int:
         ts = [self.proj, self.conv, self.o] + ([self.q_norm, self.k_norm] if self.q_norm is not None else [])
@@ -148,6 +150,7 @@ class DifferentialAttention(Mixer):
 
 @register("mixer", "latent_attention")
 class LatentAttention(Mixer):
+    scales_output = True
     NAMES = {"q": "q", "dkv": "dkv", "dkv_norm": "dkv.norm", "uk": "uk", "uv": "uv", "sink": "sink", "g": "g", "o": "o"}
 
     def __init__(self, spec: PartSpec, rt):
@@ -162,7 +165,11 @@ class LatentAttention(Mixer):
         self.window = int(spec.get("window") or 0)
         self.eps = float(spec["eps"])
         self.sinks = bool(spec.get("sinks", False))
-        self.gate = bool(spec.get("gate", False))
+        self.gate = spec.get("gate") or None
+        if self.gate is True:
+            self.gate = "head"
+        if self.gate not in (None, "head", "element"):
+            raise ValueError(f"gate {self.gate!r}: one per 'head', one per 'element' or None")
         self.shares_cache = bool(spec.get("shares_cache", False))
         self.names = _named(spec, self.NAMES)
         self.key_dim = self.latent_dim + self.rot_dim
@@ -191,8 +198,8 @@ class LatentAttention(Mixer):
             out[n["dkv_norm"]] = TensorSpec((c,), init="ones")
         if spec.get("sinks", False):
             out[n["sink"]] = TensorSpec((h,), init="uniform")
-        if spec.get("gate", False):
-            out[n["g"]] = TensorSpec((h, w))
+        if spec.get("gate"):
+            out[n["g"]] = TensorSpec((h * e if spec["gate"] == "element" else h, w))
         return out
 
     def bind(self, tensors) -> None:
@@ -227,10 +234,10 @@ class LatentAttention(Mixer):
             self.plain_dim, self.rot_dim, self.latent_dim, self.rt.dtype)
         ops.head_linear(q_plain, self.uk_t, q_full, 0)
         a = ops.paged_attention(q_full, cache.k, cache.v, cache.block_table, batch, self.heads, 1, self.key_dim, self.scale,
-                                self.window, self.latent_dim, sinks=self.sink)
+                                self.window, self.latent_dim, sinks=self.sink, wide_heads=True)
         o = torch.empty((x.shape[0], self.heads * self.value_dim), dtype=self.rt.dtype, device=x.device)
-        ops.head_linear(a, self.uv, o, 0, gate=(x32, self.g_col) if self.gate else None)
-        return ops.linear(o, self.o, accumulate_into=residual, defer=True)
+        ops.head_linear(a, self.uv, o, 0, gate=(x32, self.g_col) if self.gate else None, gate_each=self.gate == "element")
+        return ops.linear(o, self.o, accumulate_into=residual, defer=True, scale=self.out_scale)
 
     def parameters_bytes(self) -> int:
         ts = [self.proj, self.uk_t, self.uv, self.o] + [t for t in (self.dkv_norm, self.sink) if t is not None]

@@ -18,6 +18,9 @@ to bfloat16. Mixers and feed-forwards do not return their output: they either ad
 *pending* sum (``ops.SplitSum``: partial sums that still have to be added to ``residual``). Whoever
 reads the residual stream next takes the pending sum along: a norm adds it while it normalises
 (``add=``), anything else calls ``ops.add_pending`` first.
+
+A block may hang a factor per channel behind a sublayer (``Sublayer.scale_output``: a layer scale); what the sublayer adds or
+leaves pending is then already multiplied by it (a ``SplitSum`` carries the factors to the kernel that adds it).
 """
 
 from __future__ import annotations
@@ -227,7 +230,21 @@ class PositionEncoding(Part):
         return None
 
 
-class Mixer(Part):
+class Sublayer(Part):
+    """What adds to the residual stream: a mixer or a feed-forward. ``scales_output``: the part multiplies what it adds by
+    ``out_scale`` (float32 ``[width]``; None: by nothing)."""
+
+    scales_output = False
+    out_scale = None
+
+    def scale_output(self, scale) -> None:
+        """Multiply what this part adds to the stream by ``scale [width]``, element by element."""
+        if not self.scales_output:
+            raise NotImplementedError(f"{self.kind!r} cannot scale what it adds to the residual stream")
+        self.out_scale = scale.float().contiguous()
+
+
+class Mixer(Sublayer):
     def kv_need(self) -> KVNeed | None:
         return None
 
@@ -239,7 +256,7 @@ class Mixer(Part):
         raise NotImplementedError
 
 
-class FeedForward(Part):
+class FeedForward(Sublayer):
     def forward(self, x, residual):
         """Add the feed-forward's output to ``residual``, or return it as a pending sum."""
         raise NotImplementedError

@@ -13,32 +13,51 @@ from .registry import part_class, register
 
 @register("block", "prenorm")
 class PreNormBlock(Block):
+    """Options, none of which the reference has: ``mixer_scale`` / ``ffn_scale`` name a tensor ``[width]`` each by which what the
+    sublayer adds is multiplied element by element (a layer scale; the sublayer applies it, ``Sublayer.scale_output``); a
+    layer without a feed-forward has no second norm (``ffn_norm`` None), and ``spare`` then names tensors ``{name: width}``
+    that a checkpoint may still carry for it."""
+
     def __init__(self, spec: PartSpec, rt, mixer, feed_forward):
         super().__init__(spec, rt, mixer, feed_forward)
-        mn, fn = spec["mixer_norm"], spec["ffn_norm"]
+        mn, fn = spec["mixer_norm"], spec.get("ffn_norm")
         self.mixer_norm = part_class("norm", mn)(mn, rt)
-        self.ffn_norm = part_class("norm", fn)(fn, rt)
+        self.ffn_norm = part_class("norm", fn)(fn, rt) if fn is not None else None
 
     @classmethod
     def tensors(cls, spec: PartSpec) -> dict[str, TensorSpec]:
         out = {}
-        for key in ("mixer_norm", "ffn_norm"):
-            s = spec[key]
+        for key, scale in (("mixer_norm", "mixer_scale"), ("ffn_norm", "ffn_scale")):
+            s = spec.get(key)
+            if s is None:
+                continue
             out.update(part_class("norm", s).tensors(s))
+            if spec.get(scale):
+                out[spec[scale]] = TensorSpec((int(s["width"]),), init="ones")
+        for name, width in (spec.get("spare") or {}).items():
+            out[name] = TensorSpec((int(width),), optional=True)
         return out
 
     def bind(self, tensors) -> None:
         self.mixer_norm.bind(tensors)
-        self.ffn_norm.bind(tensors)
+        if self.spec.get("mixer_scale"):
+            self.mixer.scale_output(tensors[self.spec["mixer_scale"]])
+        if self.ffn_norm is not None:
+            self.ffn_norm.bind(tensors)
+            if self.spec.get("ffn_scale"):
+                self.feed_forward.scale_output(tensors[self.spec["ffn_scale"]])
 
     def forward(self, residual, batch, cache, state, pending=None):
         x = self.mixer_norm.forward(residual, add=pending)
         pending = self.mixer.forward(x, batch, cache, state, residual)
+        if self.ffn_norm is None:
+            return pending
         y = self.ffn_norm.forward(residual, add=pending)
         return self.feed_forward.forward(y, residual)
 
     def parameters_bytes(self) -> int:
-        return self.mixer_norm.parameters_bytes() + self.ffn_norm.parameters_bytes()
+        scales = sum(s.numel() * s.element_size() for s in (self.mixer.out_scale, self.feed_forward.out_scale) if s is not None)
+        return scales + self.mixer_norm.parameters_bytes() + (self.ffn_norm.parameters_bytes() if self.ffn_norm is not None else 0)
 
 
 @register("block", "parallel")

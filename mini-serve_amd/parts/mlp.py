@@ -24,7 +24,8 @@ among them); ``scoring="softmax"`` (the router's softmax runs over all its outpu
 value plus ``router_bias``, a correction that only the choice sees; the weights are the chosen outputs' softmax values
 as they stand, not renormalised); ``groups`` / ``keep_groups`` (with that scoring: the router's outputs form ``groups``
 equal groups of neighbours, a group's score is the largest choice score in it, and only outputs of the ``keep_groups``
-best groups can be chosen); ``identity`` (the router has that many outputs more than there are experts with weights; a
+best groups can be chosen); ``scoring="sigmoid"`` (the same with every output's sigmoid for its softmax value);
+``weigh="input"`` (a choice's weight multiplies what the expert reads instead of what it puts out); ``identity`` (the router has that many outputs more than there are experts with weights; a
 token that chooses one of them gets its own input back, times the weight)."""
 
 from __future__ import annotations
@@ -51,6 +52,8 @@ class NoFeedForward(FeedForward):
 
 @register("feed_forward", "gated_mlp")
 class GatedMLP(FeedForward):
+    scales_output = True
+
     def __init__(self, spec: PartSpec, rt):
         super().__init__(spec, rt)
         self.prefix = spec.get("prefix", "")
@@ -85,7 +88,7 @@ class GatedMLP(FeedForward):
     def forward(self, x, residual):
         ops = self.rt.ops
         m = ops.gated_linear(x, self.gate_up, self.activation, out_dtype=self.rt.dtype, block=self.block, limit=self.limit)
-        return ops.linear(m, self.down, accumulate_into=residual, defer=True)
+        return ops.linear(m, self.down, accumulate_into=residual, defer=True, scale=self.out_scale)
 
     def parameters_bytes(self) -> int:
         return sum(t.numel() * t.element_size() for t in (self.gate_up, self.down))
@@ -96,6 +99,8 @@ class GatedMLP(FeedForward):
 
 @register("feed_forward", "dense_mlp")
 class DenseMLP(FeedForward):
+    scales_output = True
+
     def __init__(self, spec: PartSpec, rt):
         super().__init__(spec, rt)
         self.prefix = spec.get("prefix", "")
@@ -120,7 +125,7 @@ class DenseMLP(FeedForward):
     def forward(self, x, residual):
         ops = self.rt.ops
         m = ops.activate(ops.linear(x, self.up, out_dtype=torch.float32), self.activation, self.rt.dtype)
-        return ops.linear(m, self.down, accumulate_into=residual, defer=True)
+        return ops.linear(m, self.down, accumulate_into=residual, defer=True, scale=self.out_scale)
 
     def parameters_bytes(self) -> int:
         return sum(t.numel() * t.element_size() for t in (self.up, self.down))
@@ -138,6 +143,8 @@ def _moe_names(spec: PartSpec) -> dict[str, str]:
 
 @register("feed_forward", "moe_mlp")
 class MixtureMLP(FeedForward):
+    scales_output = True
+
     def __init__(self, spec: PartSpec, rt):
         super().__init__(spec, rt)
         self.prefix = spec.get("prefix", "")
@@ -153,12 +160,15 @@ class MixtureMLP(FeedForward):
         self.keep_groups = int(spec.get("keep_groups") or self.groups)
         self.identity = int(spec.get("identity") or 0)
         self.outputs = self.num_experts + self.identity  # what the router tells apart
-        if self.scoring not in ("chosen_softmax", "softmax"):
-            raise ValueError(f"router scoring {self.scoring!r}: 'chosen_softmax' or 'softmax'")
+        self.weigh = spec.get("weigh", "output")
+        if self.scoring not in ("chosen_softmax", "softmax", "sigmoid"):
+            raise ValueError(f"router scoring {self.scoring!r}: 'chosen_softmax', 'softmax' or 'sigmoid'")
+        if self.weigh not in ("output", "input"):
+            raise ValueError(f"weigh {self.weigh!r}: what a choice's weight multiplies, 'output' or 'input'")
         if self.identity < 0 or self.num_experts < 1:
             raise ValueError(f"{self.num_experts} experts and {self.identity} identity experts")
-        if self.groups != 1 and self.scoring != "softmax":
-            raise NotImplementedError("groups of experts go with scoring='softmax'")
+        if self.groups != 1 and self.scoring == "chosen_softmax":
+            raise NotImplementedError("groups of experts go with scores over all outputs")
         if self.groups < 1 or self.outputs % self.groups or not 1 <= self.keep_groups <= self.groups:
             raise ValueError(f"{self.outputs} router outputs in {self.groups} groups of which {self.keep_groups} are kept")
         if not 1 <= self.top <= (self.outputs // self.groups) * self.keep_groups:
@@ -214,13 +224,18 @@ class MixtureMLP(FeedForward):
         if self.shared is not None:
             self.shared.bind(tensors)
 
+    def scale_output(self, scale) -> None:
+        super().scale_output(scale)
+        if self.shared is not None:
+            self.shared.scale_output(scale)
+
     def forward(self, x, residual):
         ops = self.rt.ops
         pending = self.shared.forward(x, residual) if self.shared is not None else None
         logits = ops.linear(x, self.router, out_dtype=torch.float32, defer=True)  # few rows: partial sums, added by the routing
         ids, weights = ops.moe_route(logits, self.bias, self.top, self.scoring, self.groups, self.keep_groups)
         xe = ops.cast(x, self.up.dtype)  # experts stored in 32-bit compute in 32-bit
-        ops.moe_experts(xe, ids, weights, self.gate, self.up, self.down, self.activation, residual)
+        ops.moe_experts(xe, ids, weights, self.gate, self.up, self.down, self.activation, residual, self.weigh == "input", self.out_scale)
         return pending
 
     def parameters_bytes(self) -> int:

@@ -27,6 +27,18 @@ kernel reads in place (activation, scale and gates are applied on the way in).
   each head's output is divided by its root mean square, the heads are concatenated, multiplied by a weight and by
   ``silu(W_g mix_g)`` and projected. Its five products read five different inputs, so they stay five products; they
   write into the columns of one float32 matrix that the kernels behind them read side by side.
+
+Two more have a short causal convolution over time between projection and recurrence (``ops.time_conv``; a request's last
+``conv_taps - 1`` inputs are part of its state):
+
+* ``mamba2``: one projection (``in``) to a gate, values, keys, queries and a step size per head; values, keys and queries pass
+  the convolution (with a bias) and a SiLU; ``heads / groups`` neighbouring heads share keys and queries; with ``d =
+  softplus(step + dt_bias)``, ``S_t = exp(-exp(A_log) d) S_(t-1) + d k_t v_t^T``, ``y_t = S_t^T q_t + D v_t``; ``y silu(gate)`` is
+  RMS-normed in ``norm_groups`` equal parts, multiplied by a weight and projected.
+* ``rglru``: two projections with biases in one product; one passes the convolution (with a bias), drives the recurrence and
+  its gates: ``r``, ``i`` the sigmoids of block-diagonal products, ``log a = -decay_factor r softplus(lam)``, ``S_t = a S_(t-1) +
+  sqrt(1 - a^2) i u`` per channel; the other multiplies the result through a GELU. A vector per request is all it keeps
+  beside the convolution's inputs.
 """
 
 from __future__ import annotations
@@ -48,6 +60,7 @@ class _RecurrentMixer(Mixer):
     """What the two recurrent mixers share: sizes, the fused projection and the gated output norm."""
 
     NAMES: dict = {}
+    scales_output = True
 
     def __init__(self, spec: PartSpec, rt):
         super().__init__(spec, rt)
@@ -79,7 +92,7 @@ class _RecurrentMixer(Mixer):
         n = self.heads * self.value_dim
         gate = x32[:, self.columns["g"] : self.columns["g"] + n]
         y = ops.group_rmsnorm_gate(o, group, self.norm, gate, self.eps, self.rt.dtype, gate_activation)
-        return ops.linear(y, self.o, accumulate_into=residual, defer=True)
+        return ops.linear(y, self.o, accumulate_into=residual, defer=True, scale=self.out_scale)
 
     def parameters_bytes(self) -> int:
         return sum(t.numel() * t.element_size() for t in (self.proj, self.o, self.norm) if t is not None)
@@ -272,7 +285,7 @@ class WKV(_RecurrentMixer):
             gate = x32[:, c["g"] : c["g"] + n]
             o = ops.gated_recurrence(x32, c, self.heads, self.dim, self.dim, batch, state, mode="wkv", channel_decay=decay, bonus=self.u)
         y = ops.group_rmsnorm_gate(o, self.dim, self.norm, gate, self.eps, self.rt.dtype, "silu")
-        return ops.linear(y, self.o, accumulate_into=residual, defer=True)
+        return ops.linear(y, self.o, accumulate_into=residual, defer=True, scale=self.out_scale)
 
     def parameters_bytes(self) -> int:
         ts = self.weights + [self.mu, self.w2, self.w0, self.u, self.o, self.norm]
@@ -284,6 +297,148 @@ class WKV(_RecurrentMixer):
         rank = self.rank or 0
         linear = 2 * tokens * self.hidden * (4 * n + rank) + 2 * tokens * rank * n + 2 * tokens * n * self.hidden
         return linear + 6 * tokens * self.heads * self.dim * self.dim
+
+
+def _f32(t):
+    """The tensor in float32 (widening is exact): what enters a recurrence."""
+    return t.to(torch.float32).contiguous()
+
+
+@register("mixer", "mamba2")
+class Mamba2(Mixer):
+    NAMES = {"in": "in", "conv": "conv", "conv_bias": "conv.b", "dt_bias": "dt_bias", "a_log": "A_log", "d": "D", "norm": "norm", "o": "o"}
+    scales_output = True
+
+    def __init__(self, spec: PartSpec, rt):
+        super().__init__(spec, rt)
+        self.hidden = int(spec["hidden_size"])
+        self.heads, self.groups = int(spec["num_heads"]), int(spec.get("groups") or 1)
+        self.dim, self.value_dim = int(spec["head_dim"]), int(spec["value_dim"])
+        self.taps, self.norm_groups = int(spec["conv_taps"]), int(spec.get("norm_groups") or 1)
+        self.eps = float(spec["eps"])
+        self.names = _named(spec, self.NAMES)
+        self.inner = self.heads * self.value_dim
+        self.channels = self.inner + 2 * self.groups * self.dim  # what the convolution runs over
+        if min(self.heads, self.groups, self.dim, self.value_dim, self.taps, self.norm_groups) < 1:
+            raise ValueError("heads, groups, sizes and taps must be positive")
+        if self.heads % self.groups or self.inner % self.norm_groups:
+            raise ValueError(f"{self.heads} heads in {self.groups} groups, {self.inner} channels normed in {self.norm_groups} parts")
+        if max(self.dim, self.value_dim) > 256:
+            raise ValueError(f"sizes {self.dim} / {self.value_dim}: the recurrence kernels take sizes 1..256")
+        # columns behind the convolution; in front of it a gate of `inner` columns comes first and the steps come last
+        self.columns = {"v": 0, "k": self.inner, "q": self.inner + self.groups * self.dim}
+        self.step_col = self.inner + self.channels
+        self.proj = self.conv = self.conv_bias = self.dt_bias = self.decay = self.skip = self.norm = self.o = None
+
+    @classmethod
+    def tensors(cls, spec: PartSpec) -> dict[str, TensorSpec]:
+        n = _named(spec, cls.NAMES)
+        w, h, d, e = (int(spec[k]) for k in ("hidden_size", "num_heads", "head_dim", "value_dim"))
+        inner, keys = h * e, int(spec.get("groups") or 1) * d
+        c = inner + 2 * keys
+        return {n["in"]: TensorSpec((inner + c + h, w)), n["conv"]: TensorSpec((c, int(spec["conv_taps"]))),
+                n["conv_bias"]: TensorSpec((c,), init="uniform"), n["dt_bias"]: TensorSpec((h,), init="uniform"),
+                n["a_log"]: TensorSpec((h,), init="uniform"), n["d"]: TensorSpec((h,), init="ones"),
+                n["norm"]: TensorSpec((inner,), init="ones"), n["o"]: TensorSpec((w, inner))}
+
+    def bind(self, tensors) -> None:
+        n = self.names
+        # rows of the projection up to a multiple of four, so that every row of its result starts 16-byte aligned
+        proj = tensors[n["in"]]
+        fill = -proj.shape[0] % 4
+        self.proj = torch.cat((proj, proj.new_zeros((fill, self.hidden))), dim=0).contiguous() if fill else proj
+        self.conv = _f32(tensors[n["conv"]].t())
+        self.conv_bias, self.dt_bias, self.skip = (_f32(tensors[n[k]]) for k in ("conv_bias", "dt_bias", "d"))
+        self.decay = -torch.exp(_f32(tensors[n["a_log"]]))
+        self.norm, self.o = tensors[n["norm"]], tensors[n["o"]]
+
+    def state_need(self) -> StateNeed:
+        own = (StateTensor("S", (self.heads, self.dim, self.value_dim), "float32"),)
+        return StateNeed(own + ((StateTensor("conv", (self.taps - 1, self.channels), "float32"),) if self.taps > 1 else ()))
+
+    def forward(self, x, batch, cache, state, residual):
+        ops = self.rt.ops
+        x32 = ops.linear(x, self.proj, out_dtype=torch.float32)
+        xbc = ops.time_conv(x32, self.inner, self.conv, self.conv_bias, state.get("conv"), batch, "silu")
+        y = ops.step_recurrence(xbc, self.columns, self.heads, self.dim, self.value_dim, self.groups, x32, self.step_col, self.dt_bias,
+                                self.decay, self.skip, batch, state["S"])
+        y = ops.group_rmsnorm_gate(y, self.inner // self.norm_groups, self.norm, x32[:, : self.inner], self.eps, self.rt.dtype, "silu",
+                                   gate_first=True)
+        return ops.linear(y, self.o, accumulate_into=residual, defer=True, scale=self.out_scale)
+
+    def parameters_bytes(self) -> int:
+        ts = (self.proj, self.conv, self.conv_bias, self.dt_bias, self.decay, self.skip, self.norm, self.o)
+        return sum(t.numel() * t.element_size() for t in ts)
+
+    def flops(self, rows) -> int:
+        tokens = sum(n for n, _ in rows)
+        linear = 2 * tokens * self.hidden * (self.step_col + self.heads + self.inner)
+        return linear + 2 * tokens * self.channels * self.taps + 4 * tokens * self.heads * self.dim * self.value_dim
+
+
+@register("mixer", "rglru")
+class RGLRU(Mixer):
+    NAMES = {"y": "y", "y_bias": "y.b", "x": "x", "x_bias": "x.b", "conv": "conv", "conv_bias": "conv.b", "r": "ra", "r_bias": "ra.b",
+             "i": "ri", "i_bias": "ri.b", "lam": "lam", "o": "o"}
+    scales_output = True
+
+    def __init__(self, spec: PartSpec, rt):
+        super().__init__(spec, rt)
+        self.hidden, self.width, self.blocks, self.taps = (int(spec[k]) for k in ("hidden_size", "width", "blocks", "conv_taps"))
+        self.decay_factor = float(spec["decay_factor"])
+        self.names = _named(spec, self.NAMES)
+        if min(self.hidden, self.width, self.blocks, self.taps) < 1 or self.width % self.blocks:
+            raise ValueError(f"a width of {self.width} in {self.blocks} blocks, {self.taps} taps")
+        if not self.decay_factor > 0:
+            raise ValueError(f"decay_factor must be positive, not {self.decay_factor}")
+        self.y_col = -(-self.width // 4) * 4  # the convolution's branch first, then the other, 16-byte aligned
+        self.proj = self.o = self.r = self.i = None
+        self.vectors: dict = {}
+
+    @classmethod
+    def tensors(cls, spec: PartSpec) -> dict[str, TensorSpec]:
+        n = _named(spec, cls.NAMES)
+        h, w, b = (int(spec[k]) for k in ("hidden_size", "width", "blocks"))
+        out = {n[k]: TensorSpec((w, h)) for k in ("y", "x")}
+        out.update({n[k]: TensorSpec((w,), init="uniform") for k in ("y_bias", "x_bias", "conv_bias", "lam")})
+        out[n["conv"]] = TensorSpec((w, int(spec["conv_taps"])))
+        for k in ("r", "i"):
+            out[n[k]] = TensorSpec((b, w // b, w // b))
+            out[n[k + "_bias"]] = TensorSpec((b, w // b), init="uniform")
+        out[n["o"]] = TensorSpec((h, w))
+        return out
+
+    def bind(self, tensors) -> None:
+        n = self.names
+        x, y = tensors[n["x"]], tensors[n["y"]]
+        if x.dtype != y.dtype:
+            raise ValueError(f"{n['x']} and {n['y']} are stored in different dtypes")
+        fill = x.new_zeros((self.y_col - self.width, self.hidden))
+        self.proj = torch.cat((x, fill, y, fill), dim=0).contiguous()
+        self.r, self.i, self.o = (tensors[n[k]] for k in ("r", "i", "o"))
+        self.vectors = {k: _f32(tensors[n[k]].reshape(-1)) for k in ("x_bias", "y_bias", "conv_bias", "r_bias", "i_bias")}
+        self.vectors["conv"] = _f32(tensors[n["conv"]].t())
+        self.vectors["coef"] = -self.decay_factor * torch.nn.functional.softplus(_f32(tensors[n["lam"]]))
+
+    def state_need(self) -> StateNeed:
+        own = (StateTensor("S", (self.width,), "float32"),)
+        return StateNeed(own + ((StateTensor("conv", (self.taps - 1, self.width), "float32"),) if self.taps > 1 else ()))
+
+    def forward(self, x, batch, cache, state, residual):
+        ops, v = self.rt.ops, self.vectors
+        x32 = ops.linear(x, self.proj, out_dtype=torch.float32)
+        u = ops.time_conv(x32, 0, v["conv"], v["conv_bias"], state.get("conv"), batch, None, v["x_bias"])
+        o = ops.rglru(u, self.blocks, self.r, self.i, v["r_bias"], v["i_bias"], v["coef"], x32, self.y_col, v["y_bias"], batch, state["S"],
+                      self.rt.dtype)
+        return ops.linear(o, self.o, accumulate_into=residual, defer=True, scale=self.out_scale)
+
+    def parameters_bytes(self) -> int:
+        return sum(t.numel() * t.element_size() for t in (self.proj, self.r, self.i, self.o, *self.vectors.values()))
+
+    def flops(self, rows) -> int:
+        tokens = sum(n for n, _ in rows)
+        linear = 2 * tokens * self.hidden * 3 * self.width + 4 * tokens * self.width * (self.width // self.blocks)
+        return linear + tokens * self.width * (2 * self.taps + 8)
 
 
 @register("mixer", "normed_pair")
