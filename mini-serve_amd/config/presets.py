@@ -167,6 +167,27 @@ def _zigelorn_tiny() -> dict:
 PRESETS["zigelorn-tiny"] = _zigelorn_tiny()
 
 
+def _bipazen_tiny() -> dict:
+    """Six layers that hold every part of the architecture once: the three mixers, layers that run another's weights over a
+    state or a cache of their own, and a layer without a feed-forward."""
+
+    def moe(experts, top, ff):
+        return {"kind": "moe", "router": {"experts": experts, "top": top}, "expert": {"ff": ff}}
+
+    mamba2 = {"type": "mamba2", "mixer": {"heads": 6, "vdim": 24, "state": 32, "groups": 3, "conv": 3, "norm_groups": 2}, "mlp": moe(5, 2, 48)}
+    rglru = {"type": "rglru", "mixer": {"width": 120, "blocks": 5, "conv": 4}, "mlp": moe(4, 1, 64)}
+    latent = {"type": "latent_attention", "mixer": {"heads": 4, "dim": 16, "rot_dim": 8, "vdim": 24, "kv_rank": 40, "scale": 24 ** -0.5,
+                                                    "rot": {"base": 2000.0, "dims": 8}}, "mlp": moe(6, 3, 32)}
+    return {
+        "architecture": "Bipazen", "vocab": 311, "width": 96, "norm": {"eps": 1e-5},
+        "layers": [rglru, latent, mamba2, dict(copy.deepcopy(latent), weights_of=1), dict(copy.deepcopy(rglru), weights_of=0),
+                   {"type": "mamba2", "mixer": {"heads": 2, "vdim": 40, "state": 16, "groups": 1, "conv": 2, "norm_groups": 1}, "mlp": None}],
+    }
+
+
+PRESETS["bipazen-tiny"] = _bipazen_tiny()
+
+
 def preset(name: str) -> dict:
     try:
         return copy.deepcopy(PRESETS[name])

@@ -1,6 +1,6 @@
 """Prefill and decode throughput of one architecture beside another of equal size: random weights, layers of the
 sizes real models have, the same step function for both. ``bench.py --design kakunex`` (or ``fimolix``, ``reselorn``,
-``zigelorn``) prints what this returns.
+``zigelorn``, ``bipazen``) prints what this returns.
 
 A *shape* fixes what the two share: width, query and key/value heads of 128 elements, feed-forward width, window,
 layers, vocabulary. The Kakunex model of a shape repeats (parallel, parallel, parallel, mlstm): window attention that
@@ -24,7 +24,14 @@ of each rotated, slowed frequencies) inside the shape's window, the retention as
 queries and keys, the wkv layers ``width / 64`` heads of 64 x 64 with a decay projection 64 wide. Feed-forwards alternate:
 a dense one without a gate, 1.5 times the shape's width (as many multiplications as the gated one of the shape), and a
 mixture of 28 experts of a quarter of that beside 4 identity experts, 8 groups of which 4 are kept, 4 chosen. It is
-measured beside the Kakunex model of the shape, the other design of windowed attention and linear recurrences."""
+measured beside the Kakunex model of the shape, the other design of windowed attention and linear recurrences.
+
+The Bipazen model of a shape repeats (mamba2, rglru, latent attention, rglru): the mamba2 layers have twice the width in heads
+of 64 values with a state of 128, eight heads to a group of keys and queries, four taps; the rglru layers the shape's width in blocks of 256 channels; the latent attention the shape's query heads with 128 plain and 64
+rotated elements, values of 128 and a latent of 512 per token. Every layer has a mixture of 32 experts of a quarter of the
+shape's feed-forward width, of which a token runs 4: as many multiplications as in the shape's dense feed-forward. It is
+measured beside the Zigelorn model of the shape, the other design of attention, recurrences with a matrix state and routed
+experts."""
 
 from __future__ import annotations
 
@@ -112,9 +119,22 @@ def zigelorn_config(s: dict) -> dict:
     return {"architecture": "Zigelorn", "vocab": s["vocab"], "width": s["width"], "norm": {"eps": 1e-6}, "layers": layers}
 
 
+def bipazen_config(s: dict) -> dict:
+    heads = 2 * s["width"] // 64
+    mamba2 = {"heads": heads, "vdim": 64, "state": 128, "groups": max(1, heads // 8), "conv": 4, "norm_groups": max(1, heads // 8)}
+    rglru = {"width": s["width"], "blocks": s["width"] // 256, "conv": 4}
+    latent = {"heads": s["heads"], "dim": HEAD, "rot_dim": ROTATED, "vdim": HEAD, "kv_rank": LATENT, "scale": (HEAD + ROTATED) ** -0.5,
+              "rot": {"base": 1e6, "dims": ROTATED}}
+    mlp = {"kind": "moe", "router": {"experts": EXPERTS, "top": CHOSEN}, "expert": {"ff": s["ff"] // 4}}
+    kinds = (("mamba2", mamba2), ("rglru", rglru), ("latent_attention", latent), ("rglru", rglru))
+    layers = [{"type": kinds[i % 4][0], "mixer": dict(kinds[i % 4][1]), "mlp": dict(mlp)} for i in range(s["layers"])]
+    return {"architecture": "Bipazen", "vocab": s["vocab"], "width": s["width"], "norm": {"eps": 1e-6}, "layers": layers}
+
+
 DESIGNS = {"kakunex": kakunex_config, "fimolix": fimolix_config, "reselorn": reselorn_config, "zigelorn": zigelorn_config,
+           "bipazen": bipazen_config,
            "qwen3": qwen3_config}
-BESIDE = {"zigelorn": "kakunex"}  # the model a design is measured beside (default: qwen3)
+BESIDE = {"zigelorn": "kakunex", "bipazen": "zigelorn"}  # the model a design is measured beside (default: qwen3)
 
 
 def measure(config: dict, dtype: str, prefill_tokens: int, batch: int, context: int, steps: int, warmup: int, say=lambda m: None) -> dict:
