@@ -82,19 +82,20 @@ extern "C" int ms_moe_route(const float* logits, int ld, int splits, long long s
 // `groups` equal groups of neighbours, a group's score is its largest c, and only outputs of the `keep` best groups
 // (ties: the lower group) can be chosen: the others' c counts as minus infinity. The `top` largest c are chosen, largest
 // first (ties: the lower index). One wave per token; s and c of a token pass through the wave's own rows of LDS.
-template <typename TB>
+// PER: outputs a lane holds (64 PER cover them all).
+template <typename TB, int PER>
 __global__ __launch_bounds__(256) void moe_route_scored_kernel(const float* __restrict__ logits, int ld, int splits, size_t stride,
                                                                const TB* __restrict__ correction, int T, int E, int top,
                                                                int groups, int keep, int sigmoid, int* __restrict__ ids,
                                                                float* __restrict__ weights) {
-  __shared__ float ss[4][MOE_MAX_EXPERTS], cs[4][MOE_MAX_EXPERTS];
+  __shared__ float ss[4][PER * WAVE], cs[4][PER * WAVE];
   const int wave = threadIdx.x / WAVE, lane = threadIdx.x % WAVE;
   const int t = blockIdx.x * 4 + wave;
   const bool live = t < T;  // every wave stays for the block's barriers
-  float c[MOE_MAX_EXPERTS / WAVE];
+  float c[PER];
   float m = -INFINITY;
 #pragma unroll
-  for (int i = 0; i < MOE_MAX_EXPERTS / WAVE; ++i) {
+  for (int i = 0; i < PER; ++i) {
     const int e = lane + i * WAVE;
     c[i] = (live && e < E) ? sum_splits(logits + (size_t)t * ld + e, splits, stride) : -INFINITY;
     m = fmaxf(m, c[i]);
@@ -102,13 +103,13 @@ __global__ __launch_bounds__(256) void moe_route_scored_kernel(const float* __re
   m = wave_max(m);
   float sum = 0.f;
 #pragma unroll
-  for (int i = 0; i < MOE_MAX_EXPERTS / WAVE; ++i) {
+  for (int i = 0; i < PER; ++i) {
     if (!sigmoid) c[i] = lane + i * WAVE < E ? expf(c[i] - m) : 0.f;
     sum += c[i];
   }
   sum = wave_sum(sum);
 #pragma unroll
-  for (int i = 0; i < MOE_MAX_EXPERTS / WAVE; ++i) {
+  for (int i = 0; i < PER; ++i) {
     const int e = lane + i * WAVE;
     if (e < E) {
       const float sc = sigmoid ? 1.f / (1.f + expf(-c[i])) : c[i] / sum;
@@ -122,10 +123,10 @@ __global__ __launch_bounds__(256) void moe_route_scored_kernel(const float* __re
   if (groups > 1) {
     const int n = E / groups;
     __syncthreads();
-    float gm[MOE_MAX_EXPERTS / WAVE];  // lane l holds the scores of groups l, l + 64, ...
-    bool taken[MOE_MAX_EXPERTS / WAVE];
+    float gm[PER];  // lane l holds the scores of groups l, l + 64, ...
+    bool taken[PER];
 #pragma unroll
-    for (int i = 0; i < MOE_MAX_EXPERTS / WAVE; ++i) {
+    for (int i = 0; i < PER; ++i) {
       const int g = lane + i * WAVE;
       gm[i] = -INFINITY;
       taken[i] = false;
@@ -134,13 +135,13 @@ __global__ __launch_bounds__(256) void moe_route_scored_kernel(const float* __re
     }
     __syncthreads();  // cs is read; from here on it says which groups stay (1) and which do not (0)
 #pragma unroll
-    for (int i = 0; i < MOE_MAX_EXPERTS / WAVE; ++i)
+    for (int i = 0; i < PER; ++i)
       if (lane + i * WAVE < groups) cs[wave][lane + i * WAVE] = 0.f;
     for (int j = 0; j < keep; ++j) {
       float best = -INFINITY;
       int at = 0x7fffffff;
 #pragma unroll
-      for (int i = 0; i < MOE_MAX_EXPERTS / WAVE; ++i)
+      for (int i = 0; i < PER; ++i)
         if (lane + i * WAVE < groups && !taken[i] && (at == 0x7fffffff || gm[i] > best)) { best = gm[i]; at = lane + i * WAVE; }
 #pragma unroll
       for (int off = WAVE / 2; off > 0; off >>= 1) {
@@ -149,12 +150,12 @@ __global__ __launch_bounds__(256) void moe_route_scored_kernel(const float* __re
         if (oa != 0x7fffffff && (at == 0x7fffffff || ob > best || (ob == best && oa < at))) { best = ob; at = oa; }
       }
 #pragma unroll
-      for (int i = 0; i < MOE_MAX_EXPERTS / WAVE; ++i)
+      for (int i = 0; i < PER; ++i)
         if (lane + i * WAVE == at) { taken[i] = true; cs[wave][at] = 1.f; }
     }
     __syncthreads();
 #pragma unroll
-    for (int i = 0; i < MOE_MAX_EXPERTS / WAVE; ++i) {
+    for (int i = 0; i < PER; ++i) {
       const int e = lane + i * WAVE;
       if (e < E && cs[wave][e / n] == 0.f) c[i] = -INFINITY;
     }
@@ -166,7 +167,7 @@ __global__ __launch_bounds__(256) void moe_route_scored_kernel(const float* __re
     float best = -INFINITY;
     int at = 0x7fffffff;
 #pragma unroll
-    for (int i = 0; i < MOE_MAX_EXPERTS / WAVE; ++i)
+    for (int i = 0; i < PER; ++i)
       if (c[i] > best) { best = c[i]; at = lane + i * WAVE; }
 #pragma unroll
     for (int off = WAVE / 2; off > 0; off >>= 1) {
@@ -176,7 +177,7 @@ __global__ __launch_bounds__(256) void moe_route_scored_kernel(const float* __re
     }
     if (at >= E) at = j;  // nothing left to choose by (no numbers, or fewer outputs in the kept groups than choices)
 #pragma unroll
-    for (int i = 0; i < MOE_MAX_EXPERTS / WAVE; ++i)
+    for (int i = 0; i < PER; ++i)
       if (lane + i * WAVE == at) c[i] = -INFINITY;
     if (lane == 0) {
       ids[(size_t)t * top + j] = at;
@@ -194,8 +195,11 @@ extern "C" int ms_moe_route_scored(const float* logits, int ld, int splits, long
     return MS_BAD_ARG;
   if (E > MOE_MAX_EXPERTS || top > MOE_MAX_TOP) return MS_UNSUPPORTED;
   const unsigned blocks = (unsigned)((T + 3) / 4);
-  if (correction_is_bf16) moe_route_scored_kernel<bf16><<<blocks, 256, 0, st>>>(logits, ld, splits, (size_t)stride, (const bf16*)correction, T, E, top, groups, keep, sigmoid, ids, weights);
-  else moe_route_scored_kernel<float><<<blocks, 256, 0, st>>>(logits, ld, splits, (size_t)stride, (const float*)correction, T, E, top, groups, keep, sigmoid, ids, weights);
+#define ROUTE(TB, PER) moe_route_scored_kernel<TB, PER><<<blocks, 256, 0, st>>>(logits, ld, splits, (size_t)stride, (const TB*)correction, T, E, top, groups, keep, sigmoid, ids, weights)
+#define ROUTE_PER(TB) do { if (E <= WAVE) ROUTE(TB, 1); else if (E <= 2 * WAVE) ROUTE(TB, 2); else ROUTE(TB, MOE_MAX_EXPERTS / WAVE); } while (0)
+  if (correction_is_bf16) ROUTE_PER(bf16); else ROUTE_PER(float);
+#undef ROUTE_PER
+#undef ROUTE
   return launch_status();
 }
 
@@ -214,15 +218,24 @@ __global__ __launch_bounds__(1024) void moe_plan_kernel(const int* __restrict__ 
   for (int p = tid; p < P; p += 1024)
     if (ids[p] < E) atomicAdd(&counts[max(ids[p], 0)], 1);
   __syncthreads();
-  if (tid == 0) {
+  if (tid < WAVE) {  // running sums of the counts and of the tiles, 64 experts at a time
     int off = 0, nt = 0;
-    for (int e = 0; e < E; ++e) {
-      offsets[e] = off;
-      tile_base[e] = nt;
-      off += counts[e];
-      nt += (counts[e] + tile_rows - 1) / tile_rows;
+    for (int e0 = 0; e0 < E; e0 += WAVE) {
+      const int e = e0 + tid, n = e < E ? counts[e] : 0, t = (n + tile_rows - 1) / tile_rows;
+      int no = n, to = t;
+#pragma unroll
+      for (int d = 1; d < WAVE; d <<= 1) {
+        const int a = __shfl_up(no, d, WAVE), b = __shfl_up(to, d, WAVE);
+        if (tid >= d) no += a, to += b;
+      }
+      if (e < E) {
+        offsets[e] = off + no - n;
+        tile_base[e] = nt + to - t;
+      }
+      off += __shfl(no, WAVE - 1, WAVE);
+      nt += __shfl(to, WAVE - 1, WAVE);
     }
-    total_tiles = nt;
+    if (tid == 0) total_tiles = nt;
   }
   __syncthreads();
   for (int e = tid; e < E; e += 1024) {
@@ -721,19 +734,35 @@ extern "C" int ms_moe_gemm(const void* a, int lda, const void* w1, const void* w
 // ---------------------------------------------------------------------------------------------
 // stream[t][n] += scale[n] (where it is given) times the sum over j < top of y[t * top + j][n], in ascending j. With ids: a choice whose id is `real` or more is
 // an identity expert, and its term is weights[t * top + j] * x[t][n] (y holds nothing for it).
-template <typename TX>
-__global__ void moe_combine_kernel(float* __restrict__ stream, const float* __restrict__ y, int top, int N,
-                                   const int* __restrict__ ids, const float* __restrict__ weights, const TX* __restrict__ x,
-                                   int ldx, int real, const float* __restrict__ scale) {
-  const int n = blockIdx.x * blockDim.x + threadIdx.x;
+// A thread owns VEC consecutive columns of a token.
+template <typename TX, int VEC>
+__global__ __launch_bounds__(256) void moe_combine_kernel(float* __restrict__ stream, const float* __restrict__ y, int top, int N,
+                                                          const int* __restrict__ ids, const float* __restrict__ weights,
+                                                          const TX* __restrict__ x, int ldx, int real, const float* __restrict__ scale) {
+  struct alignas(4 * VEC) Columns { float e[VEC]; };
+  const int n = (blockIdx.x * blockDim.x + threadIdx.x) * VEC;
   if (n >= N) return;
   const size_t t = blockIdx.y;
-  float acc = 0.f;
+  float acc[VEC];
+#pragma unroll
+  for (int i = 0; i < VEC; ++i) acc[i] = 0.f;
+#pragma unroll 4
   for (int j = 0; j < top; ++j) {
-    if (ids != nullptr && ids[t * top + j] >= real) acc += weights[t * top + j] * to_f32(x[t * ldx + n]);
-    else acc += y[(t * top + j) * N + n];
+    if (ids != nullptr && ids[t * top + j] >= real) {
+      const float w = weights[t * top + j];
+#pragma unroll
+      for (int i = 0; i < VEC; ++i) acc[i] += w * to_f32(x[t * ldx + n + i]);
+    } else {
+      const Columns v = *reinterpret_cast<const Columns*>(y + (t * top + j) * N + n);
+#pragma unroll
+      for (int i = 0; i < VEC; ++i) acc[i] += v.e[i];
+    }
   }
-  stream[t * N + n] += scale ? acc * scale[n] : acc;
+  Columns* s = reinterpret_cast<Columns*>(stream + t * N + n);
+  Columns v = *s;
+#pragma unroll
+  for (int i = 0; i < VEC; ++i) v.e[i] += scale ? acc[i] * scale[n + i] : acc[i];
+  *s = v;
 }
 
 extern "C" int ms_moe_combine(float* stream, const float* y, int T, int top, int N, const int* ids, const float* weights,
@@ -741,8 +770,12 @@ extern "C" int ms_moe_combine(float* stream, const float* y, int T, int top, int
   if (T <= 0 || N <= 0) return MS_OK;
   if (stream == nullptr || y == nullptr || top < 1 || T > 65535 || (ids != nullptr && (weights == nullptr || x == nullptr || ldx < N)))
     return MS_BAD_ARG;
-  const dim3 grid((N + 255) / 256, T);
-  if (x_is_bf16) moe_combine_kernel<bf16><<<grid, 256, 0, st>>>(stream, y, top, N, ids, weights, (const bf16*)x, ldx, real, scale);
-  else moe_combine_kernel<float><<<grid, 256, 0, st>>>(stream, y, top, N, ids, weights, (const float*)x, ldx, real, scale);
+  const bool vec = N % 4 == 0 && (size_t)stream % 16 == 0 && (size_t)y % 16 == 0;
+  const int cols = vec ? 1024 : 256;
+  const dim3 grid((N + cols - 1) / cols, T);
+#define COMBINE(TX, V) moe_combine_kernel<TX, V><<<grid, 256, 0, st>>>(stream, y, top, N, ids, weights, (const TX*)x, ldx, real, scale)
+  if (x_is_bf16) { if (vec) COMBINE(bf16, 4); else COMBINE(bf16, 1); }
+  else { if (vec) COMBINE(float, 4); else COMBINE(float, 1); }
+#undef COMBINE
   return launch_status();
 }

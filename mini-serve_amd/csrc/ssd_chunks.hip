@@ -34,7 +34,7 @@ struct SsdArgs {
   float* out;   // [tokens, H E]
   float* U;     // [chunks, H, D E]
   float* total; // [chunks, H]: L_last
-  int rows, vec;
+  int rows, vec, HB;
 };
 
 __device__ __forceinline__ ssd_floatx4 ssd_mfma(float a, float b, ssd_floatx4 c) { return __builtin_amdgcn_mfma_f32_16x16x4f32(a, b, c, 0, 0, 0); }
@@ -52,10 +52,9 @@ __device__ __forceinline__ void ssd_find_chunk(const int* __restrict__ row_start
   *count = left < SSD_CHUNK ? left : SSD_CHUNK;
 }
 
-// The first wave: step sizes of the chunk's tokens (zero past its end) into d[], running sums of decay * d into L[].
+// One wave, one head: step sizes of the chunk's tokens (zero past its end) into d[], running sums of decay * d into L[].
 __device__ __forceinline__ void ssd_steps(const SsdArgs& a, int h, int first, int count, float* d, double* L) {
-  const int j = threadIdx.x;
-  if (j >= WAVE) return;
+  const int j = threadIdx.x % WAVE;
   float dj = 0.f;
   if (j < count) dj = softplus(a.step[(size_t)(first + j) * a.ld_step + h] + (a.step_bias ? a.step_bias[h] : 0.f));
   double run = (double)(a.decay[h] * dj);
@@ -66,6 +65,25 @@ __device__ __forceinline__ void ssd_steps(const SsdArgs& a, int h, int first, in
   }
   d[j] = dj;
   L[j] = run;
+}
+
+// What a wave of the first and third pass works on. A block owns one chunk and up to four heads that share their keys and
+// queries: with HB = 4 (2, 1) heads a block, wave w has head w % HB and every 4 / HB-th run of 16 value columns from w / HB on.
+struct SsdWork {
+  int group, h, run0, run_step, first, count;
+  bool live;
+};
+__device__ __forceinline__ SsdWork ssd_work(const SsdArgs& a) {
+  SsdWork k;
+  const int wave = threadIdx.x / WAVE, sets = (a.share + a.HB - 1) / a.HB;
+  k.group = blockIdx.y / sets;
+  const int in_group = (blockIdx.y % sets) * a.HB + wave % a.HB;
+  k.live = in_group < a.share;
+  k.h = k.group * a.share + (k.live ? in_group : 0);
+  k.run0 = wave / a.HB;
+  k.run_step = 4 / a.HB;
+  ssd_find_chunk(a.row_start, a.rows, blockIdx.x, &k.first, &k.count);
+  return k;
 }
 
 // Rows first .. first + count - 1, columns col .. col + n - 1 of x into tile[row][column] (row stride ts); rows past count and
@@ -87,40 +105,63 @@ __device__ __forceinline__ void ssd_stage(const SsdArgs& a, int first, int count
   }
 }
 
-// Pass 1. A wave owns every fourth run of 16 state rows; the keys' fragment of a run serves all runs of 16 value columns.
-__global__ __launch_bounds__(256) void ssd_summary_kernel(SsdArgs a) {
+// Pass 1. The keys, which every head of the block reads, are staged in LDS; the values, weighted per token, stay in the
+// registers of their wave, four runs of 16 columns at a time.
+__global__ __launch_bounds__(256, 2) void ssd_summary_kernel(SsdArgs a) {
   extern __shared__ __attribute__((aligned(16))) float ssd_lds[];
-  __shared__ float d[SSD_CHUNK], wt[SSD_CHUNK];
-  __shared__ double L[SSD_CHUNK];
-  const int h = blockIdx.y, D = a.D, E = a.E, tid = threadIdx.x, wave = tid / WAVE, l16 = tid % 16, grp = (tid % WAVE) / 16;
-  const int DP = (D + 15) & ~15, EP = (E + 15) & ~15, ks = DP + 4, vs = EP + 4;
-  float* K = ssd_lds;               // [SSD_CHUNK][ks]
-  float* V = K + SSD_CHUNK * ks;    // [SSD_CHUNK][vs], times the tokens' weights
-  int first, count;
-  ssd_find_chunk(a.row_start, a.rows, blockIdx.x, &first, &count);
-  ssd_steps(a, h, first, count, d, L);
-  ssd_stage(a, first, count, a.k_off + (h / a.share) * D, D, DP, K, ks);
-  ssd_stage(a, first, count, a.v_off + h * E, E, EP, V, vs);
+  __shared__ float d[4][SSD_CHUNK];
+  __shared__ double L[4][SSD_CHUNK];
+  constexpr int KI = SSD_CHUNK / 4, RUNS = 4;  // KI: a lane's tokens, those from 4 (lane / 16) on of every 16
+  const SsdWork k = ssd_work(a);
+  const int D = a.D, E = a.E, h = k.h, first = k.first, count = k.count, wave = threadIdx.x / WAVE, l16 = threadIdx.x % 16, grp = (threadIdx.x % WAVE) / 16;
+  const int DP = (D + 15) & ~15, ks = DP + 4;
+  float* K = ssd_lds;  // [SSD_CHUNK][ks]
+  const float* vp = a.x + (size_t)first * a.ld + a.v_off + h * E;
+  float v[RUNS][KI];
+  // Columns past the last are read again and not stored; rows past the chunk's end, whose weights are zero, likewise.
+  auto load = [&](int run) __attribute__((always_inline)) {
+#pragma unroll
+    for (int u = 0; u < RUNS; ++u) {
+      const unsigned e = (unsigned)min((run + u * k.run_step) * 16 + l16, E - 1);
+#pragma unroll
+      for (int i = 0; i < KI; ++i) v[u][i] = vp[(unsigned)min((i / 4) * 16 + grp * 4 + i % 4, count - 1) * (unsigned)a.ld + e];
+    }
+  };
+  load(k.run0);
+  ssd_stage(a, first, count, a.k_off + k.group * D, D, DP, K, ks);
+  ssd_steps(a, h, first, count, d[wave], L[wave]);
   __syncthreads();
-  if (tid < SSD_CHUNK) wt[tid] = expf((float)(L[SSD_CHUNK - 1] - L[tid])) * d[tid];  // (tokens past the end add nothing to L)
-  if (tid == 0) a.total[(size_t)blockIdx.x * a.H + h] = (float)L[SSD_CHUNK - 1];
-  __syncthreads();
-  for (int i = tid; i < SSD_CHUNK * EP; i += 256) V[(i / EP) * vs + i % EP] *= wt[i / EP];
-  __syncthreads();
+  if (!k.live) return;
+  const double last = L[wave][SSD_CHUNK - 1];  // (tokens past the end add nothing)
+  if (k.run0 == 0 && threadIdx.x % WAVE == 0) a.total[(size_t)blockIdx.x * a.H + h] = (float)last;
   float* Uo = a.U + ((size_t)blockIdx.x * a.H + h) * D * E;
-  for (int nt = wave; nt * 16 < D; nt += 4) {
-    float kf[SSD_CHUNK / 4];
+  for (int run = k.run0; run * 16 < E; run += RUNS * k.run_step) {
+    if (run != k.run0) load(run);
 #pragma unroll
-    for (int i = 0; i < SSD_CHUNK / 4; ++i) kf[i] = K[((i / 4) * 16 + grp * 4 + i % 4) * ks + nt * 16 + l16];
-    for (int et = 0; et * 16 < E; ++et) {
-      ssd_floatx4 acc = {0.f, 0.f, 0.f, 0.f};
+    for (int i = 0; i < KI; ++i) {
+      const int j = (i / 4) * 16 + grp * 4 + i % 4;
+      const float w = expf((float)(last - L[wave][j])) * d[wave][j];
 #pragma unroll
-      for (int i = 0; i < SSD_CHUNK / 4; ++i) acc = ssd_mfma(kf[i], V[((i / 4) * 16 + grp * 4 + i % 4) * vs + et * 16 + l16], acc);
-      const int e = et * 16 + l16;
+      for (int u = 0; u < RUNS; ++u) v[u][i] *= w;
+    }
+    for (int n0 = 0; n0 < D; n0 += 16) {
+      ssd_floatx4 acc[RUNS];
 #pragma unroll
-      for (int r = 0; r < 4; ++r) {
-        const int n = nt * 16 + grp * 4 + r;
-        if (n < D && e < E) Uo[(size_t)n * E + e] = acc[r];
+      for (int u = 0; u < RUNS; ++u) acc[u] = ssd_floatx4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+      for (int i = 0; i < KI; ++i) {
+        const float kv = K[((i / 4) * 16 + grp * 4 + i % 4) * ks + n0 + l16];
+#pragma unroll
+        for (int u = 0; u < RUNS; ++u) acc[u] = ssd_mfma(kv, v[u][i], acc[u]);
+      }
+#pragma unroll
+      for (int u = 0; u < RUNS; ++u) {
+        const int e = (run + u * k.run_step) * 16 + l16;
+#pragma unroll
+        for (int r = 0; r < 4; ++r) {
+          const int n = n0 + grp * 4 + r;
+          if (n < D && e < E) Uo[(size_t)n * E + e] = acc[u][r];
+        }
       }
     }
   }
@@ -155,43 +196,38 @@ __global__ __launch_bounds__(256) void ssd_scan_kernel(SsdArgs a) {
   *Sg = S;
 }
 
-// Pass 3. Scores of the 16 x 16 tiles on and below the diagonal, shared among the waves, then every wave the outputs of
-// every fourth run of 16 value columns: the entry state's part and the weighted values', whose fragments of S0 and v are
-// read by this wave alone, straight from memory, and (its first run's) asked for before the scores. NK: runs of 16 keys'
-// elements, D padded to them with zeros. The weights take the keys' place in LDS.
+// Pass 3. The scores q . k of the 16 x 16 tiles on and below the diagonal are formed once for the block's heads (they take
+// the keys' place in LDS); from there on every wave works for itself: its head's weights P as operand fragments in registers,
+// then, for each of its runs of 16 value columns, the entry state's part and the weighted values'. The fragments of S0 and v
+// are read by this wave alone, straight from memory, those of the next run before the products of this one. NK: runs of 16
+// elements of a key, D padded to them with zeros.
 template <int NK>
-__global__ __launch_bounds__(256) void ssd_output_kernel(SsdArgs a) {
+__global__ __launch_bounds__(256, NK <= 8 ? 2 : 1) void ssd_output_kernel(SsdArgs a) {
   extern __shared__ __attribute__((aligned(16))) float ssd_lds[];
-  __shared__ float d[SSD_CHUNK], eL[SSD_CHUNK];
-  __shared__ double L[SSD_CHUNK];
-  constexpr int DP = NK * 16, ks = DP + 4, ps = SSD_CHUNK + 4;
-  const int h = blockIdx.y, D = a.D, E = a.E, tid = threadIdx.x, wave = tid / WAVE, l16 = tid % 16, grp = (tid % WAVE) / 16;
+  __shared__ float d[4][SSD_CHUNK];
+  __shared__ double L[4][SSD_CHUNK];
+  constexpr int DP = NK * 16, ks = DP + 4, ps = SSD_CHUNK + 4, KI = SSD_CHUNK / 4;
+  const SsdWork k = ssd_work(a);
+  const int D = a.D, E = a.E, h = k.h, first = k.first, count = k.count, wave = threadIdx.x / WAVE, l16 = threadIdx.x % 16, grp = (threadIdx.x % WAVE) / 16;
   float* Q = ssd_lds;             // [SSD_CHUNK][ks]
-  float* K = Q + SSD_CHUNK * ks;  // [SSD_CHUNK][ks], later P [SSD_CHUNK][ps]
-  float* P = K;
-  int first, count;
-  ssd_find_chunk(a.row_start, a.rows, blockIdx.x, &first, &count);
+  float* K = Q + SSD_CHUNK * ks;  // [SSD_CHUNK][ks], later the scores [SSD_CHUNK][ps]
+  float* G = K;
   const float* S0 = a.U + ((size_t)blockIdx.x * a.H + h) * D * E;
-  float s0[NK * 4], v[SSD_CHUNK / 4];
-  auto load_run = [&](int et) __attribute__((always_inline)) {
-    const int e = et * 16 + l16;
+  const float* vp = a.x + (size_t)first * a.ld + a.v_off + h * E;
+  // What lies past the last row or column is read from the last: it meets zeros (padded queries, masked weights) or is not stored.
+  float s0[NK * 4], v[KI];
+  auto load = [&](int run) __attribute__((always_inline)) {
+    const unsigned e = (unsigned)min(run * 16 + l16, E - 1);
 #pragma unroll
-    for (int i = 0; i < NK * 4; ++i) {
-      const int n = (i / 4) * 16 + grp * 4 + i % 4;
-      s0[i] = (n < D && e < E) ? S0[(size_t)n * E + e] : 0.f;
-    }
+    for (int i = 0; i < NK * 4; ++i) s0[i] = S0[(unsigned)min((i / 4) * 16 + grp * 4 + i % 4, D - 1) * (unsigned)E + e];
 #pragma unroll
-    for (int i = 0; i < SSD_CHUNK / 4; ++i) {
-      const int j = (i / 4) * 16 + grp * 4 + i % 4;
-      v[i] = (j < count && e < E) ? a.x[(size_t)(first + j) * a.ld + a.v_off + h * E + e] : 0.f;
-    }
+    for (int i = 0; i < KI; ++i) v[i] = vp[(unsigned)min((i / 4) * 16 + grp * 4 + i % 4, count - 1) * (unsigned)a.ld + e];
   };
-  if (wave * 16 < E) load_run(wave);
-  ssd_steps(a, h, first, count, d, L);
-  ssd_stage(a, first, count, a.q_off + (h / a.share) * D, D, DP, Q, ks);
-  ssd_stage(a, first, count, a.k_off + (h / a.share) * D, D, DP, K, ks);
+  load(k.run0);
+  ssd_stage(a, first, count, a.q_off + k.group * D, D, DP, Q, ks);
+  ssd_stage(a, first, count, a.k_off + k.group * D, D, DP, K, ks);
+  ssd_steps(a, h, first, count, d[wave], L[wave]);
   __syncthreads();
-  if (tid < SSD_CHUNK) eL[tid] = expf((float)L[tid]);
   // tile p of the ten on and below the diagonal: (0,0) (1,0) (1,1) (2,0) ...
   ssd_floatx4 sc[3];
 #pragma unroll
@@ -217,20 +253,41 @@ __global__ __launch_bounds__(256) void ssd_output_kernel(SsdArgs a) {
     const int p = wave + 4 * u;
     if (p >= 10) continue;
     const int ti = p >= 6 ? 3 : p >= 3 ? 2 : p >= 1 ? 1 : 0, tj = p - ti * (ti + 1) / 2;
-    const int j = tj * 16 + l16;
-    const float dj = d[j];
-    const double Lj = L[j];
 #pragma unroll
-    for (int r = 0; r < 4; ++r) {
-      const int t = ti * 16 + grp * 4 + r;
-      P[t * ps + j] = j <= t ? sc[u][r] * expf((float)(L[t] - Lj)) * dj : 0.f;
-    }
+    for (int r = 0; r < 4; ++r) G[(ti * 16 + grp * 4 + r) * ps + tj * 16 + l16] = sc[u][r];
   }
   __syncthreads();
+  if (!k.live) return;
+  float pf[10][4];  // the weights of tile (ti, tj): row ti 16 + lane % 16, columns tj 16 + 4 (lane / 16) ..
+#pragma unroll
+  for (int ti = 0; ti < 4; ++ti) {
+    const int t = ti * 16 + l16;
+    const double Lt = L[wave][t];
+#pragma unroll
+    for (int tj = 0; tj <= ti; ++tj) {
+      const int j = tj * 16 + grp * 4;
+      const float4 g = *reinterpret_cast<const float4*>(G + t * ps + j);
+      const float gv[4] = {g.x, g.y, g.z, g.w};
+#pragma unroll
+      for (int c = 0; c < 4; ++c)
+        pf[ti * (ti + 1) / 2 + tj][c] = j + c <= t ? gv[c] * expf((float)(Lt - L[wave][j + c])) * d[wave][j + c] : 0.f;
+    }
+  }
+  float eL[4][4];
+#pragma unroll
+  for (int ti = 0; ti < 4; ++ti)
+#pragma unroll
+    for (int r = 0; r < 4; ++r) eL[ti][r] = expf((float)L[wave][ti * 16 + grp * 4 + r]);
   const float skip = a.skip[h];
-  for (int et = wave; et * 16 < E; et += 4) {
-    if (et != wave) load_run(et);
-    const int e = et * 16 + l16;
+#pragma unroll 1
+  for (int run = k.run0; run * 16 < E; run += k.run_step) {
+    float s1[NK * 4], w[KI];
+#pragma unroll
+    for (int i = 0; i < NK * 4; ++i) s1[i] = s0[i];
+#pragma unroll
+    for (int i = 0; i < KI; ++i) w[i] = v[i];
+    load(run + k.run_step);
+    const int e = run * 16 + l16;
 #pragma unroll
     for (int ti = 0; ti < 4; ++ti) {
       if (ti * 16 >= count) break;
@@ -239,26 +296,21 @@ __global__ __launch_bounds__(256) void ssd_output_kernel(SsdArgs a) {
 #pragma unroll
       for (int i = 0; i < NK; ++i) {
         const float4 qv = *reinterpret_cast<const float4*>(qr + i * 16);
-        acc = ssd_mfma(qv.x, s0[i * 4 + 0], acc);
-        acc = ssd_mfma(qv.y, s0[i * 4 + 1], acc);
-        acc = ssd_mfma(qv.z, s0[i * 4 + 2], acc);
-        acc = ssd_mfma(qv.w, s0[i * 4 + 3], acc);
+        acc = ssd_mfma(qv.x, s1[i * 4 + 0], acc);
+        acc = ssd_mfma(qv.y, s1[i * 4 + 1], acc);
+        acc = ssd_mfma(qv.z, s1[i * 4 + 2], acc);
+        acc = ssd_mfma(qv.w, s1[i * 4 + 3], acc);
       }
 #pragma unroll
-      for (int r = 0; r < 4; ++r) acc[r] *= eL[ti * 16 + grp * 4 + r];
-      const float* pr = P + (ti * 16 + l16) * ps + grp * 4;
+      for (int r = 0; r < 4; ++r) acc[r] *= eL[ti][r];
 #pragma unroll
-      for (int i = 0; i <= ti; ++i) {
-        const float4 pv = *reinterpret_cast<const float4*>(pr + i * 16);
-        acc = ssd_mfma(pv.x, v[i * 4 + 0], acc);
-        acc = ssd_mfma(pv.y, v[i * 4 + 1], acc);
-        acc = ssd_mfma(pv.z, v[i * 4 + 2], acc);
-        acc = ssd_mfma(pv.w, v[i * 4 + 3], acc);
-      }
+      for (int tj = 0; tj <= ti; ++tj)
+#pragma unroll
+        for (int c = 0; c < 4; ++c) acc = ssd_mfma(pf[ti * (ti + 1) / 2 + tj][c], w[tj * 4 + c], acc);
 #pragma unroll
       for (int r = 0; r < 4; ++r) {
         const int t = ti * 16 + grp * 4 + r;  // the value of token t and column e is the fragment element the lane holds
-        if (t < count && e < E) a.out[(size_t)(first + t) * ((size_t)a.H * E) + (size_t)h * E + e] = acc[r] + skip * v[ti * 4 + r];
+        if (t < count && e < E) a.out[(size_t)(first + t) * ((size_t)a.H * E) + (size_t)h * E + e] = acc[r] + skip * w[ti * 4 + r];
       }
     }
   }
@@ -282,18 +334,18 @@ extern "C" int ms_ssd_chunked(const float* x, int ld, int q_off, int k_off, int 
   if (D > SSD_MAX_DIM || E > SSD_MAX_DIM || H > 65535 || rows > 65535) return MS_UNSUPPORTED;
   const int vec = D % 4 == 0 && E % 4 == 0 && ld % 4 == 0 && q_off % 4 == 0 && k_off % 4 == 0 && v_off % 4 == 0 && (size_t)x % 16 == 0;
   SsdArgs a{x, ld, q_off, k_off, v_off, H, D, E, share, step, ld_step, step_bias, decay, skip, S, row_start, starts, state_slots,
-            out, U, total, rows, vec};
-  const int DP = (D + 15) & ~15, EP = (E + 15) & ~15;
-  const size_t lds1 = sizeof(float) * SSD_CHUNK * (size_t)(DP + 4 + EP + 4);
+            out, U, total, rows, vec, share >= 4 ? 4 : share >= 2 ? 2 : 1};
+  const int DP = (D + 15) & ~15;
   const int nk = DP <= 32 ? 2 : DP <= 64 ? 4 : DP <= 128 ? 8 : 16;
-  const size_t k_rows = (size_t)SSD_CHUNK * (nk * 16 + 4), p_rows = (size_t)SSD_CHUNK * (SSD_CHUNK + 4);
-  const size_t lds3 = sizeof(float) * (k_rows + (k_rows > p_rows ? k_rows : p_rows));
+  const size_t lds1 = sizeof(float) * SSD_CHUNK * (size_t)(DP + 4);
+  const int k_row = nk * 16 + 4, g_row = SSD_CHUNK + 4;
+  const size_t lds3 = sizeof(float) * SSD_CHUNK * (size_t)(k_row + (k_row > g_row ? k_row : g_row));
   const void* out_kernel = nk == 2 ? (const void*)ssd_output_kernel<2> : nk == 4 ? (const void*)ssd_output_kernel<4>
                          : nk == 8 ? (const void*)ssd_output_kernel<8> : (const void*)ssd_output_kernel<16>;
   if (hipFuncSetAttribute((const void*)ssd_summary_kernel, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds1) != hipSuccess ||
       hipFuncSetAttribute(out_kernel, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds3) != hipSuccess)
     return MS_LAUNCH_FAILED;
-  const dim3 per_chunk(chunks, H);
+  const dim3 per_chunk(chunks, H / share * ((share + a.HB - 1) / a.HB));
   ssd_summary_kernel<<<per_chunk, 256, lds1, st>>>(a);
   ssd_scan_kernel<<<dim3((D * E + 255) / 256, H, rows), 256, 0, st>>>(a);
   if (nk == 2) ssd_output_kernel<2><<<per_chunk, 256, lds3, st>>>(a);

@@ -44,7 +44,7 @@ _SIGNATURES = {
                        _c_void, _c_void, _c_void, _c_void, _c_void, _c_int, _c_int, _c_void, _c_void, _c_void],
     "ms_ssd_chunk_tokens": [],
     "ms_ssd_max_dim": [],
-    "ms_rglru": [_c_void, _c_int, _c_int, _c_int, _c_void, _c_void, _c_int, _c_void, _c_void, _c_void, _c_void, _c_void, _c_void, _c_int,
+    "ms_rglru": [_c_void, _c_int, _c_int, _c_int, _c_void, _c_void, _c_int, _c_void, _c_void, _c_void, _c_void, _c_void, _c_int,
                  _c_void, _c_void, _c_int, _c_void, _c_void, _c_void, _c_void, _c_int, _c_int, _c_int, _c_void, _c_void],
     "ms_rglru_chunk_tokens": [],
     "ms_rotate_columns": [_c_void, _c_int, _c_int, _c_int, _c_int, _c_int, _c_void, _c_int, _c_int, _c_float, _c_void],
@@ -1878,12 +1878,12 @@ def rglru(u: torch.Tensor, blocks: int, r_weight: torch.Tensor, i_weight: torch.
     lib = library()
     lens = getattr(batch, "row_lens", None)
     out = torch.empty((t, w), dtype=out_dtype, device=u.device)
-    a = x = total = None
+    ax = total = None
     chunks = 0
     if batch.is_decode and batch.num_rows == t:
         form = 0
     else:
-        a, x = (torch.empty((t, w), dtype=F32, device=u.device) for _ in range(2))
+        ax = torch.empty((t, w, 2), dtype=F32, device=u.device)
         form = 1
         if lens is not None and max(lens) >= RGLRU_CHUNKED_FROM:
             form = 2
@@ -1891,7 +1891,7 @@ def rglru(u: torch.Tensor, blocks: int, r_weight: torch.Tensor, i_weight: torch.
             chunks = sum(-(-n // per) for n in lens)
             total = torch.empty((chunks, 2, w), dtype=F32, device=u.device)
     _check(lib.ms_rglru(u.data_ptr(), t, w, blocks, r_weight.data_ptr(), i_weight.data_ptr(), int(r_weight.dtype == BF16), r_bias.data_ptr(),
-                        i_bias.data_ptr(), coef.data_ptr(), _ptr(a), _ptr(x), y.data_ptr() + 4 * y_col, y.shape[1], y_bias.data_ptr(),
+                        i_bias.data_ptr(), coef.data_ptr(), _ptr(ax), y.data_ptr() + 4 * y_col, y.shape[1], y_bias.data_ptr(),
                         out.data_ptr(), int(out_dtype == BF16), S.data_ptr(), batch.row_start.data_ptr(), batch.starts.data_ptr(),
                         batch.state_slots.data_ptr(), batch.num_rows, form, chunks, _ptr(total), _stream()), "rglru")
     return out
