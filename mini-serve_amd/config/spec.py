@@ -57,12 +57,14 @@ class RunEntry:
 
     A layer may appear in several entries (its weights are run twice); then each entry normally
     names a cache slot of its own. ``writes_cache=False`` lets an entry read the slot another
-    entry wrote instead of keeping keys and values of its own.
+    entry wrote instead of keeping keys and values of its own. ``before`` names a part (category
+    ``injection``) that adds something to the residual stream right before the entry's layer.
     """
 
     layer: int
     cache: int | None
     writes_cache: bool = True
+    before: PartSpec | None = None
 
 
 @dataclass(frozen=True)
@@ -95,3 +97,8 @@ class ModelSpec:
     def num_cache_slots(self) -> int:
         used = [e.cache for e in self.run_order if e.cache is not None]
         return max(used) + 1 if used else 0
+
+    @property
+    def injections(self) -> tuple[PartSpec, ...]:
+        """What the run order adds to the stream between layers."""
+        return tuple(e.before for e in self.run_order if e.before is not None)

@@ -76,6 +76,55 @@ __device__ __forceinline__ float sum_splits(const float* __restrict__ p, int spl
   return acc;
 }
 
+// acc += parts of splits s0 .. s0 + B - 1 (those below `splits`), four floats each, in ascending order;
+// the B loads are issued before the first sum.
+template <int B>
+__device__ __forceinline__ void add_splits(float4& acc, const float* __restrict__ p, int s0, int splits, size_t split_stride) {
+  float4 t[B];
+#pragma unroll
+  for (int u = 0; u < B; ++u) {
+    const bool in = s0 + u < splits;
+    t[u] = *reinterpret_cast<const float4*>(p + (size_t)(in ? s0 + u : 0) * split_stride);
+    if (!in) t[u] = make_float4(0.f, 0.f, 0.f, 0.f);
+  }
+#pragma unroll
+  for (int u = 0; u < B; ++u) {
+    acc.x += t[u].x; acc.y += t[u].y; acc.z += t[u].z; acc.w += t[u].w;
+  }
+}
+
+// Four consecutive weights in one load (w + i is aligned to four elements), kept as loaded: what uses
+// them comes after the block's sum, and a conversion right after the load would wait for it there.
+template <typename TW> struct Weights4;
+template <> struct Weights4<float> {
+  float4 v;
+  __device__ __forceinline__ void load(const float* w) { v = *reinterpret_cast<const float4*>(w); }
+  __device__ __forceinline__ float at(int e) const { return e == 0 ? v.x : e == 1 ? v.y : e == 2 ? v.z : v.w; }
+};
+template <> struct Weights4<bf16> {
+  union { uint2 u; bf16 e[4]; } v;
+  __device__ __forceinline__ void load(const bf16* w) { v.u = *reinterpret_cast<const uint2*>(w); }
+  __device__ __forceinline__ float at(int e) const { return to_f32(v.e[e]); }
+};
+
+// The sum of `splits` slices, four floats each, in ascending order. The loads of a batch of splits go out together; few
+// splits (a tile product's two to four) take a batch of their own size, so that no load is issued for nothing.
+__device__ __forceinline__ float4 add_splits4(const float* __restrict__ p, int splits, size_t split_stride) {
+  float4 acc = make_float4(0.f, 0.f, 0.f, 0.f);
+  if (splits == 1) {
+    add_splits<1>(acc, p, 0, splits, split_stride);
+  } else if (splits <= 2) {
+    add_splits<2>(acc, p, 0, splits, split_stride);
+  } else if (splits <= 4) {
+    add_splits<4>(acc, p, 0, splits, split_stride);
+  } else if (splits <= 8) {
+    add_splits<8>(acc, p, 0, splits, split_stride);
+  } else {  // the products of a decode step leave 12 to 16: one round trip, not two
+    for (int s0 = 0; s0 < splits; s0 += 16) add_splits<16>(acc, p, s0, splits, split_stride);
+  }
+  return acc;
+}
+
 // Which elements of a head make pair j of a rotary position encoding: (j, j + rot/2) or (2j, 2j + 1).
 #define MS_ROPE_HALVES 0
 #define MS_ROPE_ADJACENT 1

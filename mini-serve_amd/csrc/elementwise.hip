@@ -23,6 +23,105 @@ extern "C" int ms_embed(const int* ids, const void* table, int table_is_bf16, fl
   return launch_status();
 }
 
+// out[t, :] = scale * float(table[ids[t], :]) + float(pairs[r, :]), where the row r belongs to the token and the one before it
+// in its sequence: r = (previous * mul_prev + ids[t] * mul_cur) mod buckets, and r = buckets for a sequence's first token.
+// `pairs` may be nullptr (no such row). The token before a row's first one comes from the request's state, last[state_slots[row]];
+// the block that reads it leaves the row's last token there for the next step. `keep` (nullable) receives the same rows
+// once more. mul_prev and mul_cur lie in [0, buckets). One block per token.
+template <typename TW>
+__global__ __launch_bounds__(256) void embed_pairs_kernel(const int* __restrict__ ids, const TW* __restrict__ table, float scale,
+                                                          const TW* __restrict__ pairs, long long buckets, long long mul_prev,
+                                                          long long mul_cur, const int* __restrict__ positions,
+                                                          const int* __restrict__ token_row, const int* __restrict__ row_start,
+                                                          const int* __restrict__ state_slots, int* __restrict__ last,
+                                                          float* __restrict__ out, float* __restrict__ keep, int width) {
+  const int t = blockIdx.x;
+  const TW* src = table + (size_t)ids[t] * width;
+  const TW* pair = nullptr;
+  if (pairs != nullptr) {
+    const int row = token_row[t], first = row_start[row];
+    int* mine = last + state_slots[row];
+    long long r = buckets;
+    if (t > first || positions[t] > 0) {
+      const long long before = t > first ? ids[t - 1] : *mine;
+      r = (before * mul_prev + (long long)ids[t] * mul_cur) % buckets;
+    }
+    pair = pairs + (size_t)r * width;
+    if (t == first) {  // the same for the whole block
+      __syncthreads();  // every thread has read what the last step left
+      if (threadIdx.x == 0) *mine = ids[row_start[row + 1] - 1];
+    }
+  }
+  const size_t at = (size_t)t * width;
+  for (int i = threadIdx.x; i < width; i += 256) {
+    float v = to_f32(src[i]) * scale;
+    if (pair != nullptr) v += to_f32(pair[i]);
+    out[at + i] = v;
+    if (keep != nullptr) keep[at + i] = v;
+  }
+}
+
+extern "C" int ms_embed_pairs(const int* ids, const void* table, int is_bf16, float scale, const void* pairs, long long buckets,
+                              long long mul_prev, long long mul_cur, const int* positions, const int* token_row,
+                              const int* row_start, const int* state_slots, int* last, float* out, float* keep, int tokens,
+                              int width, hipStream_t st) {
+  if (tokens <= 0) return MS_OK;
+  if (width <= 0 || ids == nullptr || table == nullptr || out == nullptr ||
+      (pairs != nullptr && (buckets < 1 || buckets > 0x7fffffffLL || mul_prev < 0 || mul_prev >= buckets || mul_cur < 0 ||
+                            mul_cur >= buckets || positions == nullptr || token_row == nullptr || row_start == nullptr ||
+                            state_slots == nullptr || last == nullptr)))
+    return MS_BAD_ARG;
+#define EMB(TW) embed_pairs_kernel<TW><<<tokens, 256, 0, st>>>(ids, (const TW*)table, scale, (const TW*)pairs, buckets, mul_prev, mul_cur, positions, token_row, row_start, state_slots, last, out, keep, width)
+  if (is_bf16) EMB(bf16); else EMB(float);
+#undef EMB
+  return launch_status();
+}
+
+// ---------------------------------------------------------------------------------------------
+// x[t, :] += pending + start[t, :] + step[:]: what joins the stream ahead of a pass over a run of layers. pending are partial
+// sums (`splits` slices `stride` floats apart in ascending order, times `scale` [width] where it is given; parts may be
+// nullptr); start may be nullptr. A thread owns VEC consecutive columns of a token.
+template <int VEC>
+__global__ __launch_bounds__(256) void stream_inject_kernel(float* __restrict__ x, const float* __restrict__ parts, int splits,
+                                                            size_t stride, const float* __restrict__ scale,
+                                                            const float* __restrict__ start, const float* __restrict__ step, int width) {
+  struct alignas(4 * VEC) Columns { float e[VEC]; };
+  const int i = (blockIdx.x * 256 + threadIdx.x) * VEC;
+  if (i >= width) return;
+  const size_t at = (size_t)blockIdx.y * width + i;
+  Columns v = *reinterpret_cast<const Columns*>(x + at);
+  if (parts != nullptr) {
+    Columns p;
+    if constexpr (VEC == 4) {
+      const float4 q = add_splits4(parts + at, splits, stride);
+      p.e[0] = q.x; p.e[1] = q.y; p.e[2] = q.z; p.e[3] = q.w;
+    } else {
+      p.e[0] = sum_splits(parts + at, splits, stride);
+    }
+#pragma unroll
+    for (int e = 0; e < VEC; ++e) v.e[e] += scale != nullptr ? p.e[e] * scale[i + e] : p.e[e];
+  }
+#pragma unroll
+  for (int e = 0; e < VEC; ++e) {
+    if (start != nullptr) v.e[e] += start[at + e];
+    v.e[e] += step[i + e];
+  }
+  *reinterpret_cast<Columns*>(x + at) = v;
+}
+
+extern "C" int ms_stream_inject(float* x, const float* parts, int splits, long long stride, const float* scale, const float* start,
+                                const float* step, int tokens, int width, hipStream_t st) {
+  if (tokens <= 0) return MS_OK;
+  if (width <= 0 || tokens > 65535 || x == nullptr || step == nullptr ||
+      (parts != nullptr && (splits < 1 || (splits > 1 && stride < (long long)tokens * width))))
+    return MS_BAD_ARG;
+  const bool vec = width % 4 == 0 && (size_t)x % 16 == 0 && (size_t)parts % 16 == 0 && stride % 4 == 0;
+  const dim3 grid((width + (vec ? 1024 : 256) - 1) / (vec ? 1024 : 256), tokens);
+  if (vec) stream_inject_kernel<4><<<grid, 256, 0, st>>>(x, parts, splits, (size_t)stride, scale, start, step, width);
+  else stream_inject_kernel<1><<<grid, 256, 0, st>>>(x, parts, splits, (size_t)stride, scale, start, step, width);
+  return launch_status();
+}
+
 // ---------------------------------------------------------------------------------------------
 // Token ids that are still on the device: the last token of row i becomes src[feed[i]] where
 // feed[i] >= 0 (a token an earlier step sampled and the host has not read back yet). row_start holds
@@ -104,39 +203,8 @@ __global__ __launch_bounds__(NT) void rmsnorm_kernel(float* __restrict__ x, cons
 
 // The same for few rows of a width that is a multiple of 4 and at most 8 NT, bfloat16 output: NT
 // threads per row, a thread owns up to two groups of 4 consecutive elements and moves them as vectors;
-// the partial sums of up to 16 splits are fetched at a time. Sums per element in ascending split order, as
+// the partial sums of up to 16 splits are fetched at a time (add_splits4). Sums per element in ascending split order, as
 // in the kernel above.
-// acc += parts of splits s0 .. s0 + B - 1 (those below `splits`), four floats each, in ascending order;
-// the B loads are issued before the first sum.
-template <int B>
-__device__ __forceinline__ void add_splits(float4& acc, const float* __restrict__ p, int s0, int splits, size_t split_stride) {
-  float4 t[B];
-#pragma unroll
-  for (int u = 0; u < B; ++u) {
-    const bool in = s0 + u < splits;
-    t[u] = *reinterpret_cast<const float4*>(p + (size_t)(in ? s0 + u : 0) * split_stride);
-    if (!in) t[u] = make_float4(0.f, 0.f, 0.f, 0.f);
-  }
-#pragma unroll
-  for (int u = 0; u < B; ++u) {
-    acc.x += t[u].x; acc.y += t[u].y; acc.z += t[u].z; acc.w += t[u].w;
-  }
-}
-
-// Four consecutive weights in one load (w + i is aligned to four elements), kept as loaded: what uses
-// them comes after the block's sum, and a conversion right after the load would wait for it there.
-template <typename TW> struct Weights4;
-template <> struct Weights4<float> {
-  float4 v;
-  __device__ __forceinline__ void load(const float* w) { v = *reinterpret_cast<const float4*>(w); }
-  __device__ __forceinline__ float at(int e) const { return e == 0 ? v.x : e == 1 ? v.y : e == 2 ? v.z : v.w; }
-};
-template <> struct Weights4<bf16> {
-  union { uint2 u; bf16 e[4]; } v;
-  __device__ __forceinline__ void load(const bf16* w) { v.u = *reinterpret_cast<const uint2*>(w); }
-  __device__ __forceinline__ float at(int e) const { return to_f32(v.e[e]); }
-};
-
 template <typename TW, int NT>
 __global__ __launch_bounds__(NT) void rmsnorm_vec4_kernel(float* __restrict__ x, const TW* __restrict__ w,
                                                             bf16* __restrict__ y, const int* __restrict__ rows, int width,
@@ -158,21 +226,7 @@ __global__ __launch_bounds__(NT) void rmsnorm_vec4_kernel(float* __restrict__ x,
       wk[j].load(w + i);
       v = *reinterpret_cast<const float4*>(src + i);
       if (parts != nullptr) {
-        const float* p = parts + row * width + i;
-        float4 acc = make_float4(0.f, 0.f, 0.f, 0.f);
-        // The loads of a batch of splits go out together; few splits (a tile product's two to four) take
-        // a batch of their own size, so that no load is issued for nothing. Ascending split order always.
-        if (splits == 1) {
-          add_splits<1>(acc, p, 0, splits, split_stride);
-        } else if (splits <= 2) {
-          add_splits<2>(acc, p, 0, splits, split_stride);
-        } else if (splits <= 4) {
-          add_splits<4>(acc, p, 0, splits, split_stride);
-        } else if (splits <= 8) {
-          add_splits<8>(acc, p, 0, splits, split_stride);
-        } else {  // the products of a decode step leave 12 to 16: one round trip, not two
-          for (int s0 = 0; s0 < splits; s0 += 16) add_splits<16>(acc, p, s0, splits, split_stride);
-        }
+        float4 acc = add_splits4(parts + row * width + i, splits, split_stride);
         if (scale != nullptr) {
           const float4 s = *reinterpret_cast<const float4*>(scale + i);
           acc.x *= s.x; acc.y *= s.y; acc.z *= s.z; acc.w *= s.w;

@@ -78,7 +78,8 @@ extern "C" int ms_moe_route(const float* logits, int ld, int splits, long long s
 // ---------------------------------------------------------------------------------------------
 // Routing by scores: s = softmax(logits[t]) over all E outputs, or, `sigmoid`, s = 1 / (1 + exp(-logits[t])) each on its own;
 // the choice is made by c = s + correction (correction may be absent; sigmoid scores without one are chosen by their logits,
-// which are in the same order and do not saturate), the weights are the chosen outputs' s as they stand (not renormalised). With groups > 1 the E outputs form
+// which are in the same order and do not saturate), the weights are the chosen outputs' s, as they stand or, `renorm`, divided by their sum
+// (+ 1e-20), times `factor`. With groups > 1 the E outputs form
 // `groups` equal groups of neighbours, a group's score is its largest c, and only outputs of the `keep` best groups
 // (ties: the lower group) can be chosen: the others' c counts as minus infinity. The `top` largest c are chosen, largest
 // first (ties: the lower index). One wave per token; s and c of a token pass through the wave's own rows of LDS.
@@ -86,8 +87,8 @@ extern "C" int ms_moe_route(const float* logits, int ld, int splits, long long s
 template <typename TB, int PER>
 __global__ __launch_bounds__(256) void moe_route_scored_kernel(const float* __restrict__ logits, int ld, int splits, size_t stride,
                                                                const TB* __restrict__ correction, int T, int E, int top,
-                                                               int groups, int keep, int sigmoid, int* __restrict__ ids,
-                                                               float* __restrict__ weights) {
+                                                               int groups, int keep, int sigmoid, int renorm, float factor,
+                                                               int* __restrict__ ids, float* __restrict__ weights) {
   __shared__ float ss[4][PER * WAVE], cs[4][PER * WAVE];
   const int wave = threadIdx.x / WAVE, lane = threadIdx.x % WAVE;
   const int t = blockIdx.x * 4 + wave;
@@ -163,6 +164,7 @@ __global__ __launch_bounds__(256) void moe_route_scored_kernel(const float* __re
     __syncthreads();
   }
   if (!live) return;
+  float chosen = 0.f, total = 0.f;  // lane j keeps the j-th chosen score; their sum in the order of the choices
   for (int j = 0; j < top; ++j) {
     float best = -INFINITY;
     int at = 0x7fffffff;
@@ -179,23 +181,24 @@ __global__ __launch_bounds__(256) void moe_route_scored_kernel(const float* __re
 #pragma unroll
     for (int i = 0; i < PER; ++i)
       if (lane + i * WAVE == at) c[i] = -INFINITY;
-    if (lane == 0) {
-      ids[(size_t)t * top + j] = at;
-      weights[(size_t)t * top + j] = ss[wave][at];
-    }
+    const float sc = ss[wave][at];
+    total += sc;
+    if (lane == j) chosen = sc;
+    if (lane == 0) ids[(size_t)t * top + j] = at;
   }
+  if (lane < top) weights[(size_t)t * top + lane] = (renorm ? chosen / (total + 1e-20f) : chosen) * factor;
 }
 
 extern "C" int ms_moe_route_scored(const float* logits, int ld, int splits, long long stride, const void* correction,
-                                   int correction_is_bf16, int T, int E, int top, int groups, int keep, int sigmoid, int* ids,
-                                   float* weights, hipStream_t st) {
+                                   int correction_is_bf16, int T, int E, int top, int groups, int keep, int sigmoid, int renorm,
+                                   float factor, int* ids, float* weights, hipStream_t st) {
   if (T <= 0) return MS_OK;
   if (logits == nullptr || ids == nullptr || weights == nullptr || E < 1 || top < 1 || top > E || ld < E || splits < 1 ||
       (splits > 1 && stride < (long long)T * ld) || groups < 1 || E % groups || keep < 1 || keep > groups)
     return MS_BAD_ARG;
   if (E > MOE_MAX_EXPERTS || top > MOE_MAX_TOP) return MS_UNSUPPORTED;
   const unsigned blocks = (unsigned)((T + 3) / 4);
-#define ROUTE(TB, PER) moe_route_scored_kernel<TB, PER><<<blocks, 256, 0, st>>>(logits, ld, splits, (size_t)stride, (const TB*)correction, T, E, top, groups, keep, sigmoid, ids, weights)
+#define ROUTE(TB, PER) moe_route_scored_kernel<TB, PER><<<blocks, 256, 0, st>>>(logits, ld, splits, (size_t)stride, (const TB*)correction, T, E, top, groups, keep, sigmoid, renorm, factor, ids, weights)
 #define ROUTE_PER(TB) do { if (E <= WAVE) ROUTE(TB, 1); else if (E <= 2 * WAVE) ROUTE(TB, 2); else ROUTE(TB, MOE_MAX_EXPERTS / WAVE); } while (0)
   if (correction_is_bf16) ROUTE_PER(bf16); else ROUTE_PER(float);
 #undef ROUTE_PER
@@ -278,7 +281,7 @@ extern "C" int ms_moe_plan(const int* ids, int P, int E, int tile_rows, int max_
 // where every chosen expert has a tile of its own and its weights are streamed once; the fewer tiles the step can have,
 // the narrower the waves' runs of columns, so that the chip still gets waves enough to stream with).
 //   MODE 1 (gated): rows are x[token of the pair] (K = the model's width), two weights per expert, gate and up [E, N, K];
-//          the result act(gate) * up goes to h[sorted place][N] in the compute type.
+//          the result act(gate) * up (or what an activation with a limit makes of the two) goes to h[sorted place][N] in the compute type.
 //   MODE 2 (plain first product): the same rows, one weight per expert; act(up) goes to h[sorted place][N].
 //   MODE 0: rows are h[sorted place] (K = the experts' width), one weight per expert [E, N, K]; the result times the pair's
 //          routing weight goes to y[pair][N] in float32.
@@ -306,7 +309,7 @@ template <int MODE, bool ALIGNED, int NT, bool KSPLIT = false>
 __global__ __launch_bounds__(256) void moe_gemm_bf16_kernel(
     const bf16* __restrict__ a, int lda, const bf16* __restrict__ w1, const bf16* __restrict__ w2, void* __restrict__ out,
     const int* __restrict__ order, const int* __restrict__ tile_expert, const int* __restrict__ tile_start,
-    const int* __restrict__ tile_count, const float* __restrict__ pair_weight, int top, int N, int K, int tile_rows, int act) {
+    const int* __restrict__ tile_count, const float* __restrict__ pair_weight, int top, int N, int K, int tile_rows, int act, float limit) {
   constexpr bool GATED = MODE == 1, FIRST = MODE != 0;
   const int count = tile_count[blockIdx.x];
   if (count == 0) return;
@@ -394,7 +397,7 @@ __global__ __launch_bounds__(256) void moe_gemm_bf16_kernel(
       bf16* o = (bf16*)out + (size_t)(start + m) * N + n0 + l16;
 #pragma unroll
       for (int nt = 0; nt < NT; ++nt)
-        if (col_ok[nt]) o[nt * 16] = static_cast<bf16>(gated_value(acc1[nt][r] * pw, acc2[nt][r] * pw, act, 0.f));
+        if (col_ok[nt]) o[nt * 16] = static_cast<bf16>(gated_value(acc1[nt][r] * pw, acc2[nt][r] * pw, act, limit));
     } else if (FIRST) {
       bf16* o = (bf16*)out + (size_t)(start + m) * N + n0 + l16;
 #pragma unroll
@@ -427,7 +430,7 @@ template <int MODE, int BM, int WR, int WC>
 __global__ __launch_bounds__(256, 2) void moe_gemm_bf16_lds_kernel(
     const bf16* __restrict__ a, int lda, const bf16* __restrict__ w1, const bf16* __restrict__ w2, void* __restrict__ out,
     const int* __restrict__ order, const int* __restrict__ tile_expert, const int* __restrict__ tile_start,
-    const int* __restrict__ tile_count, const float* __restrict__ pair_weight, int top, int N, int K, int act) {
+    const int* __restrict__ tile_count, const float* __restrict__ pair_weight, int top, int N, int K, int act, float limit) {
   constexpr bool GATED = MODE == 1, FIRST = MODE != 0;
   static_assert(WR * WC == 4, "four waves a block");
   constexpr int BN = 128, KS = 64, STAGES = 2;
@@ -529,7 +532,7 @@ __global__ __launch_bounds__(256, 2) void moe_gemm_bf16_lds_kernel(
         const int col = n0 + wn / 2 + (i / 2) * 16 + g * 4;
         union { uint2 u; bf16 v[4]; } q;
 #pragma unroll
-        for (int c = 0; c < 4; ++c) q.v[c] = static_cast<bf16>(gated_value(acc[i][j][c] * pw, acc[i + 1][j][c] * pw, act, 0.f));
+        for (int c = 0; c < 4; ++c) q.v[c] = static_cast<bf16>(gated_value(acc[i][j][c] * pw, acc[i + 1][j][c] * pw, act, limit));
         if (vec && col + 3 < N) *reinterpret_cast<uint2*>(o + col) = q.u;
         else
 #pragma unroll
@@ -568,7 +571,7 @@ __global__ __launch_bounds__(256, 2) void moe_gemm_bf16_lds_kernel(
 template <int MODE, int BM, int WR, int WC>
 static int moe_launch_lds(const void* a, int lda, const void* w1, const void* w2, void* out, const int* order, const int* tile_expert,
                           const int* tile_start, const int* tile_count, const float* pair_weight, int max_tiles, int top, int N,
-                          int K, int act, hipStream_t st) {
+                          int K, int act, float limit, hipStream_t st) {
   constexpr int lds_bytes = 2 * (BM + 128) * 128;
   static bool ready = false;  // more than 48 KB of LDS is asked for once per kernel
   if (!ready) {
@@ -581,7 +584,7 @@ static int moe_launch_lds(const void* a, int lda, const void* w1, const void* w2
   const dim3 grid((N + cols - 1) / cols, max_tiles);
   if (grid.y > 65535) return MS_BAD_ARG;
   moe_gemm_bf16_lds_kernel<MODE, BM, WR, WC><<<grid, 256, lds_bytes, st>>>((const bf16*)a, lda, (const bf16*)w1, (const bf16*)w2, out, order,
-                                                                           tile_expert, tile_start, tile_count, pair_weight, top, N, K, act);
+                                                                           tile_expert, tile_start, tile_count, pair_weight, top, N, K, act, limit);
   return launch_status();
 }
 
@@ -591,7 +594,7 @@ template <int MODE>
 __global__ __launch_bounds__(256) void moe_gemm_f32_kernel(
     const float* __restrict__ a, int lda, const float* __restrict__ w1, const float* __restrict__ w2, float* __restrict__ out,
     const int* __restrict__ order, const int* __restrict__ tile_expert, const int* __restrict__ tile_start,
-    const int* __restrict__ tile_count, const float* __restrict__ pair_weight, int top, int N, int K, int act) {
+    const int* __restrict__ tile_count, const float* __restrict__ pair_weight, int top, int N, int K, int act, float limit) {
   constexpr bool GATED = MODE == 1, FIRST = MODE != 0;
   const int count = tile_count[blockIdx.x];
   if (count == 0) return;
@@ -658,7 +661,7 @@ __global__ __launch_bounds__(256) void moe_gemm_f32_kernel(
     for (int j = 0; j < 4; ++j) {
       const int n = n0 + tx * 4 + j;
       if (n >= N) continue;
-      if (GATED) out[(size_t)(start + m) * N + n] = gated_value(acc1[i][j] * pw, acc2[i][j] * pw, act, 0.f);
+      if (GATED) out[(size_t)(start + m) * N + n] = gated_value(acc1[i][j] * pw, acc2[i][j] * pw, act, limit);
       else if (FIRST) out[(size_t)(start + m) * N + n] = activate(acc1[i][j] * pw, act);
       else out[(size_t)pair * N + n] = acc1[i][j] * pw;
     }
@@ -671,18 +674,19 @@ __global__ __launch_bounds__(256) void moe_gemm_f32_kernel(
 // rows), 64 in float32.
 extern "C" int ms_moe_gemm(const void* a, int lda, const void* w1, const void* w2, void* out, int is_bf16, int mode,
                            const int* order, const int* tile_expert, const int* tile_start, const int* tile_count,
-                           const float* pair_weight, int max_tiles, int top, int N, int K, int tile_rows, int act, hipStream_t st) {
+                           const float* pair_weight, int max_tiles, int top, int N, int K, int tile_rows, int act, float limit,
+                           hipStream_t st) {
   if (max_tiles <= 0 || N <= 0) return MS_OK;
   const bool gated = mode == 1;
   if (mode < 0 || mode > 2 || a == nullptr || w1 == nullptr || (gated && w2 == nullptr) || out == nullptr || order == nullptr ||
       tile_expert == nullptr || tile_start == nullptr || tile_count == nullptr || top < 1 ||
-      K <= 0 || lda < K || (gated && (act < 0 || act >= MS_ACT_COUNT)) || (mode == 2 && !ms_act_ungated_ok(act)))
+      K <= 0 || lda < K || (gated && (act < 0 || act >= MS_GATED_COUNT || (act == MS_ACT_SWIGLU_CLAMPED && !(limit > 0.f)))) || (mode == 2 && !ms_act_ungated_ok(act)))
     return MS_BAD_ARG;
   if (is_bf16) {
     if (tile_rows != 16 && tile_rows != 64 && tile_rows != 128) return MS_BAD_ARG;
     const bool rows16 = (size_t)a % 16 == 0 && (size_t)w1 % 16 == 0 && (!gated || (size_t)w2 % 16 == 0) && lda % 8 == 0;
     if (tile_rows >= 64 && K % 64 == 0 && rows16 && (mode != 0 || (size_t)out % 16 == 0)) {
-#define MOE_LDS(G, BM, WR, WC) moe_launch_lds<G, BM, WR, WC>(a, lda, w1, w2, out, order, tile_expert, tile_start, tile_count, pair_weight, max_tiles, top, N, K, act, st)
+#define MOE_LDS(G, BM, WR, WC) moe_launch_lds<G, BM, WR, WC>(a, lda, w1, w2, out, order, tile_expert, tile_start, tile_count, pair_weight, max_tiles, top, N, K, act, limit, st)
       if (tile_rows == 128) return mode == 1 ? MOE_LDS(1, 128, 2, 2) : (mode == 2 ? MOE_LDS(2, 128, 2, 2) : MOE_LDS(0, 128, 2, 2));
       return mode == 1 ? MOE_LDS(1, 64, 1, 4) : (mode == 2 ? MOE_LDS(2, 64, 1, 4) : MOE_LDS(0, 64, 1, 4));
 #undef MOE_LDS
@@ -696,7 +700,7 @@ extern "C" int ms_moe_gemm(const void* a, int lda, const void* w1, const void* w
       while (nt > 1 && busy * ((N + 64 * nt - 1) / (64 * nt)) < 1024) nt /= 2;
     }
     const bool aligned = K % 8 == 0 && lda % 8 == 0 && (size_t)a % 16 == 0 && (size_t)w1 % 16 == 0 && (!gated || (size_t)w2 % 16 == 0);
-#define MOE_ARGS (const bf16*)a, lda, (const bf16*)w1, (const bf16*)w2, out, order, tile_expert, tile_start, tile_count, pair_weight, top, N, K, tile_rows, act
+#define MOE_ARGS (const bf16*)a, lda, (const bf16*)w1, (const bf16*)w2, out, order, tile_expert, tile_start, tile_count, pair_weight, top, N, K, tile_rows, act, limit
     // still few blocks at the narrowest columns: the waves of a block share 16 columns and split K
     if (tile_rows == 16 && nt == 1 && aligned && K >= 512 && (max_tiles / 2 + 1) * ((N + 63) / 64) < 2048 && (N + 15) / 16 <= 65535) {
       const dim3 grid(max_tiles, (N + 15) / 16);
@@ -722,7 +726,7 @@ extern "C" int ms_moe_gemm(const void* a, int lda, const void* w1, const void* w
     if (tile_rows != 64) return MS_BAD_ARG;
     const dim3 grid(max_tiles, (N + 63) / 64);
     if (grid.y > 65535) return MS_BAD_ARG;
-#define MOE_F32(G) moe_gemm_f32_kernel<G><<<grid, 256, 0, st>>>((const float*)a, lda, (const float*)w1, (const float*)w2, (float*)out, order, tile_expert, tile_start, tile_count, pair_weight, top, N, K, act)
+#define MOE_F32(G) moe_gemm_f32_kernel<G><<<grid, 256, 0, st>>>((const float*)a, lda, (const float*)w1, (const float*)w2, (float*)out, order, tile_expert, tile_start, tile_count, pair_weight, top, N, K, act, limit)
     if (mode == 1) MOE_F32(1);
     else if (mode == 2) MOE_F32(2);
     else MOE_F32(0);
@@ -732,13 +736,26 @@ extern "C" int ms_moe_gemm(const void* a, int lda, const void* w1, const void* w
 }
 
 // ---------------------------------------------------------------------------------------------
-// stream[t][n] += scale[n] (where it is given) times the sum over j < top of y[t * top + j][n], in ascending j. With ids: a choice whose id is `real` or more is
-// an identity expert, and its term is weights[t * top + j] * x[t][n] (y holds nothing for it).
+// stream[t][n] += scale[n] (where it is given) times (the sum over j < top of y[t * top + j][n], in ascending j, plus the extra
+// term). With ids: a choice whose id is `real` or more is an identity expert, and its term is weights[t * top + j] * x[t][n] (y
+// holds nothing for it). The extra term (extra not nullptr) is what a feed-forward that every token runs put out, as
+// `extra_splits` partial sums extra_stride floats apart, [T, N] each, times sigmoid(z[t]) where z is given: one number per token,
+// the first column of rows z_ld apart that come as z_splits partial sums z_stride floats apart.
 // A thread owns VEC consecutive columns of a token.
+struct MoeExtra {
+  const float* sum;
+  int splits;
+  size_t stride;
+  const float* z;
+  int z_ld, z_splits;
+  size_t z_stride;
+};
+
 template <typename TX, int VEC>
 __global__ __launch_bounds__(256) void moe_combine_kernel(float* __restrict__ stream, const float* __restrict__ y, int top, int N,
                                                           const int* __restrict__ ids, const float* __restrict__ weights,
-                                                          const TX* __restrict__ x, int ldx, int real, const float* __restrict__ scale) {
+                                                          const TX* __restrict__ x, int ldx, int real, const float* __restrict__ scale,
+                                                          MoeExtra extra) {
   struct alignas(4 * VEC) Columns { float e[VEC]; };
   const int n = (blockIdx.x * blockDim.x + threadIdx.x) * VEC;
   if (n >= N) return;
@@ -758,6 +775,16 @@ __global__ __launch_bounds__(256) void moe_combine_kernel(float* __restrict__ st
       for (int i = 0; i < VEC; ++i) acc[i] += v.e[i];
     }
   }
+  if (extra.sum != nullptr) {
+    const float g = extra.z != nullptr ? 1.f / (1.f + expf(-sum_splits(extra.z + t * extra.z_ld, extra.z_splits, extra.z_stride))) : 1.f;
+    const float* p = extra.sum + t * N + n;
+    if constexpr (VEC == 4) {
+      const float4 v = add_splits4(p, extra.splits, extra.stride);
+      acc[0] += g * v.x; acc[1] += g * v.y; acc[2] += g * v.z; acc[3] += g * v.w;
+    } else {
+      acc[0] += g * sum_splits(p, extra.splits, extra.stride);
+    }
+  }
   Columns* s = reinterpret_cast<Columns*>(stream + t * N + n);
   Columns v = *s;
 #pragma unroll
@@ -766,14 +793,20 @@ __global__ __launch_bounds__(256) void moe_combine_kernel(float* __restrict__ st
 }
 
 extern "C" int ms_moe_combine(float* stream, const float* y, int T, int top, int N, const int* ids, const float* weights,
-                              const void* x, int x_is_bf16, int ldx, int real, const float* scale, hipStream_t st) {
+                              const void* x, int x_is_bf16, int ldx, int real, const float* scale, const float* extra,
+                              int extra_splits, long long extra_stride, const float* z, int z_ld, int z_splits, long long z_stride,
+                              hipStream_t st) {
   if (T <= 0 || N <= 0) return MS_OK;
-  if (stream == nullptr || y == nullptr || top < 1 || T > 65535 || (ids != nullptr && (weights == nullptr || x == nullptr || ldx < N)))
+  if (stream == nullptr || y == nullptr || top < 1 || T > 65535 || (ids != nullptr && (weights == nullptr || x == nullptr || ldx < N)) ||
+      (extra != nullptr && (extra_splits < 1 || (extra_splits > 1 && extra_stride < (long long)T * N))) ||
+      (z != nullptr && (extra == nullptr || z_ld < 1 || z_splits < 1 || (z_splits > 1 && z_stride < (long long)T * z_ld))))
     return MS_BAD_ARG;
-  const bool vec = N % 4 == 0 && (size_t)stream % 16 == 0 && (size_t)y % 16 == 0;
+  const bool vec = N % 4 == 0 && (size_t)stream % 16 == 0 && (size_t)y % 16 == 0 && (size_t)extra % 16 == 0 &&
+                   (extra == nullptr || extra_stride % 4 == 0);
   const int cols = vec ? 1024 : 256;
   const dim3 grid((N + cols - 1) / cols, T);
-#define COMBINE(TX, V) moe_combine_kernel<TX, V><<<grid, 256, 0, st>>>(stream, y, top, N, ids, weights, (const TX*)x, ldx, real, scale)
+  const MoeExtra ex{extra, extra_splits, (size_t)extra_stride, z, z_ld, z_splits, (size_t)z_stride};
+#define COMBINE(TX, V) moe_combine_kernel<TX, V><<<grid, 256, 0, st>>>(stream, y, top, N, ids, weights, (const TX*)x, ldx, real, scale, ex)
   if (x_is_bf16) { if (vec) COMBINE(bf16, 4); else COMBINE(bf16, 1); }
   else { if (vec) COMBINE(float, 4); else COMBINE(float, 1); }
 #undef COMBINE

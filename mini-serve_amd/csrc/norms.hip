@@ -1,34 +1,51 @@
 // Norms beyond the plain RMSNorm, all with float32 statistics and one rounding at the store:
-//   layer norm with weight and bias (optionally over a list of rows);
+//   layer norm with weight and bias (optionally over a list of rows, optionally with a pending sum);
 //   RMS norm over groups of a row, times a weight, times sigmoid(gate) (a gated output norm: one group per head,
 //   or one group for the whole row);
 //   the mean of several streams, each RMS-normed over the row with its own weight, added to the residual stream;
-//   a scale in place;
+//   a scale in place, a soft bound in place;
 //   RMS norm of the whole query projection and of the whole key projection of a token (before they are split into
 //   heads), rotation of part of every head, and the store of keys and values into the cache pages.
 #include "common.h"
 
 // ---------------------------------------------------------------------------------------------
 // y[r, :] = (x[row(r), :] - mean) * rsqrt(var + eps) * w + b, var = mean of squared deviations.
+// With `parts` (the partial sums of a matrix product that still has to be added to the residual stream: `splits` slices of
+// [rows_total, width], `stride` floats apart, added in ascending order, times `scale` [width] where it is given) a row is first
+// brought up to date; without a row list x is updated in place, with one x is left unchanged (a list may name a row twice).
 // One block per row. Mean first, then the deviations' squares: two passes over the row, of which a thread keeps
 // its first eight elements in registers. Sums per thread in ascending element order, then a fixed block order.
 template <typename TW, typename TO, int NT>
-__global__ __launch_bounds__(NT) void layernorm_kernel(const float* __restrict__ x, const TW* __restrict__ w,
+__global__ __launch_bounds__(NT) void layernorm_kernel(float* __restrict__ x, const TW* __restrict__ w,
                                                        const TW* __restrict__ b, TO* __restrict__ y,
-                                                       const int* __restrict__ rows, int width, float eps) {
+                                                       const int* __restrict__ rows, int width, float eps,
+                                                       const float* __restrict__ parts, int splits, size_t stride,
+                                                       const float* __restrict__ scale) {
   __shared__ float red[NT / WAVE];
   constexpr int KEEP = 8;  // elements a thread keeps in registers between the passes (wider rows are read again)
   const int r = blockIdx.x;
-  const float* xr = x + (size_t)(rows ? rows[r] : r) * width;
+  const size_t row = rows ? rows[r] : r;
+  float* xr = x + row * width;
+  const bool in_place = parts != nullptr && rows == nullptr;
+  auto pending = [&](int e) { return sum_splits(parts + row * width + e, splits, stride) * (scale ? scale[e] : 1.f); };
+  auto up_to_date = [&](int e) {  // the first pass: the stream with what is pending
+    float v = xr[e];
+    if (parts != nullptr) {
+      v += pending(e);
+      if (in_place) xr[e] = v;
+    }
+    return v;
+  };
+  auto again = [&](int e) { return parts != nullptr && !in_place ? xr[e] + pending(e) : xr[e]; };  // (in place: this thread's own update)
   float kept[KEEP];
   float s = 0.f;
 #pragma unroll
   for (int i = 0; i < KEEP; ++i) {
     const int e = threadIdx.x + i * NT;
-    kept[i] = e < width ? xr[e] : 0.f;
+    kept[i] = e < width ? up_to_date(e) : 0.f;
     s += kept[i];
   }
-  for (int e = threadIdx.x + KEEP * NT; e < width; e += NT) s += xr[e];
+  for (int e = threadIdx.x + KEEP * NT; e < width; e += NT) s += up_to_date(e);
   const float mean = block_sum<NT>(s, red) / (float)width;
   float v = 0.f;
 #pragma unroll
@@ -37,34 +54,101 @@ __global__ __launch_bounds__(NT) void layernorm_kernel(const float* __restrict__
     if (threadIdx.x + i * NT < width) v += d * d;
   }
   for (int e = threadIdx.x + KEEP * NT; e < width; e += NT) {
-    const float d = xr[e] - mean;
+    const float d = again(e) - mean;
     v += d * d;
   }
   const float rstd = 1.f / sqrtf(block_sum<NT>(v, red) / (float)width + eps);
   TO* yr = y + (size_t)r * width;
-#pragma unroll
-  for (int i = 0; i < KEEP; ++i) {
-    const int e = threadIdx.x + i * NT;
-    if (e < width) {
-      float o = (kept[i] - mean) * rstd * to_f32(w[e]);
-      if (b != nullptr) o += to_f32(b[e]);
-      yr[e] = from_f32<TO>(o);
-    }
-  }
-  for (int e = threadIdx.x + KEEP * NT; e < width; e += NT) {
-    float o = (xr[e] - mean) * rstd * to_f32(w[e]);
+  auto store = [&](float xe, int e) {
+    float o = (xe - mean) * rstd * to_f32(w[e]);
     if (b != nullptr) o += to_f32(b[e]);
     yr[e] = from_f32<TO>(o);
+  };
+#pragma unroll
+  for (int i = 0; i < KEEP; ++i)
+    if ((int)threadIdx.x + i * NT < width) store(kept[i], threadIdx.x + i * NT);
+  for (int e = threadIdx.x + KEEP * NT; e < width; e += NT) store(again(e), e);
+}
+
+// The same for widths that are multiples of 4 and at most 8 NT: a thread owns up to two groups of four consecutive elements
+// and moves them as vectors. The block's shape depends on the width alone, so a row's sums have one order in every step.
+template <typename TW, typename TO, int NT>
+__global__ __launch_bounds__(NT) void layernorm_vec4_kernel(float* __restrict__ x, const TW* __restrict__ w,
+                                                            const TW* __restrict__ b, TO* __restrict__ y,
+                                                            const int* __restrict__ rows, int width, float eps,
+                                                            const float* __restrict__ parts, int splits, size_t stride,
+                                                            const float* __restrict__ scale) {
+  __shared__ float red[NT / WAVE];
+  const int r = blockIdx.x;
+  const size_t row = rows ? rows[r] : r;
+  float* xr = x + row * width;
+  const bool in_place = parts != nullptr && rows == nullptr;
+  float4 kept[2];
+  Weights4<TW> wk[2], bk[2];  // asked for with the row: after the block's sums they would cost another wait
+  float s = 0.f;
+#pragma unroll
+  for (int j = 0; j < 2; ++j) {
+    const int i = (threadIdx.x + j * NT) * 4;
+    float4 v = make_float4(0.f, 0.f, 0.f, 0.f);
+    if (i < width) {
+      wk[j].load(w + i);
+      if (b != nullptr) bk[j].load(b + i);
+      v = *reinterpret_cast<const float4*>(xr + i);
+      if (parts != nullptr) {
+        float4 acc = add_splits4(parts + row * width + i, splits, stride);
+        if (scale != nullptr) {
+          const float4 m = *reinterpret_cast<const float4*>(scale + i);
+          acc.x *= m.x; acc.y *= m.y; acc.z *= m.z; acc.w *= m.w;
+        }
+        v.x += acc.x; v.y += acc.y; v.z += acc.z; v.w += acc.w;
+        if (in_place) *reinterpret_cast<float4*>(xr + i) = v;
+      }
+    }
+    kept[j] = v;
+    s += (v.x + v.y) + (v.z + v.w);
+  }
+  const float mean = block_sum<NT>(s, red) / (float)width;
+  float q = 0.f;
+#pragma unroll
+  for (int j = 0; j < 2; ++j) {
+    if ((int)(threadIdx.x + j * NT) * 4 >= width) continue;
+    float4& v = kept[j];
+    v.x -= mean; v.y -= mean; v.z -= mean; v.w -= mean;
+    q += (v.x * v.x + v.y * v.y) + (v.z * v.z + v.w * v.w);
+  }
+  const float rstd = 1.f / sqrtf(block_sum<NT>(q, red) / (float)width + eps);
+  TO* yr = y + (size_t)r * width;
+  struct alignas(4 * sizeof(TO)) Four { TO e[4]; };
+#pragma unroll
+  for (int j = 0; j < 2; ++j) {
+    const int i = (threadIdx.x + j * NT) * 4;
+    if (i >= width) continue;
+    const float d[4] = {kept[j].x, kept[j].y, kept[j].z, kept[j].w};
+    Four o;
+#pragma unroll
+    for (int e = 0; e < 4; ++e) {
+      float u = d[e] * rstd * wk[j].at(e);
+      if (b != nullptr) u += bk[j].at(e);
+      o.e[e] = from_f32<TO>(u);
+    }
+    *reinterpret_cast<Four*>(yr + i) = o;
   }
 }
 
-extern "C" int ms_layernorm(const float* x, const void* w, const void* b, int w_is_bf16, void* y, int y_is_bf16,
-                            const int* rows, int n_rows, int width, float eps, hipStream_t st) {
+extern "C" int ms_layernorm(float* x, const void* w, const void* b, int w_is_bf16, void* y, int y_is_bf16,
+                            const int* rows, int n_rows, int width, float eps, const float* parts, int splits, long long stride,
+                            const float* scale, hipStream_t st) {
   if (n_rows <= 0) return MS_OK;
-  if (width <= 0 || !(eps >= 0.f)) return MS_BAD_ARG;
-#define LN(TW, TO) layernorm_kernel<TW, TO, 256><<<n_rows, 256, 0, st>>>(x, (const TW*)w, (const TW*)b, (TO*)y, rows, width, eps)
-  if (w_is_bf16) { if (y_is_bf16) LN(bf16, bf16); else LN(bf16, float); }
-  else { if (y_is_bf16) LN(float, bf16); else LN(float, float); }
+  if (width <= 0 || !(eps >= 0.f) || (parts != nullptr && splits < 1)) return MS_BAD_ARG;
+  const bool vec = width % 4 == 0 && width <= 8192 && (size_t)x % 16 == 0 && (size_t)w % 16 == 0 && (size_t)b % 16 == 0 &&
+                   (parts == nullptr || ((size_t)parts % 16 == 0 && stride % 4 == 0 && (size_t)scale % 16 == 0));
+#define LN(TW, TO) layernorm_kernel<TW, TO, 256><<<n_rows, 256, 0, st>>>(x, (const TW*)w, (const TW*)b, (TO*)y, rows, width, eps, parts, splits, (size_t)stride, scale)
+#define LV(TW, TO, NT) layernorm_vec4_kernel<TW, TO, NT><<<n_rows, NT, 0, st>>>(x, (const TW*)w, (const TW*)b, (TO*)y, rows, width, eps, parts, splits, (size_t)stride, scale)
+#define LNV(TW, TO) do { if (!vec) LN(TW, TO); else if (width <= 2048) LV(TW, TO, 256); else LV(TW, TO, 1024); } while (0)
+  if (w_is_bf16) { if (y_is_bf16) LNV(bf16, bf16); else LNV(bf16, float); }
+  else { if (y_is_bf16) LNV(float, bf16); else LNV(float, float); }
+#undef LNV
+#undef LV
 #undef LN
   return launch_status();
 }
@@ -260,6 +344,19 @@ __global__ void scale_kernel(float* __restrict__ x, size_t n, float s) {
 extern "C" int ms_scale(float* x, long long n, float s, hipStream_t st) {
   if (n <= 0) return MS_OK;
   scale_kernel<<<(unsigned)((n + 255) / 256), 256, 0, st>>>(x, (size_t)n, s);
+  return launch_status();
+}
+
+// x = cap * tanh(x / cap), in place: every value stays inside (-cap, cap).
+__global__ void softcap_kernel(float* __restrict__ x, size_t n, float cap) {
+  const size_t i = (size_t)blockIdx.x * blockDim.x + threadIdx.x;
+  if (i < n) x[i] = cap * tanhf(x[i] / cap);
+}
+
+extern "C" int ms_softcap(float* x, long long n, float cap, hipStream_t st) {
+  if (n <= 0) return MS_OK;
+  if (!(cap > 0.f)) return MS_BAD_ARG;
+  softcap_kernel<<<(unsigned)((n + 255) / 256), 256, 0, st>>>(x, (size_t)n, cap);
   return launch_status();
 }
 

@@ -157,32 +157,42 @@ extern "C" int ms_map_difference_norm(const void* a, void* out, int in_is_bf16, 
 }
 
 // ---------------------------------------------------------------------------------------------
-// Latent attention, before the attention kernel. A token's projection row x [ld] (float32) holds, from q_col on, H
-// query heads of Dn plain and R rotated elements each, and, from kv_col on (kv_col < 0: this layer keeps nothing), C
-// latent elements and R elements of the one key part that every head shares.
+// Latent attention, before the attention kernel. Sources are float32 rows `ld` apart, which may come as `splits` partial sums
+// `stride` floats apart (a product over few rows leaves them so), added here in ascending order.
+//   q: H query heads of Dn plain and R rotated elements each (p == nullptr: no queries);
+//   kv: C latent elements and R elements of the one key part that every head shares (p == nullptr: nothing is kept);
+//   the kv rows may also hold, from dq on (nullptr: they do not), Q elements of a latent that the queries are made from.
 //   The first `rot` of the R elements are turned in pairs, (j, j + rot/2) or (2j, 2j + 1), by the angle whose cosine
 //   and sine are rope[t][j] and rope[t][rot/2 + j]; the rest pass.
 //   q_plain [tokens, H * Dn]: the plain query parts (a per-head matrix product takes them into the latent's space);
 //   q_full [tokens, H * (C + R)]: only the turned parts are written here, behind each head's C columns;
 //   cache row of the token's slot, [C + R]: the latent after its RMS norm (weight cw), then the turned key part;
 //   the normed latent once more as the token's value, transposed within the page ([pages, C, page_size]): the tokens of
-//   one element side by side, the order in which the matrix cores take the values.
-// One block per token.
+//   one element side by side, the order in which the matrix cores take the values;
+//   cq [tokens, Q]: the queries' latent after an RMS norm of its own (weight qw).
+// blockIdx.x: the token; blockIdx.y: q_blocks runs of the query's elements, then the cache row, then the queries' latent.
+struct LatentSource {
+  const float* p;
+  int ld, splits;
+  size_t stride;
+  __device__ __forceinline__ float at(size_t i) const { return splits == 1 ? p[i] : sum_splits(p + i, splits, stride); }
+};
+
 template <typename T, typename TW>
-__global__ __launch_bounds__(256) void latent_prepare_kernel(const float* __restrict__ x, int ld, int q_col, int kv_col,
+__global__ __launch_bounds__(256) void latent_prepare_kernel(LatentSource q, LatentSource kv, LatentSource dq, int Q,
                                                              const float* __restrict__ rope, int rot, int pairing,
-                                                             const TW* __restrict__ cw, float eps, T* __restrict__ q_plain,
-                                                             T* __restrict__ q_full, const int* __restrict__ slots,
-                                                             T* __restrict__ kc, T* __restrict__ vc, int page_size, int H, int Dn,
-                                                             int R, int C) {
+                                                             const TW* __restrict__ cw, const TW* __restrict__ qw, float eps,
+                                                             T* __restrict__ q_plain, T* __restrict__ q_full, T* __restrict__ cq,
+                                                             const int* __restrict__ slots, T* __restrict__ kc, T* __restrict__ vc,
+                                                             int page_size, int H, int Dn, int R, int C, int q_blocks) {
   __shared__ float red[256 / WAVE];
+  constexpr int KEEP = 4;  // elements of a latent a thread keeps between the two passes (wider ones are read again)
   const int t = blockIdx.x;
-  const float* row = x + (size_t)t * ld;
   const float* cs = rot > 0 ? rope + (size_t)t * rot : nullptr;
   const int half = rot / 2;
-  // element r of a turned part: its partner and the angle's index
-  auto turned = [&](const float* v, int r) -> float {
-    if (r >= rot) return v[r];
+  // element r of a turned part that begins at `base`
+  auto turned = [&](const LatentSource& src, size_t base, int r) -> float {
+    if (r >= rot) return src.at(base + r);
     int j, other;
     bool low;
     if (pairing == MS_ROPE_ADJACENT) {
@@ -191,43 +201,87 @@ __global__ __launch_bounds__(256) void latent_prepare_kernel(const float* __rest
       low = r < half, j = low ? r : r - half, other = low ? r + half : r - half;
     }
     const float c = cs[j], s = cs[half + j];
-    return low ? v[r] * c - v[other] * s : v[r] * c + v[other] * s;
+    const float v = src.at(base + r), o = src.at(base + other);
+    return low ? v * c - o * s : v * c + o * s;
   };
-  const float* qrow = row + q_col;
-  for (int i = threadIdx.x; i < H * (Dn + R); i += 256) {
-    const int h = i / (Dn + R), d = i % (Dn + R);
-    if (d < Dn) q_plain[(size_t)t * H * Dn + (size_t)h * Dn + d] = from_f32<T>(qrow[i]);
-    else q_full[(size_t)t * H * (C + R) + (size_t)h * (C + R) + C + (d - Dn)] = from_f32<T>(turned(qrow + (size_t)h * (Dn + R) + Dn, d - Dn));
+  int part = blockIdx.y;
+  if (part < q_blocks) {
+    const int n = H * (Dn + R), per = (n + q_blocks - 1) / q_blocks, end = min(n, (part + 1) * per);
+    const size_t row = (size_t)t * q.ld;
+    for (int i = part * per + threadIdx.x; i < end; i += 256) {
+      const int h = i / (Dn + R), d = i % (Dn + R);
+      if (d < Dn) q_plain[(size_t)t * H * Dn + (size_t)h * Dn + d] = from_f32<T>(q.at(row + i));
+      else q_full[(size_t)t * H * (C + R) + (size_t)h * (C + R) + C + (d - Dn)] = from_f32<T>(turned(q, row + (size_t)h * (Dn + R) + Dn, d - Dn));
+    }
+    return;
   }
-  if (kv_col < 0) return;
-  const float* kv = row + kv_col;
-  float ss = 0.f;
-  for (int j = threadIdx.x; j < C; j += 256) ss += kv[j] * kv[j];
-  const float r = 1.f / sqrtf(block_sum<256>(ss, red) / (float)C + eps);
-  const int slot = slots[t], page = slot / page_size, off = slot % page_size;
-  T* dst = kc + (size_t)slot * (C + R);
-  T* val = vc + (size_t)page * C * page_size + off;
-  for (int j = threadIdx.x; j < C; j += 256) {
-    const T c = from_f32<T>(kv[j] * r * to_f32(cw[j]));
-    dst[j] = c;
-    val[(size_t)j * page_size] = c;
+  part -= q_blocks;
+  // the RMS norm of n elements from `base` on, element j of the result handed to put(j, value)
+  auto normed = [&](const LatentSource& src, size_t base, int n, const TW* w, auto put) {
+    float kept[KEEP];
+    float ss = 0.f;
+#pragma unroll
+    for (int i = 0; i < KEEP; ++i) {
+      const int j = threadIdx.x + i * 256;
+      kept[i] = j < n ? src.at(base + j) : 0.f;
+      ss += kept[i] * kept[i];
+    }
+    for (int j = threadIdx.x + KEEP * 256; j < n; j += 256) {
+      const float v = src.at(base + j);
+      ss += v * v;
+    }
+    const float r = 1.f / sqrtf(block_sum<256>(ss, red) / (float)n + eps);
+#pragma unroll
+    for (int i = 0; i < KEEP; ++i) {
+      const int j = threadIdx.x + i * 256;
+      if (j < n) put(j, kept[i] * r * to_f32(w[j]));
+    }
+    for (int j = threadIdx.x + KEEP * 256; j < n; j += 256) put(j, src.at(base + j) * r * to_f32(w[j]));
+  };
+  if (kv.p != nullptr && part-- == 0) {
+    const size_t row = (size_t)t * kv.ld;
+    const int slot = slots[t], page = slot / page_size, off = slot % page_size;
+    T* dst = kc + (size_t)slot * (C + R);
+    T* val = vc + (size_t)page * C * page_size + off;
+    normed(kv, row, C, cw, [&](int j, float v) {
+      const T c = from_f32<T>(v);
+      dst[j] = c;
+      val[(size_t)j * page_size] = c;
+    });
+    for (int j = threadIdx.x; j < R; j += 256) dst[C + j] = from_f32<T>(turned(kv, row + C, j));
+    return;
   }
-  for (int j = threadIdx.x; j < R; j += 256) dst[C + j] = from_f32<T>(turned(kv + C, j));
+  normed(dq, (size_t)t * dq.ld, Q, qw, [&](int j, float v) { cq[(size_t)t * Q + j] = from_f32<T>(v); });
 }
 
-extern "C" int ms_latent_prepare(const float* x, int ld, int q_col, int kv_col, const float* rope, int rot, int pairing,
-                                 const void* cw, int w_is_bf16, float eps, void* q_plain, void* q_full, const int* slots,
-                                 void* kc, void* vc, int page_size, int out_is_bf16, int tokens, int H, int Dn, int R, int C,
-                                 hipStream_t st) {
+// q: the query rows, or nullptr; x: the rows that hold, from kv_col on (kv_col < 0: nothing is kept), a token's latent and shared
+// key part, and, from dq_col on (dq_col < 0: none), the Q elements of its queries' latent. x may be nullptr where neither is asked for.
+extern "C" int ms_latent_prepare(const float* q, int q_ld, int q_splits, long long q_stride, const float* x, int ld, int splits,
+                                 long long stride, int kv_col, int dq_col, int Q, const float* rope, int rot, int pairing,
+                                 const void* cw, const void* qw, int w_is_bf16, float eps, void* q_plain, void* q_full, void* cq,
+                                 const int* slots, void* kc, void* vc, int page_size, int out_is_bf16, int tokens, int H, int Dn,
+                                 int R, int C, hipStream_t st) {
   if (tokens <= 0) return MS_OK;
+  const bool keeps = kv_col >= 0, makes = dq_col >= 0;
   if (H <= 0 || Dn <= 0 || R < 0 || C <= 0 || rot < 0 || rot > R || rot % 2 || (rot > 0 && rope == nullptr) ||
-      (pairing != MS_ROPE_HALVES && pairing != MS_ROPE_ADJACENT) || q_col < 0 || ld < q_col + H * (Dn + R) ||
-      (kv_col >= 0 && (ld < kv_col + C + R || slots == nullptr || kc == nullptr || vc == nullptr || cw == nullptr || page_size < 1)) ||
-      !(eps >= 0.f))
+      (pairing != MS_ROPE_HALVES && pairing != MS_ROPE_ADJACENT) || (q == nullptr && !keeps && !makes) || !(eps >= 0.f))
     return MS_BAD_ARG;
+  if (q != nullptr && (q_ld < H * (Dn + R) || q_splits < 1 || q_plain == nullptr || q_full == nullptr ||
+                       (q_splits > 1 && q_stride < (long long)(tokens - 1) * q_ld + H * (Dn + R))))
+    return MS_BAD_ARG;
+  if ((keeps || makes) && (x == nullptr || splits < 1 || (splits > 1 && stride < (long long)tokens * ld))) return MS_BAD_ARG;
+  if (keeps && (ld < kv_col + C + R || slots == nullptr || kc == nullptr || vc == nullptr || cw == nullptr || page_size < 1)) return MS_BAD_ARG;
+  if (makes && (Q <= 0 || ld < dq_col + Q || qw == nullptr || cq == nullptr)) return MS_BAD_ARG;
+  // few tokens: runs of 512 query elements, so that more blocks share them
+  const int q_blocks = q == nullptr ? 0 : (tokens > 256 ? 1 : (H * (Dn + R) + 511) / 512);
+  if (q_blocks > 65533) return MS_BAD_ARG;
+  const LatentSource qs{q, q_ld, q_splits, (size_t)q_stride};
+  const LatentSource ks{keeps ? x + kv_col : nullptr, ld, splits, (size_t)stride};
+  const LatentSource ds{makes ? x + dq_col : nullptr, ld, splits, (size_t)stride};
+  const dim3 grid(tokens, q_blocks + keeps + makes);
 #define LP(T, TW)                                                                                                             \
-  latent_prepare_kernel<T, TW><<<tokens, 256, 0, st>>>(x, ld, q_col, kv_col, rope, rot, pairing, (const TW*)cw, eps, (T*)q_plain, \
-                                                       (T*)q_full, slots, (T*)kc, (T*)vc, page_size, H, Dn, R, C)
+  latent_prepare_kernel<T, TW><<<grid, 256, 0, st>>>(qs, ks, ds, Q, rope, rot, pairing, (const TW*)cw, (const TW*)qw, eps,      \
+                                                     (T*)q_plain, (T*)q_full, (T*)cq, slots, (T*)kc, (T*)vc, page_size, H, Dn, R, C, q_blocks)
   if (out_is_bf16) {
     if (w_is_bf16) LP(bf16, bf16); else LP(bf16, float);
   } else {

@@ -22,17 +22,22 @@ _ERRORS = {1: "bad argument", 2: "unsupported size", 3: "kernel launch failed"}
 
 _SIGNATURES = {
     "ms_embed": [_c_void, _c_void, _c_int, _c_void, _c_int, _c_int, _c_void],
+    "ms_embed_pairs": [_c_void, _c_void, _c_int, _c_float, _c_void, _c_ll, _c_ll, _c_ll, _c_void, _c_void, _c_void, _c_void, _c_void, _c_void,
+                       _c_void, _c_int, _c_int, _c_void],
+    "ms_stream_inject": [_c_void, _c_void, _c_int, _c_ll, _c_void, _c_void, _c_void, _c_int, _c_int, _c_void],
     "ms_feed_tokens": [_c_void, _c_void, _c_void, _c_void, _c_int, _c_int, _c_void],
     "ms_rmsnorm": [_c_void, _c_void, _c_int, _c_void, _c_int, _c_void, _c_int, _c_int, _c_float, _c_void, _c_int, _c_ll, _c_void, _c_void],
     "ms_act_mul": [_c_void, _c_void, _c_int, _c_int, _c_int, _c_int, _c_int, _c_float, _c_void],
     "ms_act_mul_parts": [_c_void, _c_int, _c_ll, _c_void, _c_int, _c_int, _c_int, _c_int, _c_int, _c_float, _c_void],
-    "ms_layernorm": [_c_void, _c_void, _c_void, _c_int, _c_void, _c_int, _c_void, _c_int, _c_int, _c_float, _c_void],
+    "ms_layernorm": [_c_void, _c_void, _c_void, _c_int, _c_void, _c_int, _c_void, _c_int, _c_int, _c_float, _c_void, _c_int, _c_ll,
+                     _c_void, _c_void],
     "ms_group_rmsnorm_gate": [_c_void, _c_void, _c_int, _c_void, _c_int, _c_void, _c_int, _c_int, _c_int, _c_int, _c_float, _c_int, _c_int,
                               _c_void],
     "ms_normed_mean_add": [_c_void, _c_void, _c_void, _c_int, _c_int, _c_int, _c_int, _c_float, _c_float, _c_void],
     "ms_normed_add_pending": [_c_void, _c_void, _c_void, _c_int, _c_ll, _c_void, _c_int, _c_int, _c_int, _c_float, _c_void, _c_int,
                               _c_void],
     "ms_scale": [_c_void, _c_ll, _c_float, _c_void],
+    "ms_softcap": [_c_void, _c_ll, _c_float, _c_void],
     "ms_qkv_norm_rope_store": [_c_void, _c_int, _c_void, _c_int, _c_void, _c_void, _c_void, _c_void, _c_int, _c_int, _c_float, _c_void,
                                _c_int, _c_int, _c_void, _c_void, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_void],
     "ms_gated_recurrence": [_c_void, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_float,
@@ -80,8 +85,9 @@ _SIGNATURES = {
                            _c_void, _c_float, _c_void, _c_void, _c_void, _c_void, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int,
                            _c_int, _c_int, _c_int, _c_void],
     "ms_map_difference_norm": [_c_void, _c_void, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_float, _c_float, _c_float, _c_void],
-    "ms_latent_prepare": [_c_void, _c_int, _c_int, _c_int, _c_void, _c_int, _c_int, _c_void, _c_int, _c_float, _c_void, _c_void,
-                          _c_void, _c_void, _c_void, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_void],
+    "ms_latent_prepare": [_c_void, _c_int, _c_int, _c_ll, _c_void, _c_int, _c_int, _c_ll, _c_int, _c_int, _c_int, _c_void, _c_int, _c_int,
+                          _c_void, _c_void, _c_int, _c_float, _c_void, _c_void, _c_void, _c_void, _c_void, _c_void, _c_int, _c_int,
+                          _c_int, _c_int, _c_int, _c_int, _c_int, _c_void],
     "ms_paged_attention_tiled_mfma_wide": [_c_void, _c_int, _c_void, _c_void, _c_void, _c_int, _c_void, _c_void, _c_int, _c_void, _c_void,
                                            _c_void, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_float, _c_int, _c_int, _c_float,
                                            _c_void, _c_int, _c_int, _c_void, _c_void, _c_void],
@@ -117,12 +123,13 @@ _SIGNATURES = {
                               _c_int, _c_void, _c_int, _c_float, _c_void, _c_void, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int,
                               _c_void],
     "ms_moe_route": [_c_void, _c_int, _c_int, _c_ll, _c_void, _c_int, _c_int, _c_int, _c_int, _c_void, _c_void, _c_void],
-    "ms_moe_route_scored": [_c_void, _c_int, _c_int, _c_ll, _c_void, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_void, _c_void,
-                            _c_void],
+    "ms_moe_route_scored": [_c_void, _c_int, _c_int, _c_ll, _c_void, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int,
+                            _c_float, _c_void, _c_void, _c_void],
     "ms_moe_plan": [_c_void, _c_int, _c_int, _c_int, _c_int, _c_void, _c_void, _c_void, _c_void, _c_void],
     "ms_moe_gemm": [_c_void, _c_int, _c_void, _c_void, _c_void, _c_int, _c_int, _c_void, _c_void, _c_void, _c_void, _c_void,
-                    _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_void],
-    "ms_moe_combine": [_c_void, _c_void, _c_int, _c_int, _c_int, _c_void, _c_void, _c_void, _c_int, _c_int, _c_int, _c_void, _c_void],
+                    _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_float, _c_void],
+    "ms_moe_combine": [_c_void, _c_void, _c_int, _c_int, _c_int, _c_void, _c_void, _c_void, _c_int, _c_int, _c_int, _c_void, _c_void,
+                       _c_int, _c_ll, _c_void, _c_int, _c_int, _c_ll, _c_void],
     "ms_measure_read": [_c_void, _c_ll, _c_int, _c_void, _c_void],
     "ms_measure_copy": [_c_void, _c_void, _c_ll, _c_int, _c_void],
 }
@@ -263,6 +270,60 @@ def embed(token_ids: torch.Tensor, table: torch.Tensor) -> torch.Tensor:
     return out
 
 
+def embed_pairs(token_ids: torch.Tensor, table: torch.Tensor, scale: float = 1.0, pairs: torch.Tensor | None = None, mul_prev: int = 0,
+                mul_cur: int = 0, batch=None, last: torch.Tensor | None = None, keep: bool = False):
+    """``scale * table[id]`` as float32 ``[T, width]``, plus, with ``pairs [n + 1, width]`` (the table's dtype), the row
+    ``(previous * mul_prev + id * mul_cur) mod n`` for the token before it in its sequence and row ``n`` for a sequence's first
+    token. ``last`` (int32 ``[slots, 1]``) is what the requests keep: the last token of the step before, replaced by
+    this step's. ``keep``: returns the result twice, as two tensors (one to add to, one that stays as it is)."""
+    _dev(token_ids, "token_ids", I32, 1)
+    _dev(table, "table", (F32, BF16), 2)
+    t, width = token_ids.shape[0], table.shape[1]
+    meta, n = (None,) * 5, 1
+    if pairs is not None:
+        _dev(pairs, "pairs", table.dtype, 2)
+        _dev(last, "last", I32, 2)
+        if pairs.shape[1] != width or pairs.shape[0] < 2 or last.shape[1] != 1:
+            raise ValueError(f"a pair table {tuple(pairs.shape)} for width {width}: one row per bucket and one for the first token")
+        n = pairs.shape[0] - 1
+        fields = (batch.positions, batch.token_row, batch.row_start, batch.state_slots)
+        for f in fields:
+            _dev(f, "the batch's fields", I32, 1)
+        if fields[0].shape[0] != t or fields[1].shape[0] != t or fields[2].shape[0] != fields[3].shape[0] + 1:
+            raise ValueError("batch metadata does not match the number of tokens or rows")
+        meta = (*(f.data_ptr() for f in fields), last.data_ptr())
+    out = torch.empty((t, width), dtype=F32, device=table.device)
+    copy = torch.empty_like(out) if keep else None
+    _check(library().ms_embed_pairs(token_ids.data_ptr(), table.data_ptr(), int(table.dtype == BF16), float(scale), _ptr(pairs), n,
+                                    int(mul_prev) % n, int(mul_cur) % n, *meta, out.data_ptr(), _ptr(copy), t, width, _stream()),
+           "embed_pairs")
+    return (out, copy) if keep else out
+
+
+def stream_inject(x: torch.Tensor, step: torch.Tensor, start: torch.Tensor | None = None, add: SplitSum | None = None) -> None:
+    """``x += add + start + step`` in place: float32 ``x [T, width]``, a pending sum, rows of the same shape and one vector
+    ``[width]`` for all rows."""
+    _dev(x, "x", F32, 2)
+    _dev(step, "step", F32, 1)
+    if step.shape[0] != x.shape[1]:
+        raise ValueError(f"a step of {step.shape[0]} elements for width {x.shape[1]}")
+    if start is not None:
+        _dev(start, "start", F32, 2)
+        if start.shape != x.shape:
+            raise ValueError("start must have the stream's shape")
+    parts, splits, stride, scale = _pending(add, x.shape)
+    _check(library().ms_stream_inject(x.data_ptr(), parts, splits, stride, scale, _ptr(start), step.data_ptr(), x.shape[0], x.shape[1],
+                                      _stream()), "stream_inject")
+
+
+def _pending(add: SplitSum | None, shape):
+    """A pending sum as kernels take it: pointer, number of partial sums, their distance, pointer of the scale."""
+    if add is None:
+        return None, 0, 0, None
+    _check_split(add, "add", shape)
+    return add.parts.data_ptr(), add.splits, add.stride, _ptr(add.scale)
+
+
 def feed_tokens(token_ids: torch.Tensor, row_start: torch.Tensor | None, feed: torch.Tensor, source: torch.Tensor) -> None:
     """In place: the last token of row ``i`` of ``token_ids`` becomes ``source[feed[i]]`` where
     ``feed[i] >= 0``. ``row_start``: ``rows + 1`` offsets of the rows in ``token_ids`` (None: one token
@@ -296,10 +357,7 @@ def rmsnorm(x: torch.Tensor, weight: torch.Tensor, eps: float, out_dtype, rows: 
     if rows is not None:
         _dev(rows, "rows", I32, 1)
         n = rows.shape[0]
-    parts, splits, stride, scale = None, 0, 0, None
-    if add is not None:
-        _check_split(add, "add", x.shape)
-        parts, splits, stride, scale = add.parts.data_ptr(), add.splits, add.stride, _ptr(add.scale)
+    parts, splits, stride, scale = _pending(add, x.shape)
     out = torch.empty((n, x.shape[1]), dtype=out_dtype, device=x.device)
     _check(library().ms_rmsnorm(x.data_ptr(), weight.data_ptr(), int(weight.dtype == BF16), out.data_ptr(),
                                 int(out_dtype == BF16), _ptr(rows), n, x.shape[1], float(eps), parts, splits, stride,
@@ -324,7 +382,7 @@ def interleave_gate_up(gate: torch.Tensor, up: torch.Tensor) -> torch.Tensor:
 # Activations of the gated feed-forward and the numbers the kernels know them by (MS_ACT_* in csrc/common.h):
 # silu(x) = x sigmoid(x); gelu_tanh(x) = x / 2 (1 + tanh(sqrt(2 / pi) (x + 0.044715 x^3))).
 # swiglu_clamped(gate, up) = g sigmoid(1.702 g) (u + 1) with g = min(gate, limit), u = clamp(up, -limit, limit): not of
-# the form act(gate) * up, it takes ``limit`` along and runs in the activation kernels (no matrix kernel's epilogue knows it).
+# the form act(gate) * up, it takes ``limit`` along.
 ACTIVATIONS = {"silu": 0, "gelu_tanh": 1, "swiglu_clamped": 2, "relu_squared": 3, "tanh": 4}
 ACTIVATIONS_UNGATED_ONLY = {"relu_squared", "tanh"}  # no kernel finishes act(gate) * up with these
 ACTIVATIONS_WITH_LIMIT = {"swiglu_clamped"}
@@ -505,13 +563,18 @@ def linear(x: torch.Tensor, weight: torch.Tensor, out_dtype=None, accumulate_int
     return None if accumulate_into is not None else res
 
 
+def linear_sum(x: torch.Tensor, weight: torch.Tensor) -> SplitSum:
+    """``x weight^T`` as partial sums (one of them, where the kernels leave no more)."""
+    res = linear(x, weight, out_dtype=F32, defer=True)
+    return res if isinstance(res, SplitSum) else SplitSum(res.view(1, *res.shape))
+
+
 def _linear_scaled(x, weight, residual, scale, defer: bool) -> SplitSum | None:
     m, n = x.shape[0], weight.shape[0]
     _dev(residual, "accumulate_into", F32, 2)
     if tuple(residual.shape) != (m, n):
         raise ValueError(f"linear: accumulator is {tuple(residual.shape)}, expected {(m, n)}")
-    res = linear(x, weight, out_dtype=F32, defer=True)
-    pending = SplitSum(res.parts if isinstance(res, SplitSum) else res.view(1, m, n), scale)
+    pending = SplitSum(linear_sum(x, weight).parts, scale)
     if defer:
         return pending
     add_pending(residual, pending)
@@ -546,8 +609,9 @@ MOE_SMALL_TILE_PAIRS = 16  # (token, expert) pairs per expert, on average, up to
 MOE_LARGE_TILE_PAIRS = 128  # ... and from which it runs 128-pair tiles (widths that are multiples of 64)
 
 
-def moe_route(logits, bias: torch.Tensor | None, top: int, scoring: str = "chosen_softmax", groups: int = 1, keep: int = 1):
-    """Per row of the float32 router logits ``[T, E]``: the ``top`` chosen outputs, best first (ties: the lower index), as
+def moe_route(logits, bias: torch.Tensor | None, top: int, scoring: str = "chosen_softmax", groups: int = 1, keep: int = 1,
+              outputs: int | None = None, renormalise: bool = False, factor: float = 1.0):
+    """Per row of the float32 router logits ``[T, E]`` (the first ``outputs`` columns of them, where that is given): the ``top`` chosen outputs, best first (ties: the lower index), as
     int32 ``[T, top]``, and their weights, float32 ``[T, top]``. The logits may be a ``SplitSum``: the kernel adds the
     partial sums itself.
 
@@ -555,16 +619,20 @@ def moe_route(logits, bias: torch.Tensor | None, top: int, scoring: str = "chose
     alone. ``scoring="softmax"``: ``s = softmax(logits)`` over all ``E`` outputs; the choice goes by ``s + bias`` (a
     correction that only the choice sees), the weights are the chosen outputs' ``s`` as they stand; with ``groups > 1``
     the outputs form that many equal groups of neighbours, a group's score is the largest ``s + bias`` in it, and only
-    outputs of the ``keep`` best groups can be chosen. ``scoring="sigmoid"``: the same with ``s = sigmoid(logits)``."""
+    outputs of the ``keep`` best groups can be chosen. ``scoring="sigmoid"``: the same with ``s = sigmoid(logits)``.
+    ``renormalise`` (with these two): the chosen outputs' ``s`` are divided by their sum plus ``1e-20``; ``factor`` multiplies
+    the weights."""
     if isinstance(logits, SplitSum):
         _no_scale(logits, "the routing")
         parts, splits, stride = logits.parts, logits.splits, logits.stride
         _dev(parts, "logits", F32, 3)
-        t, e = logits.shape
     else:
         _dev(logits, "logits", F32, 2)
         parts, splits, stride = logits, 1, 0
-        t, e = logits.shape
+    t, ld = logits.shape
+    e = ld if outputs is None else int(outputs)
+    if not 1 <= e <= ld:
+        raise ValueError(f"{e} router outputs in rows of {ld}")
     if not 1 <= top <= e:
         raise ValueError(f"top {top} of {e} experts")
     if e > MOE_MAX_EXPERTS or top > MOE_MAX_TOP:
@@ -582,33 +650,39 @@ def moe_route(logits, bias: torch.Tensor | None, top: int, scoring: str = "chose
             raise ValueError(f"{e} router outputs in {groups} groups of which {keep} are kept")
         if top > (e // groups) * keep:
             raise ValueError(f"top {top} of the {(e // groups) * keep} outputs in the kept groups")
-        _check(library().ms_moe_route_scored(parts.data_ptr(), e, splits, stride, _ptr(bias), int(bias is not None and bias.dtype == BF16),
-                                             t, e, top, int(groups), int(keep), int(scoring == "sigmoid"), ids.data_ptr(), weights.data_ptr(), _stream()),
-               "moe_route_scored")
+        _check(library().ms_moe_route_scored(parts.data_ptr(), ld, splits, stride, _ptr(bias), int(bias is not None and bias.dtype == BF16),
+                                             t, e, top, int(groups), int(keep), int(scoring == "sigmoid"), int(renormalise), float(factor),
+                                             ids.data_ptr(), weights.data_ptr(), _stream()), "moe_route_scored")
         return ids, weights
     if groups != 1:
         raise NotImplementedError("groups of experts go with scores over all outputs")
-    _check(library().ms_moe_route(parts.data_ptr(), e, splits, stride, _ptr(bias), int(bias is not None and bias.dtype == BF16), t, e,
+    if renormalise or factor != 1.0:
+        raise NotImplementedError("a softmax over the chosen logits alone is neither renormalised nor scaled")
+    _check(library().ms_moe_route(parts.data_ptr(), ld, splits, stride, _ptr(bias), int(bias is not None and bias.dtype == BF16), t, e,
                                   top, ids.data_ptr(), weights.data_ptr(), _stream()), "moe_route")
     return ids, weights
 
 
 def moe_experts(x: torch.Tensor, ids: torch.Tensor, weights: torch.Tensor, gate: torch.Tensor | None, up: torch.Tensor,
                 down: torch.Tensor, activation: str, stream: torch.Tensor, weigh_input: bool = False,
-                scale: torch.Tensor | None = None) -> None:
+                scale: torch.Tensor | None = None, limit: float | None = None, extra: SplitSum | None = None, extra_gate=None) -> None:
     """``stream[t] += sum_j weights[t, j] * expert_e(x[t])`` with ``e = ids[t, j]``, the sum in ascending ``j``; with
     ``weigh_input`` ``stream[t] += sum_j expert_e(weights[t, j] * x[t])`` (the weight multiplies the first products' float32
     results, which is the same); ``scale`` (float32 ``[W]``) multiplies the sum element by element. A gated
     expert is ``down[e] (act(gate[e] x) * (up[e] x))``; with ``gate=None`` it is ``down[e] act(up[e] x)``. An id of
     ``E`` (the number of experts that have weights) or more names an identity expert: its term is ``weights[t, j] * x[t]``.
+    ``activation`` may be one that bounds gate and up by ``limit``. ``extra`` (``[T, W]``) is what a feed-forward that every
+    token runs put out: it joins the sum, times ``sigmoid(z[t])`` with ``extra_gate = (rows, column)`` naming ``z`` in
+    float32 rows (a tensor or a ``SplitSum``).
     ``x [T, W]`` in the compute dtype, ``gate`` / ``up`` ``[E, F, W]`` and ``down [E, W, F]`` in the same, ``stream`` float32
     ``[T, W]``. The step's (token, expert) pairs are sorted by expert on the device and every expert's run is multiplied
     in tiles (bfloat16: on the matrix cores; float32: fused multiply-adds in ascending k); the launches cover the most
     tiles the step can have, so nothing is read back and a captured step replays."""
     gated = gate is not None
-    act = _activation(activation, gated=gated)
-    if act == ACTIVATIONS["swiglu_clamped"]:
-        raise NotImplementedError(f"activation {activation!r} is not of the form act(gate) * up")
+    act = _activation(activation, limit, gated)
+    if not gated and activation in ACTIVATIONS_WITH_LIMIT:
+        raise NotImplementedError(f"activation {activation!r} takes a gate")
+    limit = float(limit or 0.0)
     _dev(x, "x", (F32, BF16), 2)
     for w, nm in ((gate, "gate"), (up, "up"), (down, "down")):
         if w is not None:
@@ -627,6 +701,22 @@ def moe_experts(x: torch.Tensor, ids: torch.Tensor, weights: torch.Tensor, gate:
         _dev(scale, "scale", F32, 1)
         if scale.shape[0] != width:
             raise ValueError(f"a scale of {scale.shape[0]} elements for width {width}")
+    more = (None, 0, 0, None, 0, 0, 0)
+    if extra is not None:
+        _check_split(extra, "extra", stream.shape)
+        _no_scale(extra, "the combine")
+        z = (None, 0, 0, 0)
+        if extra_gate is not None:
+            rows, col = extra_gate
+            of = rows.parts if isinstance(rows, SplitSum) else rows
+            _dev(of, "extra_gate", F32, 3 if isinstance(rows, SplitSum) else 2)
+            if rows.shape[0] != t or not 0 <= col < rows.shape[1]:
+                raise ValueError("extra_gate needs one row per token and a column of it")
+            z = (of.data_ptr() + 4 * col, rows.shape[1], rows.splits if isinstance(rows, SplitSum) else 1,
+                 rows.stride if isinstance(rows, SplitSum) else 0)
+        more = (extra.parts.data_ptr(), extra.splits, extra.stride, *z)
+    elif extra_gate is not None:
+        raise ValueError("a gate without what it gates")
     if e > MOE_MAX_EXPERTS:
         raise ValueError(f"{e} experts: the kernels take up to {MOE_MAX_EXPERTS}")
     if t == 0:
@@ -649,12 +739,12 @@ def moe_experts(x: torch.Tensor, ids: torch.Tensor, weights: torch.Tensor, gate:
     plan = (order.data_ptr(), tiles[0].data_ptr(), tiles[1].data_ptr(), tiles[2].data_ptr())
     h = torch.empty((pairs, f), dtype=x.dtype, device=dev)
     _check(lib.ms_moe_gemm(x.data_ptr(), width, (gate if gated else up).data_ptr(), up.data_ptr() if gated else None, h.data_ptr(), int(bf),
-                           1 if gated else 2, *plan, weights.data_ptr() if weigh_input else None, max_tiles, top, f, width, tile_rows, act, _stream()), "moe_gemm")
+                           1 if gated else 2, *plan, weights.data_ptr() if weigh_input else None, max_tiles, top, f, width, tile_rows, act, limit, _stream()), "moe_gemm")
     y = torch.empty((pairs, width), dtype=F32, device=dev)
     _check(lib.ms_moe_gemm(h.data_ptr(), f, down.data_ptr(), None, y.data_ptr(), int(bf), 0, *plan, None if weigh_input else weights.data_ptr(), max_tiles, top,
-                           width, f, tile_rows, act, _stream()), "moe_gemm")
+                           width, f, tile_rows, act, limit, _stream()), "moe_gemm")
     _check(lib.ms_moe_combine(stream.data_ptr(), y.data_ptr(), t, top, width, ids.data_ptr(), weights.data_ptr(), x.data_ptr(), int(bf),
-                              width, e, _ptr(scale), _stream()), "moe_combine")
+                              width, e, _ptr(scale), *more, _stream()), "moe_combine")
 
 
 # ------------------------------------------------------------------------------------- attention
@@ -1186,9 +1276,10 @@ def _prefill_parts_plan(batch, tile_tokens: int, kv_heads: int, part_bytes: int)
 
 
 def layernorm(x: torch.Tensor, weight: torch.Tensor, bias: torch.Tensor | None, eps: float, out_dtype,
-              rows: torch.Tensor | None = None) -> torch.Tensor:
+              rows: torch.Tensor | None = None, add: SplitSum | None = None) -> torch.Tensor:
     """``(x - mean) / sqrt(var + eps) * weight + bias`` over the float32 rows of ``x`` (all, or those named by
-    ``rows``), statistics in float32, the variance being the mean of the squared deviations."""
+    ``rows``), statistics in float32, the variance being the mean of the squared deviations. ``add``: a pending sum that is
+    added to the rows first, as ``rmsnorm`` does (in place without ``rows``)."""
     _dev(x, "x", F32, 2)
     _dev(weight, "weight", (F32, BF16), 1)
     if weight.shape[0] != x.shape[1]:
@@ -1203,9 +1294,11 @@ def layernorm(x: torch.Tensor, weight: torch.Tensor, bias: torch.Tensor | None, 
     if rows is not None:
         _dev(rows, "rows", I32, 1)
         n = rows.shape[0]
+    parts, splits, stride, scale = _pending(add, x.shape)
     out = torch.empty((n, x.shape[1]), dtype=out_dtype, device=x.device)
     _check(library().ms_layernorm(x.data_ptr(), weight.data_ptr(), _ptr(bias), int(weight.dtype == BF16), out.data_ptr(),
-                                  int(out_dtype == BF16), _ptr(rows), n, x.shape[1], float(eps), _stream()), "layernorm")
+                                  int(out_dtype == BF16), _ptr(rows), n, x.shape[1], float(eps), parts, splits, stride, scale,
+                                  _stream()), "layernorm")
     return out
 
 
@@ -1298,6 +1391,13 @@ def scale_(x: torch.Tensor, factor: float) -> torch.Tensor:
     """``x *= factor`` in place (float32)."""
     _dev(x, "x", F32)
     _check(library().ms_scale(x.data_ptr(), x.numel(), float(factor), _stream()), "scale")
+    return x
+
+
+def softcap_(x: torch.Tensor, cap: float) -> torch.Tensor:
+    """``x = cap * tanh(x / cap)`` in place (float32)."""
+    _dev(x, "x", F32)
+    _check(library().ms_softcap(x.data_ptr(), x.numel(), float(cap), _stream()), "softcap")
     return x
 
 
@@ -1501,39 +1601,56 @@ def map_difference_norm(a: torch.Tensor, groups: int, per_group: int, value_dim:
     return out
 
 
-def latent_prepare(x, q_col: int, kv_col: int | None, rope, rot: int, pairing: str, latent_weight, eps, slots, k_cache, v_cache,
-                   heads: int, plain_dim: int, rot_dim: int, latent_dim: int, out_dtype):
-    """From the float32 projection ``x``: every head's plain query part into ``q_plain [T, H Dn]``, its turned part into
-    the last ``R`` columns of that head in ``q_full [T, H (C + R)]`` (the first ``C`` are left for the caller), and, with
-    ``kv_col``, the token's cache row ``[C + R]`` at ``slots`` (``k_cache [pages, 1, page, C + R]``): the latent after an
-    RMS norm (``latent_weight``) and the turned shared key part; the normed latent goes to ``v_cache [pages, 1, C, page]``
-    as well, as the token's value. The first ``rot`` of the ``R`` elements turn by ``rope``'s angles. Returns
-    ``(q_plain, q_full)``."""
-    _dev(x, "x", F32, 2)
-    t = x.shape[0]
+def latent_prepare(x, q_col: int | None, kv_col: int | None, rope, rot: int, pairing: str, latent_weight, eps, slots, k_cache, v_cache,
+                   heads: int, plain_dim: int, rot_dim: int, latent_dim: int, out_dtype, query_latent=None):
+    """From the float32 projection ``x`` (a tensor or a ``SplitSum``): every head's plain query part into ``q_plain [T, H Dn]``,
+    its turned part into the last ``R`` columns of that head in ``q_full [T, H (C + R)]`` (the first ``C`` are left for the
+    caller; both None with ``q_col=None``: ``x`` holds no queries), and, with ``kv_col``, the token's cache row ``[C + R]`` at
+    ``slots`` (``k_cache [pages, 1, page, C + R]``): the latent after an RMS norm (``latent_weight``) and the turned shared key
+    part; the normed latent goes to ``v_cache [pages, 1, C, page]`` as well, as the token's value. The first ``rot`` of the ``R``
+    elements turn by ``rope``'s angles. ``query_latent = (column, weight [Q])``: ``x`` also holds a latent that the queries are made
+    from; it is returned after an RMS norm with that weight. Returns ``(q_plain, q_full)``, and with ``query_latent`` the
+    normed latent ``[T, Q]`` behind them."""
+    split = isinstance(x, SplitSum)
+    _no_scale(x, "the latent's preparation")
+    rows = x.parts if split else x
+    _dev(rows, "x", F32, 3 if split else 2)
+    t, ld = x.shape
+    src, splits, stride = rows.data_ptr(), x.splits if split else 1, x.stride if split else 0
     if out_dtype not in (F32, BF16):
         raise TypeError(f"unsupported output dtype {out_dtype}")
     if rot:
         _dev(rope, "rope", F32, 2)
         if tuple(rope.shape) != (t, rot):
             raise ValueError(f"rotation table is {tuple(rope.shape)}, expected [{t}, {rot}]")
-    w_bf16 = 0
+    w_dtype, page = None, 1
     if kv_col is not None:
         _dev(slots, "slots", I32, 1)
         page = _check_special_caches(k_cache, v_cache, out_dtype, 1, latent_dim + rot_dim, latent_dim, 1, False)
         _dev(latent_weight, "latent_weight", (F32, BF16), 1)
         if slots.shape[0] != t or latent_weight.shape[0] != latent_dim:
             raise ValueError("one slot per token and a weight of C elements are needed")
-        w_bf16 = int(latent_weight.dtype == BF16)
-    q_plain = torch.empty((t, heads * plain_dim), dtype=out_dtype, device=x.device)
-    q_full = torch.empty((t, heads * (latent_dim + rot_dim)), dtype=out_dtype, device=x.device)
+        w_dtype = latent_weight.dtype
+    q_plain = q_full = latent = None
+    if q_col is not None:
+        if q_col < 0 or ld < q_col + heads * (plain_dim + rot_dim):
+            raise ValueError(f"rows of {ld} hold no {heads} query heads of {plain_dim} + {rot_dim} elements from column {q_col} on")
+        q_plain = torch.empty((t, heads * plain_dim), dtype=out_dtype, device=rows.device)
+        q_full = torch.empty((t, heads * (latent_dim + rot_dim)), dtype=out_dtype, device=rows.device)
+    dq_col, qw, size = -1, None, 0
+    if query_latent is not None:
+        dq_col, qw = query_latent
+        _dev(qw, "the query latent's weight", (F32, BF16) if w_dtype is None else w_dtype, 1)
+        w_dtype, size = qw.dtype, qw.shape[0]
+        latent = torch.empty((t, size), dtype=out_dtype, device=rows.device)
+    keeps = kv_col is not None
     _check(library().ms_latent_prepare(
-        x.data_ptr(), x.shape[1], int(q_col), -1 if kv_col is None else int(kv_col), _ptr(rope) if rot else None, int(rot),
-        _pairing(pairing), _ptr(latent_weight) if kv_col is not None else None, w_bf16, float(eps), q_plain.data_ptr(),
-        q_full.data_ptr(), _ptr(slots) if kv_col is not None else None, _ptr(k_cache) if kv_col is not None else None,
-        _ptr(v_cache) if kv_col is not None else None, page if kv_col is not None else 1, int(out_dtype == BF16), t, heads, plain_dim,
-        rot_dim, latent_dim, _stream()), "latent_prepare")
-    return q_plain, q_full
+        src + 4 * q_col if q_col is not None else None, ld, splits, stride, src, ld, splits, stride, int(kv_col) if keeps else -1,
+        int(dq_col), size, _ptr(rope) if rot else None, int(rot), _pairing(pairing), _ptr(latent_weight) if keeps else None, _ptr(qw),
+        int(w_dtype == BF16), float(eps), _ptr(q_plain), _ptr(q_full), _ptr(latent), _ptr(slots) if keeps else None,
+        _ptr(k_cache) if keeps else None, _ptr(v_cache) if keeps else None, page, int(out_dtype == BF16), t, heads, plain_dim, rot_dim,
+        latent_dim, _stream()), "latent_prepare")
+    return (q_plain, q_full) if query_latent is None else (q_plain, q_full, latent)
 
 
 def head_gate_(o: torch.Tensor, x: torch.Tensor, col: int, heads: int, each: bool = False) -> torch.Tensor:

@@ -19,7 +19,8 @@ elements over one key head whose rows are ``[c, rotated part]`` and whose values
 those rows and, as the values, ``c`` once more with the tokens of one element side by side (the order in which the
 matrix cores take the second product's operand). Options: a sliding ``window``, a learned sink per head in the softmax's
 denominator (``sinks``), a sigmoid gate read off the mixer's input (``gate``: ``"head"`` or True, one per head;
-``"element"``, one per element of the concatenated heads), and ``shares_cache``: the
+``"element"``, one per element of the concatenated heads), ``query_rank`` (the queries come from a latent of that size of
+their own: a product, an RMS norm, a second product; tensors ``dq dq.norm uq`` in the place of ``q``), and ``shares_cache``: the
 layer has no projection of its own for the latent and reads the cache rows another layer wrote (its run-order entry
 names that layer's cache slot), with query, up-projections, window and the rest of its own.
 """
@@ -151,7 +152,8 @@ class DifferentialAttention(Mixer):
 @register("mixer", "latent_attention")
 class LatentAttention(Mixer):
     scales_output = True
-    NAMES = {"q": "q", "dkv": "dkv", "dkv_norm": "dkv.norm", "uk": "uk", "uv": "uv", "sink": "sink", "g": "g", "o": "o"}
+    NAMES = {"q": "q", "dq": "dq", "dq_norm": "dq.norm", "uq": "uq", "dkv": "dkv", "dkv_norm": "dkv.norm", "uk": "uk", "uv": "uv",
+             "sink": "sink", "g": "g", "o": "o"}
 
     def __init__(self, spec: PartSpec, rt):
         super().__init__(spec, rt)
@@ -171,28 +173,35 @@ class LatentAttention(Mixer):
         if self.gate not in (None, "head", "element"):
             raise ValueError(f"gate {self.gate!r}: one per 'head', one per 'element' or None")
         self.shares_cache = bool(spec.get("shares_cache", False))
+        self.query_rank = int(spec.get("query_rank") or 0)
         self.names = _named(spec, self.NAMES)
         self.key_dim = self.latent_dim + self.rot_dim
-        if min(self.heads, self.plain_dim, self.value_dim, self.latent_dim) < 1 or self.rot_dim < 0 or self.window < 0:
-            raise ValueError("heads and sizes must be positive, rot_dim and window not negative")
+        if min(self.heads, self.plain_dim, self.value_dim, self.latent_dim) < 1 or min(self.rot_dim, self.window, self.query_rank) < 0:
+            raise ValueError("heads and sizes must be positive, rot_dim, window and query_rank not negative")
         if self.key_dim > 1024:
             raise ValueError(f"latent and rotated sizes {self.latent_dim} + {self.rot_dim}: the attention kernel takes up to 1024 together")
         if not self.scale > 0:
             raise ValueError(f"the attention scale must be positive, not {self.scale}")
         pos = spec.get("position") or PartSpec("none")
         self.position = part_class("position", pos)(pos, rt)
-        self.q_col = 0
-        self.kv_col = None if self.shares_cache else self.heads * (self.plain_dim + self.rot_dim)
-        self.g_col = self.heads * (self.plain_dim + self.rot_dim) + (0 if self.shares_cache else self.key_dim)
-        self.proj = self.o = self.dkv_norm = self.uk_t = self.uv = self.sink = None
+        # the first projection's columns: the queries (or the latent they come from), the token's latent and key part, the gates
+        self.q_width = self.heads * (self.plain_dim + self.rot_dim)
+        first = self.query_rank or self.q_width
+        self.kv_col = None if self.shares_cache else first
+        self.g_col = first + (0 if self.shares_cache else self.key_dim)
+        self.proj = self.o = self.dkv_norm = self.uk_t = self.uv = self.sink = self.uq = self.dq_norm = None
 
     @classmethod
     def tensors(cls, spec: PartSpec) -> dict[str, TensorSpec]:
         n = _named(spec, cls.NAMES)
         w, h = int(spec["hidden_size"]), int(spec["num_heads"])
         d, r, e, c = (int(spec[k]) for k in ("head_dim", "rot_dim", "value_dim", "latent_dim"))
-        out = {n["q"]: TensorSpec((h * (d + r), w)), n["uk"]: TensorSpec((h * d, c)), n["uv"]: TensorSpec((h * e, c)),
-               n["o"]: TensorSpec((w, h * e))}
+        out = {n["uk"]: TensorSpec((h * d, c)), n["uv"]: TensorSpec((h * e, c)), n["o"]: TensorSpec((w, h * e))}
+        rank = int(spec.get("query_rank") or 0)
+        if rank:
+            out.update({n["dq"]: TensorSpec((rank, w)), n["dq_norm"]: TensorSpec((rank,), init="ones"), n["uq"]: TensorSpec((h * (d + r), rank))})
+        else:
+            out[n["q"]] = TensorSpec((h * (d + r), w))
         if not spec.get("shares_cache", False):
             out[n["dkv"]] = TensorSpec((c + r, w))
             out[n["dkv_norm"]] = TensorSpec((c,), init="ones")
@@ -204,10 +213,12 @@ class LatentAttention(Mixer):
 
     def bind(self, tensors) -> None:
         n = self.names
-        parts = [tensors[n["q"]]] + ([] if self.shares_cache else [tensors[n["dkv"]]]) + ([tensors[n["g"]]] if self.gate else [])
+        parts = [tensors[n["dq" if self.query_rank else "q"]]] + ([] if self.shares_cache else [tensors[n["dkv"]]]) + ([tensors[n["g"]]] if self.gate else [])
         if len({t.dtype for t in parts}) != 1:
-            raise ValueError(f"{n['q']} and its neighbours are stored in different dtypes")
+            raise ValueError(f"{n['dq' if self.query_rank else 'q']} and its neighbours are stored in different dtypes")
         self.proj = torch.cat(parts, dim=0).contiguous()
+        if self.query_rank:
+            self.uq, self.dq_norm = tensors[n["uq"]], tensors[n["dq_norm"]]
         h, d, e, c = self.heads, self.plain_dim, self.value_dim, self.latent_dim
         self.uk_t = tensors[n["uk"]].view(h, d, c).transpose(1, 2).contiguous()  # per head [C, D]: q_plain -> the latent's space
         self.uv = tensors[n["uv"]].view(h, e, c).contiguous()
@@ -224,14 +235,23 @@ class LatentAttention(Mixer):
         ops = self.rt.ops
         if cache.writes == self.shares_cache:
             raise ValueError("a latent attention writes the cache exactly when it has a latent projection of its own")
-        x32 = ops.linear(x, self.proj, out_dtype=torch.float32)
+        # few rows leave partial sums, which the preparation adds itself; a gate reads the finished projection
+        x32 = ops.linear(x, self.proj, out_dtype=torch.float32, defer=self.gate is None)
         rot = self.position.rotation(batch)
         if rot is not None and rot.dim > self.rot_dim:
             raise ValueError(f"{rot.dim} rotated elements in a part of {self.rot_dim}")
-        q_plain, q_full = ops.latent_prepare(
-            x32, self.q_col, self.kv_col, rot.table if rot is not None else None, rot.dim if rot is not None else 0,
-            rot.pairing if rot is not None else "halves", self.dkv_norm, self.eps, cache.slots, cache.k, cache.v, self.heads,
-            self.plain_dim, self.rot_dim, self.latent_dim, self.rt.dtype)
+
+        def prepare(rows, q_col, kv_col, query_latent=None):
+            return ops.latent_prepare(
+                rows, q_col, kv_col, rot.table if rot is not None else None, rot.dim if rot is not None else 0,
+                rot.pairing if rot is not None else "halves", self.dkv_norm, self.eps, cache.slots, cache.k, cache.v, self.heads,
+                self.plain_dim, self.rot_dim, self.latent_dim, self.rt.dtype, query_latent)
+
+        if self.query_rank:
+            latent = prepare(x32, None, self.kv_col, (0, self.dq_norm))[2]
+            q_plain, q_full = prepare(ops.linear(latent, self.uq, out_dtype=torch.float32, defer=True), 0, None)
+        else:
+            q_plain, q_full = prepare(x32, 0, self.kv_col)
         ops.head_linear(q_plain, self.uk_t, q_full, 0)
         a = ops.paged_attention(q_full, cache.k, cache.v, cache.block_table, batch, self.heads, 1, self.key_dim, self.scale,
                                 self.window, self.latent_dim, sinks=self.sink, wide_heads=True)
@@ -240,7 +260,7 @@ class LatentAttention(Mixer):
         return ops.linear(o, self.o, accumulate_into=residual, defer=True, scale=self.out_scale)
 
     def parameters_bytes(self) -> int:
-        ts = [self.proj, self.uk_t, self.uv, self.o] + [t for t in (self.dkv_norm, self.sink) if t is not None]
+        ts = [self.proj, self.uk_t, self.uv, self.o] + [t for t in (self.dkv_norm, self.sink, self.uq, self.dq_norm) if t is not None]
         return sum(t.numel() * t.element_size() for t in ts)
 
     def flops(self, rows) -> int:
@@ -252,5 +272,6 @@ class LatentAttention(Mixer):
             else:
                 pairs += n * cached + n * (n + 1) // 2
         linear = 2 * tokens * self.hidden * (self.proj.shape[0] if self.proj is not None else 0) + 2 * tokens * self.hidden * self.heads * self.value_dim
+        linear += 2 * tokens * self.query_rank * self.q_width
         per_head = 2 * tokens * self.heads * self.latent_dim * (self.plain_dim + self.value_dim)
         return linear + per_head + 2 * pairs * self.heads * (self.key_dim + self.latent_dim)

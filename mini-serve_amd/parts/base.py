@@ -9,7 +9,8 @@ those. No part knows which model it is in. The kinds:
 * ``Mixer``           ``forward(x, batch, cache, state, residual) -> pending`` (``state``: name -> tensor)
 * ``FeedForward``     ``forward(x, residual) -> pending``
 * ``Block``           ``forward(residual, batch, cache, state, pending) -> pending`` (where norms and sums sit)
-* ``Embedding``       ``forward(token_ids) -> residual``            (float32 ``[T, width]``)
+* ``Embedding``       ``forward(token_ids, batch, state, keep) -> residual``  (float32 ``[T, width]``)
+* ``Injection``       ``forward(residual, start, pending)``        (what joins the stream ahead of a run-order entry)
 * ``Head``            ``forward(x) -> logits``                      (float32 ``[rows, vocab]``)
 
 The residual stream is float32 in every compute dtype: sums of layer outputs are never rounded
@@ -275,7 +276,24 @@ class Block(Part):
 
 
 class Embedding(Part):
-    def forward(self, token_ids):
+    """``state_need``: what it keeps per request (a token's vector may depend on tokens of earlier steps)."""
+
+    def state_need(self) -> StateNeed | None:
+        return None
+
+    def forward(self, token_ids, batch=None, state=None, keep=False):
+        """The residual stream of the step's tokens; ``keep``: the pair (stream, a copy that nobody adds to)."""
+        raise NotImplementedError
+
+
+class Injection(Part):
+    """What joins the residual stream right before a run-order entry. ``needs_start``: it reads what the embedding put out."""
+
+    needs_start = False
+
+    def forward(self, residual, start, pending=None) -> None:
+        """Add to ``residual`` in place, together with ``pending``. ``start``: the embedding's output (None unless an
+        injection of the model needs it)."""
         raise NotImplementedError
 
 

@@ -14,7 +14,8 @@ from .registry import part_class, register
 @register("block", "prenorm")
 class PreNormBlock(Block):
     """Options, none of which the reference has: ``mixer_scale`` / ``ffn_scale`` name a tensor ``[width]`` each by which what the
-    sublayer adds is multiplied element by element (a layer scale; the sublayer applies it, ``Sublayer.scale_output``); a
+    sublayer adds is multiplied element by element (a layer scale; the sublayer applies it, ``Sublayer.scale_output``); ``residual_scale``
+    is one number by which what both sublayers add is multiplied (applied the same way); a
     layer without a feed-forward has no second norm (``ffn_norm`` None), and ``spare`` then names tensors ``{name: width}``
     that a checkpoint may still carry for it."""
 
@@ -23,6 +24,7 @@ class PreNormBlock(Block):
         mn, fn = spec["mixer_norm"], spec.get("ffn_norm")
         self.mixer_norm = part_class("norm", mn)(mn, rt)
         self.ffn_norm = part_class("norm", fn)(fn, rt) if fn is not None else None
+        self.residual_scale = 1.0 if spec.get("residual_scale") is None else float(spec["residual_scale"])
 
     @classmethod
     def tensors(cls, spec: PartSpec) -> dict[str, TensorSpec]:
@@ -40,12 +42,19 @@ class PreNormBlock(Block):
 
     def bind(self, tensors) -> None:
         self.mixer_norm.bind(tensors)
-        if self.spec.get("mixer_scale"):
-            self.mixer.scale_output(tensors[self.spec["mixer_scale"]])
+        self._scale(self.mixer, "mixer", tensors)
         if self.ffn_norm is not None:
             self.ffn_norm.bind(tensors)
-            if self.spec.get("ffn_scale"):
-                self.feed_forward.scale_output(tensors[self.spec["ffn_scale"]])
+            self._scale(self.feed_forward, "ffn", tensors)
+
+    def _scale(self, sublayer, which: str, tensors) -> None:
+        scale = tensors[self.spec[f"{which}_scale"]].float() if self.spec.get(f"{which}_scale") else None
+        if self.residual_scale != 1.0:
+            if scale is None:
+                scale = torch.ones(int(self.spec[f"{which}_norm"]["width"]), device=self.rt.device if self.rt is not None else "cpu")
+            scale = scale * self.residual_scale
+        if scale is not None:
+            sublayer.scale_output(scale)
 
     def forward(self, residual, batch, cache, state, pending=None):
         x = self.mixer_norm.forward(residual, add=pending)

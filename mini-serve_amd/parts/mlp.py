@@ -25,6 +25,10 @@ value plus ``router_bias``, a correction that only the choice sees; the weights 
 as they stand, not renormalised); ``groups`` / ``keep_groups`` (with that scoring: the router's outputs form ``groups``
 equal groups of neighbours, a group's score is the largest choice score in it, and only outputs of the ``keep_groups``
 best groups can be chosen); ``scoring="sigmoid"`` (the same with every output's sigmoid for its softmax value);
+``renormalise`` (with either: the weights are the chosen outputs' values divided by their sum) and ``factor`` (multiplies the
+weights); ``limit`` (of an activation that bounds gate and up); ``shared_gate`` (what the shared feed-forward puts out is
+multiplied by the sigmoid of one number per token, a product of the token with the tensor ``names["shared_gate"]`` ``[1, W]``: it
+is one more row of the router's product, and the kernel that adds the experts' results adds the gated one as well);
 ``weigh="input"`` (a choice's weight multiplies what the expert reads instead of what it puts out); ``identity`` (the router has that many outputs more than there are experts with weights; a
 token that chooses one of them gets its own input back, times the weight)."""
 
@@ -85,10 +89,15 @@ class GatedMLP(FeedForward):
         self.gate_up = ops.interleave_gate_up(g, u) if self.block else torch.cat((g, u), dim=0).contiguous()
         self.down = tensors[self.names["down"]]
 
+    def _inner(self, x):
+        return self.rt.ops.gated_linear(x, self.gate_up, self.activation, out_dtype=self.rt.dtype, block=self.block, limit=self.limit)
+
     def forward(self, x, residual):
-        ops = self.rt.ops
-        m = ops.gated_linear(x, self.gate_up, self.activation, out_dtype=self.rt.dtype, block=self.block, limit=self.limit)
-        return ops.linear(m, self.down, accumulate_into=residual, defer=True, scale=self.out_scale)
+        return self.rt.ops.linear(self._inner(x), self.down, accumulate_into=residual, defer=True, scale=self.out_scale)
+
+    def product(self, x):
+        """What the feed-forward puts out, as a ``SplitSum`` that nothing has scaled or added anywhere."""
+        return self.rt.ops.linear_sum(self._inner(x), self.down)
 
     def parameters_bytes(self) -> int:
         return sum(t.numel() * t.element_size() for t in (self.gate_up, self.down))
@@ -122,10 +131,16 @@ class DenseMLP(FeedForward):
     def bind(self, tensors) -> None:
         self.up, self.down = tensors[self.names["up"]], tensors[self.names["down"]]
 
-    def forward(self, x, residual):
+    def _inner(self, x):
         ops = self.rt.ops
-        m = ops.activate(ops.linear(x, self.up, out_dtype=torch.float32), self.activation, self.rt.dtype)
-        return ops.linear(m, self.down, accumulate_into=residual, defer=True, scale=self.out_scale)
+        return ops.activate(ops.linear(x, self.up, out_dtype=torch.float32), self.activation, self.rt.dtype)
+
+    def forward(self, x, residual):
+        return self.rt.ops.linear(self._inner(x), self.down, accumulate_into=residual, defer=True, scale=self.out_scale)
+
+    def product(self, x):
+        """What the feed-forward puts out, as a ``SplitSum`` that nothing has scaled or added anywhere."""
+        return self.rt.ops.linear_sum(self._inner(x), self.down)
 
     def parameters_bytes(self) -> int:
         return sum(t.numel() * t.element_size() for t in (self.up, self.down))
@@ -137,7 +152,8 @@ class DenseMLP(FeedForward):
 def _moe_names(spec: PartSpec) -> dict[str, str]:
     given = spec.get("names") or {}
     default = {"router": "router.weight", "router_bias": "router.bias", "expert": "experts.{}.", "gate": "gate_proj.weight",
-               "up": "up_proj.weight", "down": "down_proj.weight"}
+               "up": "up_proj.weight", "down": "down_proj.weight",
+               "shared_gate": "shared_gate.weight"}
     return {k: given.get(k, d) for k, d in default.items()}
 
 
@@ -161,6 +177,10 @@ class MixtureMLP(FeedForward):
         self.identity = int(spec.get("identity") or 0)
         self.outputs = self.num_experts + self.identity  # what the router tells apart
         self.weigh = spec.get("weigh", "output")
+        self.renormalise = bool(spec.get("renormalise", False))
+        self.factor = 1.0 if spec.get("factor") is None else float(spec["factor"])
+        self.limit = float(spec["limit"]) if spec.get("limit") is not None else None
+        self.shared_gate = bool(spec.get("shared_gate", False))
         if self.scoring not in ("chosen_softmax", "softmax", "sigmoid"):
             raise ValueError(f"router scoring {self.scoring!r}: 'chosen_softmax', 'softmax' or 'sigmoid'")
         if self.weigh not in ("output", "input"):
@@ -169,13 +189,20 @@ class MixtureMLP(FeedForward):
             raise ValueError(f"{self.num_experts} experts and {self.identity} identity experts")
         if self.groups != 1 and self.scoring == "chosen_softmax":
             raise NotImplementedError("groups of experts go with scores over all outputs")
+        if (self.renormalise or self.factor != 1.0) and self.scoring == "chosen_softmax":
+            raise NotImplementedError("a softmax over the chosen logits alone is neither renormalised nor scaled")
+        if self.shared_gate and spec.get("shared") is None:
+            raise ValueError("a gate on a shared feed-forward that the mixture does not have")
         if self.groups < 1 or self.outputs % self.groups or not 1 <= self.keep_groups <= self.groups:
             raise ValueError(f"{self.outputs} router outputs in {self.groups} groups of which {self.keep_groups} are kept")
         if not 1 <= self.top <= (self.outputs // self.groups) * self.keep_groups:
             raise ValueError(f"top {self.top} of {self.outputs} router outputs in {self.groups} groups of which {self.keep_groups} are kept")
         if rt is not None:
             ops = rt.ops
-            if self.activation not in ops.ACTIVATIONS or self.activation in ops.ACTIVATIONS_WITH_LIMIT or (
+            limited = self.activation in ops.ACTIVATIONS_WITH_LIMIT
+            if limited and self.gated and not (self.limit is not None and self.limit > 0):
+                raise ValueError(f"activation {self.activation!r} needs a positive limit, got {self.limit!r}")
+            if self.activation not in ops.ACTIVATIONS or (limited and not self.gated) or (
                     self.gated and self.activation in ops.ACTIVATIONS_UNGATED_ONLY):
                 raise NotImplementedError(f"activation {self.activation!r} is not of the form "
                                           f"{'act(gate) * up' if self.gated else 'act(up)'}")
@@ -208,11 +235,18 @@ class MixtureMLP(FeedForward):
         sh = spec.get("shared")
         if sh is not None:
             out.update(part_class("feed_forward", sh).tensors(sh))
+            if spec.get("shared_gate", False):
+                out[p + n["shared_gate"]] = TensorSpec((1, h))
         return out
 
     def bind(self, tensors) -> None:
         n, p = self.names, self.prefix
         self.router = tensors[p + n["router"]]
+        if self.shared_gate:  # one more row of the same product
+            gate = tensors[p + n["shared_gate"]]
+            if gate.dtype != self.router.dtype:
+                raise ValueError(f"{p}: the router and the shared feed-forward's gate are stored in different dtypes")
+            self.router = torch.cat((self.router, gate), dim=0).contiguous()
         self.bias = tensors[p + n["router_bias"]] if self.router_bias else None
         kinds = ("gate", "up", "down") if self.gated else ("up", "down")
         per = [{k: v for k, v in self._expert_names(self.spec, j).items() if k in kinds} for j in range(self.num_experts)]
@@ -231,11 +265,14 @@ class MixtureMLP(FeedForward):
 
     def forward(self, x, residual):
         ops = self.rt.ops
-        pending = self.shared.forward(x, residual) if self.shared is not None else None
+        joins = self.shared is not None and self.shared_gate  # the combine adds what the shared feed-forward puts out
+        pending = self.shared.forward(x, residual) if self.shared is not None and not joins else None
         logits = ops.linear(x, self.router, out_dtype=torch.float32, defer=True)  # few rows: partial sums, added by the routing
-        ids, weights = ops.moe_route(logits, self.bias, self.top, self.scoring, self.groups, self.keep_groups)
+        ids, weights = ops.moe_route(logits, self.bias, self.top, self.scoring, self.groups, self.keep_groups, self.outputs,
+                                     self.renormalise, self.factor)
         xe = ops.cast(x, self.up.dtype)  # experts stored in 32-bit compute in 32-bit
-        ops.moe_experts(xe, ids, weights, self.gate, self.up, self.down, self.activation, residual, self.weigh == "input", self.out_scale)
+        ops.moe_experts(xe, ids, weights, self.gate, self.up, self.down, self.activation, residual, self.weigh == "input", self.out_scale,
+                        self.limit, self.shared.product(x) if joins else None, (logits, self.outputs) if joins else None)
         return pending
 
     def parameters_bytes(self) -> int:

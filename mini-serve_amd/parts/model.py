@@ -26,6 +26,8 @@ def expected_tensors(spec: ModelSpec) -> dict[str, TensorSpec]:
             out[full] = ts
 
     add(part_class("embedding", spec.embedding).tensors(spec.embedding))
+    for p in spec.injections:  # (several may read rows of one table)
+        add(part_class("injection", p).tensors(p))
     for layer in spec.layers:
         add(part_class("block", layer.block).tensors(layer.block), layer.prefix)
         add(part_class("mixer", layer.mixer).tensors(layer.mixer), layer.prefix)
@@ -96,6 +98,15 @@ class DecoderModel:
             block = part_class("block", layer.block)(layer.block, rt, mixer, ffn)
             block.bind(local(layer.prefix, type(block), layer.block))
             self.blocks.append(block)
+        self.injections = []  # per run-order entry: what joins the stream before it, or None
+        for e in spec.run_order:
+            part = part_class("injection", e.before)(e.before, rt) if e.before is not None else None
+            if part is not None:
+                part.bind(weights)
+            self.injections.append(part)
+        self.keeps_start = any(p is not None and p.needs_start for p in self.injections)
+        # what the embedding keeps per request lies in a slot of its own, behind the run order's
+        self.embedding_slot = spec.num_cache_slots if self.embedding.state_need() is not None else None
         self.final_norm = part_class("norm", spec.final_norm)(spec.final_norm, rt)
         self.final_norm.bind(weights)
         self.head = part_class("head", spec.head)(spec.head, rt)
@@ -104,7 +115,7 @@ class DecoderModel:
     # ------------------------------------------------------------------ cache needs
 
     def cache_slots(self) -> list[CacheSlotNeed]:
-        """One entry per cache slot of the run order, from the mixer that writes it. An entry that reads a slot
+        """One entry per cache slot of the run order, from the mixer that writes it (and one for what the embedding keeps). An entry that reads a slot
         another entry wrote must keep the same planes and state; its window may differ, and the slot then keeps
         the widest of them (every token, if one of its readers sees every token)."""
         needs: dict[int, CacheSlotNeed] = {}
@@ -126,6 +137,8 @@ class DecoderModel:
                 window = 0 if 0 in (held.kv.window, need.kv.window) else max(held.kv.window, need.kv.window)
                 keep = max(held.kv.keep_first, need.kv.keep_first) if window else 0
                 needs[e.cache] = CacheSlotNeed(e.cache, KVNeed(held.kv.planes, window, keep), held.state)
+        if self.embedding_slot is not None:
+            needs[self.embedding_slot] = CacheSlotNeed(self.embedding_slot, None, self.embedding.state_need())
         return [needs[s] for s in sorted(needs)]
 
     # ------------------------------------------------------------------ forward
@@ -138,9 +151,15 @@ class DecoderModel:
 
     def _forward(self, batch, pool):
         batch.memo = {}  # what parts share between layers is made anew in every pass (a captured pass records it)
-        residual = self.embedding.forward(batch.token_ids)
+        kept = pool.state_view(self.embedding_slot, batch) if self.embedding_slot is not None else None
+        residual = self.embedding.forward(batch.token_ids, batch, kept, self.keeps_start)
+        residual, start = residual if self.keeps_start else (residual, None)
         pending = None  # a sum a layer left to be added to the residual stream by its next reader
-        for e in self.spec.run_order:
+        for e, injection in zip(self.spec.run_order, self.injections):
+            if injection is not None:
+                injection.forward(residual, start, pending)
+                pending = None
+                batch.memo.pop(ROUNDED_RESIDUAL, None)
             cache = pool.view(e.cache, batch, e.writes_cache) if e.cache is not None else None
             state = pool.state_view(e.cache, batch) if e.cache is not None else None
             left = batch.memo.get(ROUNDED_RESIDUAL)
@@ -166,6 +185,7 @@ class DecoderModel:
         norm and the head (embedding rows are only gathered). Only parts that route tokens to some of their weights read
         more for more tokens."""
         total = self.final_norm.parameters_bytes() + self.head.parameters_bytes()
+        total += sum(p.parameters_bytes() for p in self.injections if p is not None)
         for e in self.spec.run_order:
             b = self.blocks[e.layer]
             total += b.parameters_bytes() + b.mixer.step_read_bytes(tokens) + b.feed_forward.step_read_bytes(tokens)

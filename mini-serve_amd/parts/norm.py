@@ -78,9 +78,7 @@ class LayerNorm(Norm):
         self.bias = tensors[self.spec["bias_tensor"]] if self.spec.get("bias_tensor") else None
 
     def forward(self, x, rows=None, add=None):
-        ops = self.rt.ops
-        ops.add_pending(x, add)  # the kernel takes no pending sum along: the stream is brought up to date first
-        return ops.layernorm(x, self.weight, self.bias, self.eps, self.rt.dtype, rows)
+        return self.rt.ops.layernorm(x, self.weight, self.bias, self.eps, self.rt.dtype, rows, add)
 
     def parameters_bytes(self) -> int:
         return sum(t.numel() * t.element_size() for t in (self.weight, self.bias) if t is not None)

@@ -1,12 +1,12 @@
 """Registries of parts by category and kind. A new mixer, feed-forward, norm, position encoding,
-block arrangement, embedding or head is one class plus one ``register`` call; configurations
+block arrangement, embedding, head or injection is one class plus one ``register`` call; configurations
 then name it by ``kind`` in a ``PartSpec``."""
 
 from __future__ import annotations
 
 from ..config.spec import PartSpec
 
-CATEGORIES = ("mixer", "feed_forward", "norm", "position", "block", "embedding", "head")
+CATEGORIES = ("mixer", "feed_forward", "norm", "position", "block", "embedding", "head", "injection")
 PARTS: dict[str, dict[str, type]] = {c: {} for c in CATEGORIES}
 
 
