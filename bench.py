@@ -25,9 +25,9 @@ with its share of the roofline), ``measured_peaks`` (what this box gives a strea
 and the engine's bfloat16 product) and ``sidecar`` (device, clocks and power while the headline point
 ran, versions, commit, the engine's effective configuration).
 
-``--design kakunex`` (or ``fimolix``, ``reselorn``, ``zigelorn``, ``bipazen``) measures something else and leaves the above as it is: prefill
-and decode throughput of that architecture beside Qwen3 models of equal size (Zigelorn: beside Kakunex models, Bipazen:
-beside Zigelorn models; ``miniserve_amd/measurement/designs.py``), one JSON line.
+``--design kakunex`` (or ``fimolix``, ``reselorn``, ``zigelorn``, ``bipazen``, ``lutosun``) measures something else and leaves the above as it is:
+prefill and decode throughput of that architecture beside Qwen3 models of equal size (Zigelorn: beside Kakunex models, Bipazen:
+beside Zigelorn models, Lutosun: beside Bipazen models; ``miniserve_amd/measurement/designs.py``), one JSON line.
 
 Peaks: MI355X's published 8 TB/s HBM and 2.5 PFLOP/s dense bf16 (157.3 TFLOP/s float32).
 """
@@ -75,8 +75,8 @@ def main() -> int:
     ap.add_argument("--prefill-tokens", type=int, default=2048, help="tokens of the timed prefill step")
     ap.add_argument("--prefill-cached", type=int, default=0,
                     help="tokens of the same sequence already in the cache when the timed step runs (fed untimed, 2,048 a step)")
-    ap.add_argument("--design", choices=("kakunex", "fimolix", "reselorn", "zigelorn", "bipazen"), default=None,
-                    help="instead of the workload above: prefill and decode of this architecture beside Qwen3 (zigelorn: Kakunex, bipazen: Zigelorn) of equal size")
+    ap.add_argument("--design", choices=("kakunex", "fimolix", "reselorn", "zigelorn", "bipazen", "lutosun"), default=None,
+                    help="instead of the workload above: prefill and decode of this architecture beside Qwen3 (zigelorn: Kakunex, bipazen: Zigelorn, lutosun: Bipazen) of equal size")
     ap.add_argument("--shapes", default=None, help="with --design: the shapes to run, with commas between them (default: all)")
     args = ap.parse_args()
     if args.gpus != 1:

@@ -188,6 +188,31 @@ def _bipazen_tiny() -> dict:
 PRESETS["bipazen-tiny"] = _bipazen_tiny()
 
 
+def _lutosun_tiny() -> dict:
+    """Four layers that hold every part of the architecture once: a row per pair of tokens, layers in front of and behind a run
+    of two layers that is run three times, mixtures of different sizes, and a layer without a feed-forward."""
+
+    def latent(heads, dim, rot_dim, vdim, q_rank, kv_rank, mlp):
+        return {"type": "latent_attention", "mlp": mlp,
+                "mixer": {"heads": heads, "dim": dim, "rot_dim": rot_dim, "vdim": vdim, "q_rank": q_rank, "kv_rank": kv_rank,
+                          "scale": (dim + rot_dim) ** -0.5, "rot": {"base": 3000.0, "dims": rot_dim}}}
+
+    def moe(experts, top, ff, shared):
+        return {"kind": "moe", "router": {"experts": experts, "top": top, "scale": 1.5}, "expert": {"ff": ff, "limit": 2.0},
+                "shared": {"ff": shared, "limit": 3.0}}
+
+    return {
+        "architecture": "Lutosun", "vocab": 311, "width": 96, "norm": {"eps": 1e-5}, "residual_mult": 0.7, "logit_softcap": 20.0,
+        "embedding": {"scale": 2.0, "bigram": {"buckets": 401, "mul_prev": 31, "mul_cur": 7}},
+        "loop": {"start": 1, "stop": 3, "times": 3},
+        "layers": [latent(4, 16, 8, 24, 48, 40, moe(5, 2, 48, 80)), latent(3, 24, 12, 16, 40, 32, moe(6, 3, 32, 64)),
+                   latent(2, 32, 16, 40, 64, 56, None), latent(6, 8, 8, 8, 24, 24, moe(4, 1, 64, 48))],
+    }
+
+
+PRESETS["lutosun-tiny"] = _lutosun_tiny()
+
+
 def preset(name: str) -> dict:
     try:
         return copy.deepcopy(PRESETS[name])

@@ -1,6 +1,6 @@
 """Prefill and decode throughput of one architecture beside another of equal size: random weights, layers of the
 sizes real models have, the same step function for both. ``bench.py --design kakunex`` (or ``fimolix``, ``reselorn``,
-``zigelorn``, ``bipazen``) prints what this returns.
+``zigelorn``, ``bipazen``, ``lutosun``) prints what this returns.
 
 A *shape* fixes what the two share: width, query and key/value heads of 128 elements, feed-forward width, window,
 layers, vocabulary. The Kakunex model of a shape repeats (parallel, parallel, parallel, mlstm): window attention that
@@ -31,7 +31,14 @@ of 64 values with a state of 128, eight heads to a group of keys and queries, fo
 rotated elements, values of 128 and a latent of 512 per token. Every layer has a mixture of 32 experts of a quarter of the
 shape's feed-forward width, of which a token runs 4: as many multiplications as in the shape's dense feed-forward. It is
 measured beside the Zigelorn model of the shape, the other design of attention, recurrences with a matrix state and routed
-experts."""
+experts.
+
+The Lutosun model of a shape has as many layer runs as the shape has layers: all layers but the first and the last run twice, so
+``layers / 2 + 1`` of them have weights. Every layer is latent attention with the shape's query heads of 128 plain and 64 rotated elements, values
+of 128, a latent of 512 per token and a query latent of three quarters of the width; in every layer a mixture of 32 experts of
+an eighth of the shape's feed-forward width, of which a token runs 4, beside a shared expert of half the width: as many
+multiplications as in the shape's dense feed-forward. Its pair table has 65,521 rows and one. It is measured beside the Bipazen model
+of the shape, the other design of latent attention and routed experts in every layer."""
 
 from __future__ import annotations
 
@@ -131,10 +138,22 @@ def bipazen_config(s: dict) -> dict:
     return {"architecture": "Bipazen", "vocab": s["vocab"], "width": s["width"], "norm": {"eps": 1e-6}, "layers": layers}
 
 
+def lutosun_config(s: dict) -> dict:
+    latent = {"heads": s["heads"], "dim": HEAD, "rot_dim": ROTATED, "vdim": HEAD, "q_rank": s["width"] * 3 // 4, "kv_rank": LATENT,
+              "scale": (HEAD + ROTATED) ** -0.5, "rot": {"base": 1e6, "dims": ROTATED}}
+    mlp = {"kind": "moe", "router": {"experts": EXPERTS, "top": CHOSEN, "scale": 2.5}, "expert": {"ff": s["ff"] // 8, "limit": 7.0},
+           "shared": {"ff": s["ff"] // 2, "limit": 7.0}}
+    n = s["layers"] // 2 + 1
+    return {"architecture": "Lutosun", "vocab": s["vocab"], "width": s["width"], "norm": {"eps": 1e-6}, "residual_mult": 0.4,
+            "embedding": {"scale": 1.5, "bigram": {"buckets": 65521, "mul_prev": 8191, "mul_cur": 131}}, "logit_softcap": 30.0,
+            "loop": {"start": 1, "stop": n - 1, "times": 2},
+            "layers": [{"type": "latent_attention", "mixer": dict(latent), "mlp": dict(mlp)} for _ in range(n)]}
+
+
 DESIGNS = {"kakunex": kakunex_config, "fimolix": fimolix_config, "reselorn": reselorn_config, "zigelorn": zigelorn_config,
-           "bipazen": bipazen_config,
+           "bipazen": bipazen_config, "lutosun": lutosun_config,
            "qwen3": qwen3_config}
-BESIDE = {"zigelorn": "kakunex", "bipazen": "zigelorn"}  # the model a design is measured beside (default: qwen3)
+BESIDE = {"zigelorn": "kakunex", "bipazen": "zigelorn", "lutosun": "bipazen"}  # the model a design is measured beside (default: qwen3)
 
 
 def measure(config: dict, dtype: str, prefill_tokens: int, batch: int, context: int, steps: int, warmup: int, say=lambda m: None) -> dict:
