@@ -132,11 +132,10 @@ __device__ __forceinline__ float4 add_splits4(const float* __restrict__ p, int s
 // Activations of the gated feed-forward, by the number the host passes: out = act(gate) * up, in float32.
 #define MS_ACT_SILU 0
 #define MS_ACT_GELU_TANH 1
-#define MS_ACT_COUNT 2  // the activations of the form act(gate) * up, which the matrix kernels' epilogues know
 // A gated feed-forward with bounded inputs: g = min(gate, limit), u = clamp(up, -limit, limit),
 // out = g sigmoid(1.702 g) (u + 1). Not of the form act(gate) * up: it takes `limit` beside the number.
 #define MS_ACT_SWIGLU_CLAMPED 2
-#define MS_GATED_COUNT 3
+#define MS_GATED_COUNT 3  // what a gated feed-forward may run: the matrix kernels' epilogues and the activation kernels know them
 // The square of max(x, 0): only as the activation of a feed-forward without a gate.
 #define MS_ACT_RELU_SQUARED 3
 // The hyperbolic tangent: between the two steps of a small projection, never in a feed-forward's gate.

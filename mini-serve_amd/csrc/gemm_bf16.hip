@@ -86,6 +86,16 @@ __device__ __forceinline__ float activate_fast(float x, int act) {
   return x * __builtin_amdgcn_rcpf(1.f + __builtin_amdgcn_exp2f(x * -1.4426950408889634f));
 }
 
+// What a gated epilogue makes of one gate and one up value: gated_value on the same hardware functions.
+template <int ACT> __device__ __forceinline__ float gated_fast(float gate, float up, float limit) {
+  if constexpr (ACT == MS_ACT_SWIGLU_CLAMPED) {
+    const float g = fminf(gate, limit), u = fminf(fmaxf(up, -limit), limit);
+    return g * __builtin_amdgcn_rcpf(1.f + __builtin_amdgcn_exp2f(g * (-1.702f * 1.4426950408889634f))) * (u + 1.f);
+  } else {
+    return activate_fast(gate, ACT) * up;
+  }
+}
+
 // Four consecutive n of row m: the store of one accumulator fragment. MODE 0: bf16, 1: float, 2: float +=.
 // INSIDE: the tile's columns lie within the matrix and a lane's four are aligned for one store, so only
 // the row is tested (a ragged last row of tiles, which any token count makes, runs the same code as the rest:
@@ -113,13 +123,15 @@ __device__ __forceinline__ void store_fragment(void* __restrict__ C, int m, int 
 }
 
 // Gate and up fragments of the same four outputs (W holds alternating blocks of 16 gate rows and 16 up
-// rows): out[m, col ..] = act(gate) * up, bf16 with row stride ldc; `half` = N / 2 columns.
+// rows): out[m, col ..] = act(gate) * up, bf16 with row stride ldc; `half` = N / 2 columns. limit: of an activation that
+// bounds gate and up (here and below).
 template <int ACT, bool INSIDE>
-__device__ __forceinline__ void store_gated(bf16* __restrict__ out, int m, int col, int M, int half, int ldc, floatx4 gate, floatx4 up) {
+__device__ __forceinline__ void store_gated(bf16* __restrict__ out, int m, int col, int M, int half, int ldc, floatx4 gate, floatx4 up,
+                                            float limit) {
   if (m >= M || (!INSIDE && col >= half)) return;
   union { uint2 u; bf16 e[4]; } o;
 #pragma unroll
-  for (int e = 0; e < 4; ++e) o.e[e] = static_cast<bf16>(activate_fast(gate[e], ACT) * up[e]);
+  for (int e = 0; e < 4; ++e) o.e[e] = static_cast<bf16>(gated_fast<ACT>(gate[e], up[e], limit));
   *reinterpret_cast<uint2*>(out + (size_t)m * ldc + col) = o.u;
 }
 
@@ -127,14 +139,14 @@ __device__ __forceinline__ void store_gated(bf16* __restrict__ out, int m, int c
 // row and first column in fragment (0, 0). MODE as above (3 + activation: gated, C unused).
 template <int MODE, bool INSIDE, int FN, int FM>
 __device__ __forceinline__ void store_fragments(const floatx4 (&acc)[FN][FM], void* C, void* Cbase, int m, int n, int M, int N, int ldc,
-                                                bool vec_store) {
+                                                bool vec_store, float limit) {
   if constexpr (MODE >= 3) {
     const int g4 = n % 16;  // the lane's group of four columns
 #pragma unroll
     for (int i = 0; i + 1 < FN; i += 2)
 #pragma unroll
       for (int j = 0; j < FM; ++j)
-        store_gated<MODE - 3, INSIDE>((bf16*)Cbase, m + j * 16, (n - g4 + i * 16) / 2 + g4, M, N / 2, ldc, acc[i][j], acc[i + 1][j]);
+        store_gated<MODE - 3, INSIDE>((bf16*)Cbase, m + j * 16, (n - g4 + i * 16) / 2 + g4, M, N / 2, ldc, acc[i][j], acc[i + 1][j], limit);
   } else {
 #pragma unroll
     for (int i = 0; i < FN; ++i)
@@ -146,7 +158,7 @@ __device__ __forceinline__ void store_fragments(const floatx4 (&acc)[FN][FM], vo
 // The same into a tile image in LDS as bfloat16 (MODE 0, or 3 + activation: gated). at: this lane's place
 // in fragment (0, 0); row_bytes: stride of the image's rows.
 template <int MODE, int FN, int FM>
-__device__ __forceinline__ void stage_fragments(const floatx4 (&acc)[FN][FM], unsigned char* at, int row_bytes) {
+__device__ __forceinline__ void stage_fragments(const floatx4 (&acc)[FN][FM], unsigned char* at, int row_bytes, float limit) {
   union { uint2 u; bf16 e[4]; } o;
   if constexpr (MODE >= 3) {
 #pragma unroll
@@ -154,7 +166,7 @@ __device__ __forceinline__ void stage_fragments(const floatx4 (&acc)[FN][FM], un
 #pragma unroll
       for (int j = 0; j < FM; ++j) {
 #pragma unroll
-        for (int e = 0; e < 4; ++e) o.e[e] = static_cast<bf16>(activate_fast(acc[i][j][e], MODE - 3) * acc[i + 1][j][e]);
+        for (int e = 0; e < 4; ++e) o.e[e] = static_cast<bf16>(gated_fast<MODE - 3>(acc[i][j][e], acc[i + 1][j][e], limit));
         *reinterpret_cast<uint2*>(at + j * 16 * row_bytes + (i / 2) * 32) = o.u;
       }
   } else {
@@ -346,7 +358,7 @@ template <int BM, int BN, int KS, int STAGES, int BLOCKS_PER_CU, int WR = 2, int
 __global__ __launch_bounds__(WR * WC * WAVE, BLOCKS_PER_CU) void gemm_bf16_dma_kernel(const bf16* __restrict__ X, const bf16* __restrict__ W,
                                                                void* __restrict__ Cbase, int mode, int M, int N, int Kfull,
                                                                int ldx, int ldc, int k_per, size_t c_split_stride, int xcd_rows,
-                                                               int band_cols) {
+                                                               int band_cols, float limit) {
   constexpr int NW = WR * WC;
   constexpr int WM = BM / WR, WN = BN / WC;
   constexpr int FM = WM / 16, FN = WN / 16;
@@ -458,10 +470,11 @@ __global__ __launch_bounds__(WR * WC * WAVE, BLOCKS_PER_CU) void gemm_bf16_dma_k
       ((mode == 0 && BM * OUT_ROW <= STAGES * STAGE_BYTES) || (mode >= 3 && BM * GATED_ROW <= STAGES * STAGE_BYTES))) {
     __syncthreads();  // every wave has read the last slab's fragments
     const int row_bytes = mode == 0 ? OUT_ROW : GATED_ROW;
-    static_assert(MS_ACT_COUNT == 2, "one case per activation below");
-    if (mode == 0) stage_fragments<0, FN, FM>(acc, lds + (wm + r) * OUT_ROW + (wn + g * 4) * 2, OUT_ROW);
-    else if (mode == 3) stage_fragments<3, FN, FM>(acc, lds + (wm + r) * GATED_ROW + (wn / 2 + g * 4) * 2, GATED_ROW);
-    else stage_fragments<4, FN, FM>(acc, lds + (wm + r) * GATED_ROW + (wn / 2 + g * 4) * 2, GATED_ROW);
+    static_assert(MS_GATED_COUNT == 3, "one case per activation below");
+    if (mode == 0) stage_fragments<0, FN, FM>(acc, lds + (wm + r) * OUT_ROW + (wn + g * 4) * 2, OUT_ROW, limit);
+    else if (mode == 3) stage_fragments<3, FN, FM>(acc, lds + (wm + r) * GATED_ROW + (wn / 2 + g * 4) * 2, GATED_ROW, limit);
+    else if (mode == 4) stage_fragments<4, FN, FM>(acc, lds + (wm + r) * GATED_ROW + (wn / 2 + g * 4) * 2, GATED_ROW, limit);
+    else stage_fragments<5, FN, FM>(acc, lds + (wm + r) * GATED_ROW + (wn / 2 + g * 4) * 2, GATED_ROW, limit);
     __syncthreads();
     const int chunks = (row_bytes - 16) / 16;  // 16-byte chunks of an output row of the tile
     bf16* out = (bf16*)Cbase + (size_t)m0 * ldc + (mode == 0 ? n0 : n0 / 2);
@@ -475,19 +488,21 @@ __global__ __launch_bounds__(WR * WC * WAVE, BLOCKS_PER_CU) void gemm_bf16_dma_k
   const int m = m0 + wm + r, n = n0 + wn + g * 4;
   if (inside) {
     switch (mode) {
-      case 0: store_fragments<0, true, FN, FM>(acc, C, Cbase, m, n, M, N, ldc, vec_store); break;
-      case 1: store_fragments<1, true, FN, FM>(acc, C, Cbase, m, n, M, N, ldc, vec_store); break;
-      case 2: store_fragments<2, true, FN, FM>(acc, C, Cbase, m, n, M, N, ldc, vec_store); break;
-      case 3: store_fragments<3, true, FN, FM>(acc, C, Cbase, m, n, M, N, ldc, vec_store); break;
-      default: store_fragments<4, true, FN, FM>(acc, C, Cbase, m, n, M, N, ldc, vec_store); break;
+      case 0: store_fragments<0, true, FN, FM>(acc, C, Cbase, m, n, M, N, ldc, vec_store, limit); break;
+      case 1: store_fragments<1, true, FN, FM>(acc, C, Cbase, m, n, M, N, ldc, vec_store, limit); break;
+      case 2: store_fragments<2, true, FN, FM>(acc, C, Cbase, m, n, M, N, ldc, vec_store, limit); break;
+      case 3: store_fragments<3, true, FN, FM>(acc, C, Cbase, m, n, M, N, ldc, vec_store, limit); break;
+      case 4: store_fragments<4, true, FN, FM>(acc, C, Cbase, m, n, M, N, ldc, vec_store, limit); break;
+      default: store_fragments<5, true, FN, FM>(acc, C, Cbase, m, n, M, N, ldc, vec_store, limit); break;
     }
   } else {
     switch (mode) {
-      case 0: store_fragments<0, false, FN, FM>(acc, C, Cbase, m, n, M, N, ldc, vec_store); break;
-      case 1: store_fragments<1, false, FN, FM>(acc, C, Cbase, m, n, M, N, ldc, vec_store); break;
-      case 2: store_fragments<2, false, FN, FM>(acc, C, Cbase, m, n, M, N, ldc, vec_store); break;
-      case 3: store_fragments<3, false, FN, FM>(acc, C, Cbase, m, n, M, N, ldc, vec_store); break;
-      default: store_fragments<4, false, FN, FM>(acc, C, Cbase, m, n, M, N, ldc, vec_store); break;
+      case 0: store_fragments<0, false, FN, FM>(acc, C, Cbase, m, n, M, N, ldc, vec_store, limit); break;
+      case 1: store_fragments<1, false, FN, FM>(acc, C, Cbase, m, n, M, N, ldc, vec_store, limit); break;
+      case 2: store_fragments<2, false, FN, FM>(acc, C, Cbase, m, n, M, N, ldc, vec_store, limit); break;
+      case 3: store_fragments<3, false, FN, FM>(acc, C, Cbase, m, n, M, N, ldc, vec_store, limit); break;
+      case 4: store_fragments<4, false, FN, FM>(acc, C, Cbase, m, n, M, N, ldc, vec_store, limit); break;
+      default: store_fragments<5, false, FN, FM>(acc, C, Cbase, m, n, M, N, ldc, vec_store, limit); break;
     }
   }
 }
@@ -533,11 +548,11 @@ __device__ __forceinline__ floatx4 wide_acc() {
 // number: as gate and up. m: this lane's row in row block 0; nb: the wave tile's first column; g: the
 // lane's group of four columns.
 template <int MODE, bool INSIDE, int P, int J>
-__device__ __forceinline__ void wide_store(void* C, void* Cbase, int m, int nb, int g, int M, int N, int ldc, bool vec_store) {
+__device__ __forceinline__ void wide_store(void* C, void* Cbase, int m, int nb, int g, int M, int N, int ldc, bool vec_store, float limit) {
   const floatx4 a = wide_acc<(2 * P) * 8 + J>(), b = wide_acc<(2 * P + 1) * 8 + J>();
   const int row = m + J * 16;
   if constexpr (MODE >= 3) {
-    store_gated<MODE - 3, INSIDE>((bf16*)Cbase, row, nb / 2 + P * 16 + g * 4, M, N / 2, ldc, a, b);
+    store_gated<MODE - 3, INSIDE>((bf16*)Cbase, row, nb / 2 + P * 16 + g * 4, M, N / 2, ldc, a, b, limit);
   } else {
     store_fragment<MODE, INSIDE>(C, row, nb + (2 * P) * 16 + g * 4, M, N, ldc, a, vec_store);
     store_fragment<MODE, INSIDE>(C, row, nb + (2 * P + 1) * 16 + g * 4, M, N, ldc, b, vec_store);
@@ -546,8 +561,8 @@ __device__ __forceinline__ void wide_store(void* C, void* Cbase, int m, int nb, 
 
 template <int MODE, bool INSIDE, int... I>
 __device__ __forceinline__ void wide_stores(std::integer_sequence<int, I...>, void* C, void* Cbase, int m, int nb, int g, int M, int N,
-                                            int ldc, bool vec_store) {
-  (wide_store<MODE, INSIDE, I / 8, I % 8>(C, Cbase, m, nb, g, M, N, ldc, vec_store), ...);
+                                            int ldc, bool vec_store, float limit) {
+  (wide_store<MODE, INSIDE, I / 8, I % 8>(C, Cbase, m, nb, g, M, N, ldc, vec_store, limit), ...);
 }
 
 // The same through LDS, for bfloat16 outputs of tiles whose columns lie inside the matrix, with 16-byte
@@ -557,14 +572,14 @@ __device__ __forceinline__ void wide_stores(std::integer_sequence<int, I...>, vo
 // cost four times the requests at the L2, and a tile's stores then took as long as ten slabs of products.
 constexpr int WIDE_STAGED_BYTES = 128 * (256 + 16);  // per wave: 128 rows of 128 bf16
 template <int MODE, int P, int J>
-__device__ __forceinline__ void wide_stage(unsigned char* part, int r, int g) {
+__device__ __forceinline__ void wide_stage(unsigned char* part, int r, int g, float limit) {
   const floatx4 a = wide_acc<(2 * P) * 8 + J>(), b = wide_acc<(2 * P + 1) * 8 + J>();
   constexpr int STRIDE = (MODE >= 3 ? 128 : 256) + 16;
   unsigned char* row = part + (J * 16 + r) * STRIDE;
   union { uint2 u; bf16 e[4]; } o;
   if constexpr (MODE >= 3) {
 #pragma unroll
-    for (int e = 0; e < 4; ++e) o.e[e] = static_cast<bf16>(activate_fast(a[e], MODE - 3) * b[e]);
+    for (int e = 0; e < 4; ++e) o.e[e] = static_cast<bf16>(gated_fast<MODE - 3>(a[e], b[e], limit));
     *reinterpret_cast<uint2*>(row + (P * 16 + g * 4) * 2) = o.u;
   } else {
 #pragma unroll
@@ -576,13 +591,13 @@ __device__ __forceinline__ void wide_stage(unsigned char* part, int r, int g) {
   }
 }
 template <int MODE, int... I>
-__device__ __forceinline__ void wide_stage_all(std::integer_sequence<int, I...>, unsigned char* part, int r, int g) {
-  (wide_stage<MODE, I / 8, I % 8>(part, r, g), ...);
+__device__ __forceinline__ void wide_stage_all(std::integer_sequence<int, I...>, unsigned char* part, int r, int g, float limit) {
+  (wide_stage<MODE, I / 8, I % 8>(part, r, g, limit), ...);
 }
 // out: the wave tile's first output element; MODE 0 or 3 + an MS_ACT_* number.
 template <int MODE>
-__device__ __forceinline__ void wide_store_staged(bf16* __restrict__ out, int ldc, int rows, unsigned char* part, int lane) {
-  wide_stage_all<MODE>(std::make_integer_sequence<int, 32>{}, part, lane % 16, lane / 16);
+__device__ __forceinline__ void wide_store_staged(bf16* __restrict__ out, int ldc, int rows, unsigned char* part, int lane, float limit) {
+  wide_stage_all<MODE>(std::make_integer_sequence<int, 32>{}, part, lane % 16, lane / 16, limit);
   constexpr int CHUNKS = MODE >= 3 ? 8 : 16, STRIDE = CHUNKS * 16 + 16, ROWS = 64 / CHUNKS;
   const int lrow = lane / CHUNKS, ch = lane % CHUNKS;
 #pragma unroll 8
@@ -595,15 +610,17 @@ __device__ __forceinline__ void wide_store_staged(bf16* __restrict__ out, int ld
 
 // The mode is told apart once, not per fragment: each mode's stores are one straight run of code.
 template <bool INSIDE>
-__device__ __forceinline__ void wide_epilogue(void* C, void* Cbase, int mode, int m, int nb, int g, int M, int N, int ldc, bool vec_store) {
+__device__ __forceinline__ void wide_epilogue(void* C, void* Cbase, int mode, int m, int nb, int g, int M, int N, int ldc, bool vec_store,
+                                              float limit) {
   constexpr auto all = std::make_integer_sequence<int, 32>{};
-  static_assert(MS_ACT_COUNT == 2, "one case per activation below");
+  static_assert(MS_GATED_COUNT == 3, "one case per activation below");
   switch (mode) {
-    case 0: wide_stores<0, INSIDE>(all, C, Cbase, m, nb, g, M, N, ldc, vec_store); break;
-    case 1: wide_stores<1, INSIDE>(all, C, Cbase, m, nb, g, M, N, ldc, vec_store); break;
-    case 2: wide_stores<2, INSIDE>(all, C, Cbase, m, nb, g, M, N, ldc, vec_store); break;
-    case 3: wide_stores<3, INSIDE>(all, C, Cbase, m, nb, g, M, N, ldc, vec_store); break;
-    default: wide_stores<4, INSIDE>(all, C, Cbase, m, nb, g, M, N, ldc, vec_store); break;
+    case 0: wide_stores<0, INSIDE>(all, C, Cbase, m, nb, g, M, N, ldc, vec_store, limit); break;
+    case 1: wide_stores<1, INSIDE>(all, C, Cbase, m, nb, g, M, N, ldc, vec_store, limit); break;
+    case 2: wide_stores<2, INSIDE>(all, C, Cbase, m, nb, g, M, N, ldc, vec_store, limit); break;
+    case 3: wide_stores<3, INSIDE>(all, C, Cbase, m, nb, g, M, N, ldc, vec_store, limit); break;
+    case 4: wide_stores<4, INSIDE>(all, C, Cbase, m, nb, g, M, N, ldc, vec_store, limit); break;
+    default: wide_stores<5, INSIDE>(all, C, Cbase, m, nb, g, M, N, ldc, vec_store, limit); break;
   }
 }
 
@@ -620,7 +637,7 @@ __device__ __forceinline__ void wide_epilogue(void* C, void* Cbase, int mode, in
 __global__ __launch_bounds__(256, 1) void gemm_bf16_wide_kernel(const bf16* __restrict__ X, const bf16* __restrict__ W,
                                                                 void* __restrict__ Cbase, int mode, int M, int N, int Kfull,
                                                                 int ldx, int ldc, int k_per, size_t c_split_stride,
-                                                                int xcd_rows, int band_cols, int items) {
+                                                                int xcd_rows, int band_cols, int items, float limit) {
   constexpr int BM = 256, BN = 256, KS = 64, ROW_BYTES = KS * 2, STAGE_BYTES = (BM + BN) * ROW_BYTES;
   static_assert(STAGE_BYTES == 0x10000, "the loop flips stages by 64 KB");
   extern __shared__ __attribute__((aligned(1024))) unsigned char lds[];  // 2 * STAGE_BYTES, and 4 * WIDE_STAGED_BYTES for the stores
@@ -829,15 +846,16 @@ __global__ __launch_bounds__(256, 1) void gemm_bf16_wide_kernel(const bf16* __re
   if (inside && (mode == 0 || mode >= 3) && ldc % 8 == 0 && (size_t)Cbase % 16 == 0) {
     unsigned char* part = lds + wave * WIDE_STAGED_BYTES;
     const int rows = M - (m0 + wm);  // of the wave tile's 128 that exist
-    static_assert(MS_ACT_COUNT == 2, "one case per activation below");
-    if (mode == 0) wide_store_staged<0>((bf16*)Cbase + (size_t)(m0 + wm) * ldc + n0 + wn, ldc, rows, part, lane_now);
-    else if (mode == 3) wide_store_staged<3>((bf16*)Cbase + (size_t)(m0 + wm) * ldc + (n0 + wn) / 2, ldc, rows, part, lane_now);
-    else wide_store_staged<4>((bf16*)Cbase + (size_t)(m0 + wm) * ldc + (n0 + wn) / 2, ldc, rows, part, lane_now);
+    static_assert(MS_GATED_COUNT == 3, "one case per activation below");
+    if (mode == 0) wide_store_staged<0>((bf16*)Cbase + (size_t)(m0 + wm) * ldc + n0 + wn, ldc, rows, part, lane_now, limit);
+    else if (mode == 3) wide_store_staged<3>((bf16*)Cbase + (size_t)(m0 + wm) * ldc + (n0 + wn) / 2, ldc, rows, part, lane_now, limit);
+    else if (mode == 4) wide_store_staged<4>((bf16*)Cbase + (size_t)(m0 + wm) * ldc + (n0 + wn) / 2, ldc, rows, part, lane_now, limit);
+    else wide_store_staged<5>((bf16*)Cbase + (size_t)(m0 + wm) * ldc + (n0 + wn) / 2, ldc, rows, part, lane_now, limit);
     __syncthreads();  // the next item's loads go where other waves may still be reading their parts
   } else if (inside) {
-    wide_epilogue<true>(C, Cbase, mode, m0 + wm + r, n0 + wn, g, M, N, ldc, vec_store);
+    wide_epilogue<true>(C, Cbase, mode, m0 + wm + r, n0 + wn, g, M, N, ldc, vec_store, limit);
   } else {
-    wide_epilogue<false>(C, Cbase, mode, m0 + wm + r, n0 + wn, g, M, N, ldc, vec_store);
+    wide_epilogue<false>(C, Cbase, mode, m0 + wm + r, n0 + wn, g, M, N, ldc, vec_store, limit);
   }
   }
 }
@@ -1063,7 +1081,7 @@ static TileWalk tile_walk(int M, int N, int K, int BM, int BN) {
 
 template <int BM, int BN, int KS, int STAGES, int BLOCKS_PER_CU, int WR = 2, int WC = 2>
 static int launch_dma(const bf16* x, const bf16* w, void* C, int mode, int M, int N, int K, int ldx, int ldc, int k_per,
-                      size_t stride, int splits, hipStream_t st) {
+                      size_t stride, int splits, hipStream_t st, float limit = 0.f) {
   constexpr int lds_bytes = STAGES * (BM + BN) * KS * 2;
   static bool ready = false;  // more than 64 KB of LDS has to be asked for once per kernel
   if (!ready) {
@@ -1075,7 +1093,7 @@ static int launch_dma(const bf16* x, const bf16* w, void* C, int mode, int M, in
   const long blocks = (long)((N + BN - 1) / BN) * ((M + BM - 1) / BM) * splits;
   if (blocks > 0x7fffffffL) return MS_BAD_ARG;
   const TileWalk walk = tile_walk(M, N, K, BM, BN);
-  gemm_bf16_dma_kernel<BM, BN, KS, STAGES, BLOCKS_PER_CU, WR, WC><<<(unsigned)blocks, WR * WC * WAVE, lds_bytes, st>>>(x, w, C, mode, M, N, K, ldx, ldc, k_per, stride, walk.xcd_rows, walk.band_cols);
+  gemm_bf16_dma_kernel<BM, BN, KS, STAGES, BLOCKS_PER_CU, WR, WC><<<(unsigned)blocks, WR * WC * WAVE, lds_bytes, st>>>(x, w, C, mode, M, N, K, ldx, ldc, k_per, stride, walk.xcd_rows, walk.band_cols, limit);
   return launch_status();
 }
 
@@ -1097,10 +1115,10 @@ static int compute_units() {
 // The 256 x 256 tile: four waves with the loop written out where every split has at least two slabs and a
 // tile's rows lie within 4 GB of its first (the loop adds 32-bit offsets to a tile's base), else 128 x 128 tiles.
 static int launch_256(const bf16* x, const bf16* w, void* C, int mode, int M, int N, int K, int ldx, int ldc, int k_per,
-                      size_t stride, int splits, hipStream_t st) {
+                      size_t stride, int splits, hipStream_t st, float limit = 0.f) {
   const int last_slabs = (K - (splits - 1) * k_per) / BK;  // of the last split, the shortest
   if (last_slabs < 2 || k_per < 2 * BK || !wide_tile_offsets_fit(ldx, K))
-    return launch_dma<128, 128, BK, 2, 2>(x, w, C, mode, M, N, K, ldx, ldc, k_per, stride, splits, st);
+    return launch_dma<128, 128, BK, 2, 2>(x, w, C, mode, M, N, K, ldx, ldc, k_per, stride, splits, st, limit);
   constexpr int lds_bytes = 4 * WIDE_STAGED_BYTES;  // the loop's two stages are 128 KB of it
   static_assert(lds_bytes >= 2 * (256 + 256) * BK * 2 && lds_bytes <= 160 * 1024, "LDS of the wide tile");
   static bool ready = false;
@@ -1114,7 +1132,7 @@ static int launch_256(const bf16* x, const bf16* w, void* C, int mode, int M, in
   const TileWalk walk = tile_walk(M, N, K, 256, 256);
   const int cus = compute_units();
   const int blocks = items <= cus ? (int)items : cus / 8 * 8;
-  gemm_bf16_wide_kernel<<<(unsigned)blocks, 256, lds_bytes, st>>>(x, w, C, mode, M, N, K, ldx, ldc, k_per, stride, walk.xcd_rows, walk.band_cols, (int)items);
+  gemm_bf16_wide_kernel<<<(unsigned)blocks, 256, lds_bytes, st>>>(x, w, C, mode, M, N, K, ldx, ldc, k_per, stride, walk.xcd_rows, walk.band_cols, (int)items, limit);
   return launch_status();
 }
 
@@ -1180,13 +1198,13 @@ static int pick_tile_cols(int M, int N, int K, int splits, bool pairs, float* pr
 }
 
 static int launch_picked(int cols, const bf16* x, const bf16* w, void* C, int mode, int M, int N, int K, int ldx, int ldc,
-                         int k_per, size_t stride, int splits, hipStream_t st) {
+                         int k_per, size_t stride, int splits, hipStream_t st, float limit = 0.f) {
   switch (cols) {
-    case 256: return launch_256(x, w, C, mode, M, N, K, ldx, ldc, k_per, stride, splits, st);
-    case 192: return launch_dma<128, 192, BK, 2, 2>(x, w, C, mode, M, N, K, ldx, ldc, k_per, stride, splits, st);
-    case 160: return launch_dma<128, 160, BK, 2, 2>(x, w, C, mode, M, N, K, ldx, ldc, k_per, stride, splits, st);
-    case 64: return launch_dma<128, 64, BK, 2, 2>(x, w, C, mode, M, N, K, ldx, ldc, k_per, stride, splits, st);
-    default: return launch_dma<128, 128, BK, 2, 2>(x, w, C, mode, M, N, K, ldx, ldc, k_per, stride, splits, st);
+    case 256: return launch_256(x, w, C, mode, M, N, K, ldx, ldc, k_per, stride, splits, st, limit);
+    case 192: return launch_dma<128, 192, BK, 2, 2>(x, w, C, mode, M, N, K, ldx, ldc, k_per, stride, splits, st, limit);
+    case 160: return launch_dma<128, 160, BK, 2, 2>(x, w, C, mode, M, N, K, ldx, ldc, k_per, stride, splits, st, limit);
+    case 64: return launch_dma<128, 64, BK, 2, 2>(x, w, C, mode, M, N, K, ldx, ldc, k_per, stride, splits, st, limit);
+    default: return launch_dma<128, 128, BK, 2, 2>(x, w, C, mode, M, N, K, ldx, ldc, k_per, stride, splits, st, limit);
   }
 }
 
@@ -1312,7 +1330,7 @@ extern "C" int ms_gemm_bf16_small(const void* X, const void* W, float* partials,
 template <int MB, int ACT>
 __global__ __launch_bounds__(512) void gemm_bf16_small_gated_kernel(const bf16* __restrict__ X, const bf16* __restrict__ W,
                                                                     bf16* __restrict__ out, int M, int inter, int K,
-                                                                    int ldx) {
+                                                                    int ldx, float limit) {
   __shared__ float red[8][MB][WAVE][4];
   const int tid = threadIdx.x, wave = tid / WAVE, lane = tid % WAVE;
   const int r = lane % 16, g = lane / 16;
@@ -1367,21 +1385,28 @@ __global__ __launch_bounds__(512) void gemm_bf16_small_gated_kernel(const bf16* 
         gate += red[w][i][lane][e];
         up += red[4 + w][i][lane][e];
       }
-      o.e[e] = static_cast<bf16>(activate(gate, ACT) * up);
+      o.e[e] = static_cast<bf16>(gated_value(gate, up, ACT, limit));
     }
     *reinterpret_cast<uint2*>(out + (size_t)m * inter + blockIdx.x * 16 + g * 4) = o.u;
   }
 }
 
 // out bf16 [M, inter] = act(X gate^T) * (X up^T) (act: an MS_ACT_* number) for W [2 inter, K] with gate and up rows in
-// alternating blocks of 16. MS_UNSUPPORTED for shapes no fused kernel takes (the caller then runs the
+// alternating blocks of 16; limit: the bound of MS_ACT_SWIGLU_CLAMPED. MS_UNSUPPORTED for shapes no fused kernel takes (the caller then runs the
 // product and the activation separately): K no multiple of 64 (of 256 for M <= 64) or unaligned rows,
 // more K than a block of the small kernel should walk alone (2048 up to 16 rows, 1024 up to 32), 33 to
 // 64 rows of a large matrix (those stream the weights with K split over blocks).
+#define SMALL_GATED_ACT(MB, ACT) gemm_bf16_small_gated_kernel<MB, ACT><<<inter / 16, 512, 0, st>>>(x, w, (bf16*)out, M, inter, K, ldx, limit)
+#define SMALL_GATED(MB)                                                          \
+  do {                                                                           \
+    if (act == MS_ACT_SILU) SMALL_GATED_ACT(MB, MS_ACT_SILU);                    \
+    else if (act == MS_ACT_GELU_TANH) SMALL_GATED_ACT(MB, MS_ACT_GELU_TANH);     \
+    else SMALL_GATED_ACT(MB, MS_ACT_SWIGLU_CLAMPED);                             \
+  } while (0)
 extern "C" int ms_gemm_bf16_gated(const void* X, const void* W, void* out, int M, int inter, int K, int ldx, int act,
-                                  hipStream_t st) {
+                                  float limit, hipStream_t st) {
   if (M <= 0 || inter <= 0) return MS_OK;
-  if (K <= 0 || ldx < K || act < 0 || act >= MS_ACT_COUNT) return MS_BAD_ARG;
+  if (K <= 0 || ldx < K || act < 0 || act >= MS_GATED_COUNT || (act == MS_ACT_SWIGLU_CLAMPED && !(limit > 0.f))) return MS_BAD_ARG;
   const int gated = 3 + act;  // the tile kernel's mode
   if (inter % 16 || ldx % 8) return MS_UNSUPPORTED;
   const bf16* x = (const bf16*)X;
@@ -1389,8 +1414,7 @@ extern "C" int ms_gemm_bf16_gated(const void* X, const void* W, void* out, int M
   const int N = 2 * inter;
   if (M <= 16) {
     if (K % SMALL_SLAB || K / SMALL_SLAB > 8) return MS_UNSUPPORTED;
-    if (act == MS_ACT_SILU) gemm_bf16_small_gated_kernel<1, MS_ACT_SILU><<<inter / 16, 512, 0, st>>>(x, w, (bf16*)out, M, inter, K, ldx);
-    else gemm_bf16_small_gated_kernel<1, MS_ACT_GELU_TANH><<<inter / 16, 512, 0, st>>>(x, w, (bf16*)out, M, inter, K, ldx);
+    SMALL_GATED(1);
     return launch_status();
   }
   if (M <= 32 && K % SMALL_SLAB == 0 && K / SMALL_SLAB <= 4) {
@@ -1398,8 +1422,7 @@ extern "C" int ms_gemm_bf16_gated(const void* X, const void* W, void* out, int M
     // slabs covers K (each wave then holds its slab of every row at once): 7.8 against 9.2 us at the
     // 0.6B shape. Larger K streams the weights with K split over blocks and runs the activation as a
     // kernel of its own.
-    if (act == MS_ACT_SILU) gemm_bf16_small_gated_kernel<2, MS_ACT_SILU><<<inter / 16, 512, 0, st>>>(x, w, (bf16*)out, M, inter, K, ldx);
-    else gemm_bf16_small_gated_kernel<2, MS_ACT_GELU_TANH><<<inter / 16, 512, 0, st>>>(x, w, (bf16*)out, M, inter, K, ldx);
+    SMALL_GATED(2);
     return launch_status();
   }
   if (K % BK) return MS_UNSUPPORTED;
@@ -1407,16 +1430,18 @@ extern "C" int ms_gemm_bf16_gated(const void* X, const void* W, void* out, int M
     // 33 to 64 rows (one row of 64 x 64 tiles): the tile kernel with the activation in its epilogue
     // where the matrix is small enough that K need not be split to keep the chip busy.
     if (M > 32 && (long)N * K * 2 <= (16L << 20) && (N + 63) / 64 >= 96)
-      return launch_dma<64, 64, BK, 2, 4>(x, w, out, gated, M, N, K, ldx, inter, K, 0, 1, st);
+      return launch_dma<64, 64, BK, 2, 4>(x, w, out, gated, M, N, K, ldx, inter, K, 0, 1, st, limit);
     return MS_UNSUPPORTED;
   }
   const long big = (long)((M + 127) / 128) * ((N + 127) / 128);
-  if (big >= 256) return launch_picked(pick_tile_cols(M, N, K, 1, true), x, w, out, gated, M, N, K, ldx, inter, K, 0, 1, st);
+  if (big >= 256) return launch_picked(pick_tile_cols(M, N, K, 1, true), x, w, out, gated, M, N, K, ldx, inter, K, 0, 1, st, limit);
   // 64 x 64 tiles from 128 of them on: half the CUs without a split of K still beat the split product
   // followed by the activation kernel (10.2 against 11.8 to 13.1 us at 65 to 128 rows of the 0.6B shape).
-  if ((long)((M + 63) / 64) * ((N + 63) / 64) >= 128) return launch_dma<64, 64, BK, 2, 4>(x, w, out, gated, M, N, K, ldx, inter, K, 0, 1, st);
+  if ((long)((M + 63) / 64) * ((N + 63) / 64) >= 128) return launch_dma<64, 64, BK, 2, 4>(x, w, out, gated, M, N, K, ldx, inter, K, 0, 1, st, limit);
   return MS_UNSUPPORTED;  // too few tiles without a split of K
 }
+#undef SMALL_GATED
+#undef SMALL_GATED_ACT
 
 // Splits of K for the tile kernel when the caller takes partial sums and 128 x 128 tiles alone would
 // not fill the chip. Up to 512 rows (large decode batches, short portions of prompts) the

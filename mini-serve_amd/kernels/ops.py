@@ -64,7 +64,7 @@ _SIGNATURES = {
                                     _c_void, _c_void, _c_int, _c_int, _c_void, _c_void, _c_void, _c_void],
     "ms_gated_recurrence_chunk_tokens": [],
     "ms_gated_recurrence_chunk_max_dim": [],
-    "ms_gemm_bf16_gated": [_c_void, _c_void, _c_void, _c_int, _c_int, _c_int, _c_int, _c_int, _c_void],
+    "ms_gemm_bf16_gated": [_c_void, _c_void, _c_void, _c_int, _c_int, _c_int, _c_int, _c_int, _c_float, _c_void],
     "ms_cast": [_c_void, _c_int, _c_void, _c_int, _c_ll, _c_void],
     "ms_rope_table": [_c_void, _c_void, _c_void, _c_int, _c_int, _c_float, _c_void],
     "ms_qk_norm_rope_store": [_c_void, _c_void, _c_int, _c_ll, _c_void, _c_int, _c_int, _c_void, _c_void, _c_void,
@@ -445,10 +445,10 @@ def gated_linear(x: torch.Tensor, gate_up: torch.Tensor, activation: str = "silu
     if gate_up.shape[1] != k or gate_up.shape[0] % 2:
         raise ValueError(f"gated_linear: x is [{m}, {k}], gate_up is {tuple(gate_up.shape)}")
     inter = gate_up.shape[0] // 2
-    if block == GATE_BLOCK and gate_up.dtype == BF16 and out_dtype == BF16 and m > 0 and activation not in ACTIVATIONS_WITH_LIMIT:
+    if block == GATE_BLOCK and gate_up.dtype == BF16 and out_dtype == BF16 and m > 0:
         xa = cast(x, BF16)
         out = torch.empty((m, inter), dtype=BF16, device=x.device)
-        rc = library().ms_gemm_bf16_gated(xa.data_ptr(), gate_up.data_ptr(), out.data_ptr(), m, inter, k, k, act, _stream())
+        rc = library().ms_gemm_bf16_gated(xa.data_ptr(), gate_up.data_ptr(), out.data_ptr(), m, inter, k, k, act, float(limit or 0.0), _stream())
         if rc == 0:
             return out
         if rc != 2:  # 2: no fused kernel for this shape

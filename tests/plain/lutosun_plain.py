@@ -171,6 +171,11 @@ def run_plan(cfg):
     return [(i, None) for i in range(a)] + looped + [(i, None) for i in range(b, n)]
 
 
+def begin_pass(x, start, steps, t):
+    """What joins the stream ``x`` ahead of pass ``t``: its own vector, and from the second pass on the embedding's output."""
+    return x + steps[t] + (start if t > 0 else 0.0)
+
+
 def bound_logits(z, cap):
     return cap * np.tanh(z / cap) if cap else z
 
@@ -199,7 +204,7 @@ def _forward(cfg, weights, tokens, return_layers, watch):
     for run, (i, t) in enumerate(run_plan(cfg)):
         layer, p = cfg["layers"][i], f"l{i}."
         if t is not None:
-            x = x + (start if t > 0 else 0.0) + weights["loop.step"][t]
+            x = begin_pass(x, start, weights["loop.step"], t)
         if layer["type"] != "latent_attention":
             raise ValueError(f"layer {i}: unknown mixer {layer['type']!r}")
         h = _round(layer_norm(x, weights[p + "norm1"], weights[p + "norm1.b"], eps))

@@ -142,23 +142,33 @@ GATED_TILES = {(3000, 128, 4096): (128, 128), (200, 1024, 3072): (64, 64), (2048
                (2048, 512, 12288): (256, 256), (4090, 512, 4080): (256, 256)}  # the last: ragged in both directions
 
 
-@pytest.mark.parametrize("act", ["silu", "gelu_tanh"])
+def gated_values(act, gate, up, limit):
+    if act != "swiglu_clamped":
+        return activation(act, gate) * up
+    g = gate.clamp(max=limit)
+    return g * torch.sigmoid(1.702 * g) * (up.clamp(-limit, limit) + 1)
+
+
+@pytest.mark.parametrize("act", ["silu", "gelu_tanh", "swiglu_clamped"])
 @pytest.mark.parametrize("dtype", [F32, BF16])
 @pytest.mark.parametrize("m,k,inter", GATED)
 def test_gated_linear(ops, dtype, m, k, inter, act):
     x = rand((m, k), dtype, 70)
     gate, up = rand((inter, k), dtype, 71, 0.05), rand((inter, k), dtype, 72, 0.05)
     g, u = x.double() @ gate.double().T, x.double() @ up.double().T
-    want = activation(act, g) * u
+    limit = float(g.std()) if act == "swiglu_clamped" else None  # about one in three values lies beyond it
+    want = gated_values(act, g, u, limit)
     w = ops.interleave_gate_up(gate, up)
     assert w.shape == (2 * inter, k) and torch.equal(w[:16], gate[:16]) and torch.equal(w[16:32], up[:16])
     if (m, k, inter) in GATED_TILES:
         assert ops.tile_shape(m, 2 * inter, k, gated=True) == GATED_TILES[(m, k, inter)], "pick other sizes for this tile shape"
-    got = ops.gated_linear(x, w, act, out_dtype=dtype, block=ops.GATE_BLOCK)
+    got = ops.gated_linear(x, w, act, out_dtype=dtype, block=ops.GATE_BLOCK, limit=limit)
     assert got.shape == (m, inter) and got.dtype == dtype
     close(got, want, 1e-5 if dtype == F32 else 8e-3, f"gated {m}x{k}->{inter}")
-    # and with the plain layout (gates, then ups) through the two-kernel path
-    close(ops.gated_linear(x, torch.cat((gate, up)).contiguous(), act, out_dtype=dtype), want, 1e-5 if dtype == F32 else 8e-3, "halves")
+    # and with the plain layout (gates, then ups) through the two-kernel path, which rounds gate and up as well: where the limits cap
+    # the largest results, three roundings of 2^-8 at gate, up and result next to a power of two weigh 2.8 of them together
+    tol = 1e-5 if dtype == F32 else (8e-3 if limit is None else 2.8 * 2.0 ** -8)
+    close(ops.gated_linear(x, torch.cat((gate, up)).contiguous(), act, out_dtype=dtype, limit=limit), want, tol, "halves")
 
 
 # ------------------------------------------------------------------------------------------ matrix products
@@ -263,10 +273,11 @@ def test_wide_tile_at_random_sizes(ops, seed):
         if gated:
             pairs = want.view(m, n // 32, 2, 16)
             g, u = pairs[:, :, 0].reshape(m, n // 2), pairs[:, :, 1].reshape(m, n // 2)
-            for act in ("silu", "gelu_tanh"):
-                a = ops.gated_linear(x, w, act, out_dtype=BF16, block=ops.GATE_BLOCK)
-                close(a, activation(act, g) * u, 8e-3, f"{what} {act}")
-                assert torch.equal(a, ops.gated_linear(x, w, act, out_dtype=BF16, block=ops.GATE_BLOCK)), what
+            for act in ("silu", "gelu_tanh", "swiglu_clamped"):
+                limit = float(g.std())
+                a = ops.gated_linear(x, w, act, out_dtype=BF16, block=ops.GATE_BLOCK, limit=limit)
+                close(a, gated_values(act, g, u, limit), 8e-3, f"{what} {act}")
+                assert torch.equal(a, ops.gated_linear(x, w, act, out_dtype=BF16, block=ops.GATE_BLOCK, limit=limit)), what
             continue
         a = ops.linear(x, w, out_dtype=BF16)
         close(a, want, 5e-3, f"{what} -> bf16")
