@@ -27,8 +27,8 @@ extern "C" int ms_embed(const int* ids, const void* table, int table_is_bf16, fl
 // in its sequence: r = (previous * mul_prev + ids[t] * mul_cur) mod buckets, and r = buckets for a sequence's first token.
 // `pairs` may be nullptr (no such row). The token before a row's first one comes from the request's state, last[state_slots[row]];
 // the block that reads it leaves the row's last token there for the next step. `keep` (nullable) receives the same rows
-// once more. mul_prev and mul_cur lie in [0, buckets). One block per token.
-template <typename TW>
+// once more. mul_prev and mul_cur lie in [0, buckets). One block per token; a thread moves VEC consecutive columns at a time.
+template <typename TW, int VEC>
 __global__ __launch_bounds__(256) void embed_pairs_kernel(const int* __restrict__ ids, const TW* __restrict__ table, float scale,
                                                           const TW* __restrict__ pairs, long long buckets, long long mul_prev,
                                                           long long mul_cur, const int* __restrict__ positions,
@@ -52,12 +52,21 @@ __global__ __launch_bounds__(256) void embed_pairs_kernel(const int* __restrict_
       if (threadIdx.x == 0) *mine = ids[row_start[row + 1] - 1];
     }
   }
+  struct alignas(VEC * sizeof(TW)) Stored { TW e[VEC]; };
+  struct alignas(VEC * 4 > 16 ? 16 : VEC * 4) Columns { float e[VEC]; };
   const size_t at = (size_t)t * width;
-  for (int i = threadIdx.x; i < width; i += 256) {
-    float v = to_f32(src[i]) * scale;
-    if (pair != nullptr) v += to_f32(pair[i]);
-    out[at + i] = v;
-    if (keep != nullptr) keep[at + i] = v;
+  for (int i = threadIdx.x * VEC; i < width; i += 256 * VEC) {
+    const Stored a = *reinterpret_cast<const Stored*>(src + i);
+    Columns v;
+#pragma unroll
+    for (int e = 0; e < VEC; ++e) v.e[e] = to_f32(a.e[e]) * scale;
+    if (pair != nullptr) {
+      const Stored b = *reinterpret_cast<const Stored*>(pair + i);
+#pragma unroll
+      for (int e = 0; e < VEC; ++e) v.e[e] += to_f32(b.e[e]);
+    }
+    *reinterpret_cast<Columns*>(out + at + i) = v;
+    if (keep != nullptr) *reinterpret_cast<Columns*>(keep + at + i) = v;
   }
 }
 
@@ -71,8 +80,10 @@ extern "C" int ms_embed_pairs(const int* ids, const void* table, int is_bf16, fl
                             mul_cur >= buckets || positions == nullptr || token_row == nullptr || row_start == nullptr ||
                             state_slots == nullptr || last == nullptr)))
     return MS_BAD_ARG;
-#define EMB(TW) embed_pairs_kernel<TW><<<tokens, 256, 0, st>>>(ids, (const TW*)table, scale, (const TW*)pairs, buckets, mul_prev, mul_cur, positions, token_row, row_start, state_slots, last, out, keep, width)
-  if (is_bf16) EMB(bf16); else EMB(float);
+  const bool vec = width % 8 == 0 && (size_t)table % 16 == 0 && (size_t)pairs % 16 == 0 && (size_t)out % 16 == 0 && (size_t)keep % 16 == 0;
+#define EMB(TW, V) embed_pairs_kernel<TW, V><<<tokens, 256, 0, st>>>(ids, (const TW*)table, scale, (const TW*)pairs, buckets, mul_prev, mul_cur, positions, token_row, row_start, state_slots, last, out, keep, width)
+  if (is_bf16) { if (vec) EMB(bf16, 8); else EMB(bf16, 1); }
+  else { if (vec) EMB(float, 4); else EMB(float, 1); }
 #undef EMB
   return launch_status();
 }

@@ -171,14 +171,24 @@ extern "C" int ms_map_difference_norm(const void* a, void* out, int in_is_bf16, 
 //   one element side by side, the order in which the matrix cores take the values;
 //   cq [tokens, Q]: the queries' latent after an RMS norm of its own (weight qw).
 // blockIdx.x: the token; blockIdx.y: q_blocks runs of the query's elements, then the cache row, then the queries' latent.
+// A thread owns VEC consecutive elements at a time; VEC = 4 where every part's size, its first column and the rows are
+// multiples of four, and the pairs of a rotation by halves lie whole fours apart.
 struct LatentSource {
   const float* p;
   int ld, splits;
   size_t stride;
-  __device__ __forceinline__ float at(size_t i) const { return splits == 1 ? p[i] : sum_splits(p + i, splits, stride); }
+  // VEC consecutive elements from i on
+  template <int VEC> __device__ __forceinline__ void load(size_t i, float* v) const {
+    if constexpr (VEC == 4) {
+      const float4 q = splits == 1 ? *reinterpret_cast<const float4*>(p + i) : add_splits4(p + i, splits, stride);
+      v[0] = q.x; v[1] = q.y; v[2] = q.z; v[3] = q.w;
+    } else {
+      v[0] = splits == 1 ? p[i] : sum_splits(p + i, splits, stride);
+    }
+  }
 };
 
-template <typename T, typename TW>
+template <typename T, typename TW, int VEC>
 __global__ __launch_bounds__(256) void latent_prepare_kernel(LatentSource q, LatentSource kv, LatentSource dq, int Q,
                                                              const float* __restrict__ rope, int rot, int pairing,
                                                              const TW* __restrict__ cw, const TW* __restrict__ qw, float eps,
@@ -186,72 +196,114 @@ __global__ __launch_bounds__(256) void latent_prepare_kernel(LatentSource q, Lat
                                                              const int* __restrict__ slots, T* __restrict__ kc, T* __restrict__ vc,
                                                              int page_size, int H, int Dn, int R, int C, int q_blocks) {
   __shared__ float red[256 / WAVE];
-  constexpr int KEEP = 4;  // elements of a latent a thread keeps between the two passes (wider ones are read again)
+  constexpr int KEEP = VEC == 4 ? 2 : 4;  // runs of a latent a thread keeps between the two passes (wider ones are read again)
+  struct alignas(VEC * sizeof(T)) Out { T e[VEC]; };
   const int t = blockIdx.x;
   const float* cs = rot > 0 ? rope + (size_t)t * rot : nullptr;
   const int half = rot / 2;
-  // element r of a turned part that begins at `base`
-  auto turned = [&](const LatentSource& src, size_t base, int r) -> float {
-    if (r >= rot) return src.at(base + r);
-    int j, other;
-    bool low;
-    if (pairing == MS_ROPE_ADJACENT) {
-      j = r / 2, low = (r % 2) == 0, other = low ? r + 1 : r - 1;
+  // elements r .. r + VEC - 1 of a turned part that begins at `base`, to dst
+  auto put_turned = [&](const LatentSource& src, size_t base, int r, T* dst) {
+    float v[VEC];
+    src.load<VEC>(base + r, v);
+    Out o;
+    if (r >= rot) {  // (rot is a multiple of VEC)
+#pragma unroll
+      for (int e = 0; e < VEC; ++e) o.e[e] = from_f32<T>(v[e]);
+    } else if (pairing == MS_ROPE_ADJACENT) {
+      if constexpr (VEC == 4) {
+#pragma unroll
+        for (int e = 0; e < 4; e += 2) {
+          const float c = cs[(r + e) / 2], s = cs[half + (r + e) / 2];
+          o.e[e] = from_f32<T>(v[e] * c - v[e + 1] * s);
+          o.e[e + 1] = from_f32<T>(v[e + 1] * c + v[e] * s);
+        }
+      } else {
+        float w[1];
+        src.load<1>(base + (r ^ 1), w);
+        const float c = cs[r / 2], s = cs[half + r / 2];
+        o.e[0] = from_f32<T>(r % 2 == 0 ? v[0] * c - w[0] * s : v[0] * c + w[0] * s);
+      }
     } else {
-      low = r < half, j = low ? r : r - half, other = low ? r + half : r - half;
+      const bool low = r < half;
+      float w[VEC];
+      src.load<VEC>(base + (low ? r + half : r - half), w);
+      const float* c = cs + (low ? r : r - half);
+#pragma unroll
+      for (int e = 0; e < VEC; ++e) o.e[e] = from_f32<T>(low ? v[e] * c[e] - w[e] * c[half + e] : v[e] * c[e] + w[e] * c[half + e]);
     }
-    const float c = cs[j], s = cs[half + j];
-    const float v = src.at(base + r), o = src.at(base + other);
-    return low ? v * c - o * s : v * c + o * s;
+    *reinterpret_cast<Out*>(dst) = o;
   };
   int part = blockIdx.y;
   if (part < q_blocks) {
-    const int n = H * (Dn + R), per = (n + q_blocks - 1) / q_blocks, end = min(n, (part + 1) * per);
+    const int n = H * (Dn + R) / VEC, per = (n + q_blocks - 1) / q_blocks, end = min(n, (part + 1) * per);
     const size_t row = (size_t)t * q.ld;
     for (int i = part * per + threadIdx.x; i < end; i += 256) {
-      const int h = i / (Dn + R), d = i % (Dn + R);
-      if (d < Dn) q_plain[(size_t)t * H * Dn + (size_t)h * Dn + d] = from_f32<T>(q.at(row + i));
-      else q_full[(size_t)t * H * (C + R) + (size_t)h * (C + R) + C + (d - Dn)] = from_f32<T>(turned(q, row + (size_t)h * (Dn + R) + Dn, d - Dn));
+      const int h = i * VEC / (Dn + R), d = i * VEC % (Dn + R);
+      if (d < Dn) {
+        float v[VEC];
+        q.load<VEC>(row + (size_t)i * VEC, v);
+        Out o;
+#pragma unroll
+        for (int e = 0; e < VEC; ++e) o.e[e] = from_f32<T>(v[e]);
+        *reinterpret_cast<Out*>(q_plain + (size_t)t * H * Dn + (size_t)h * Dn + d) = o;
+      } else {
+        put_turned(q, row + (size_t)h * (Dn + R) + Dn, d - Dn, q_full + (size_t)t * H * (C + R) + (size_t)h * (C + R) + C + (d - Dn));
+      }
     }
     return;
   }
   part -= q_blocks;
-  // the RMS norm of n elements from `base` on, element j of the result handed to put(j, value)
+  // the RMS norm of n elements from `base` on, runs of VEC results from element j on handed to put(j, run)
   auto normed = [&](const LatentSource& src, size_t base, int n, const TW* w, auto put) {
-    float kept[KEEP];
+    float kept[KEEP][VEC];
     float ss = 0.f;
 #pragma unroll
     for (int i = 0; i < KEEP; ++i) {
-      const int j = threadIdx.x + i * 256;
-      kept[i] = j < n ? src.at(base + j) : 0.f;
-      ss += kept[i] * kept[i];
+      const int j = (threadIdx.x + i * 256) * VEC;
+#pragma unroll
+      for (int e = 0; e < VEC; ++e) kept[i][e] = 0.f;
+      if (j < n) src.load<VEC>(base + j, kept[i]);
+#pragma unroll
+      for (int e = 0; e < VEC; ++e) ss += kept[i][e] * kept[i][e];
     }
-    for (int j = threadIdx.x + KEEP * 256; j < n; j += 256) {
-      const float v = src.at(base + j);
-      ss += v * v;
+    for (int j = (threadIdx.x + KEEP * 256) * VEC; j < n; j += 256 * VEC) {
+      float v[VEC];
+      src.load<VEC>(base + j, v);
+#pragma unroll
+      for (int e = 0; e < VEC; ++e) ss += v[e] * v[e];
     }
     const float r = 1.f / sqrtf(block_sum<256>(ss, red) / (float)n + eps);
+    auto finish = [&](const float* v, int j) {
+      Out o;
+#pragma unroll
+      for (int e = 0; e < VEC; ++e) o.e[e] = from_f32<T>(v[e] * r * to_f32(w[j + e]));
+      put(j, o);
+    };
 #pragma unroll
     for (int i = 0; i < KEEP; ++i) {
-      const int j = threadIdx.x + i * 256;
-      if (j < n) put(j, kept[i] * r * to_f32(w[j]));
+      const int j = (threadIdx.x + i * 256) * VEC;
+      if (j < n) finish(kept[i], j);
     }
-    for (int j = threadIdx.x + KEEP * 256; j < n; j += 256) put(j, src.at(base + j) * r * to_f32(w[j]));
+    for (int j = (threadIdx.x + KEEP * 256) * VEC; j < n; j += 256 * VEC) {
+      float v[VEC];
+      src.load<VEC>(base + j, v);
+      finish(v, j);
+    }
   };
   if (kv.p != nullptr && part-- == 0) {
     const size_t row = (size_t)t * kv.ld;
     const int slot = slots[t], page = slot / page_size, off = slot % page_size;
     T* dst = kc + (size_t)slot * (C + R);
     T* val = vc + (size_t)page * C * page_size + off;
-    normed(kv, row, C, cw, [&](int j, float v) {
-      const T c = from_f32<T>(v);
-      dst[j] = c;
-      val[(size_t)j * page_size] = c;
+    normed(kv, row, C, cw, [&](int j, const Out& o) {
+      *reinterpret_cast<Out*>(dst + j) = o;
+#pragma unroll
+      for (int e = 0; e < VEC; ++e) val[(size_t)(j + e) * page_size] = o.e[e];
     });
-    for (int j = threadIdx.x; j < R; j += 256) dst[C + j] = from_f32<T>(turned(kv, row + C, j));
+    for (int j = threadIdx.x * VEC; j < R; j += 256 * VEC) put_turned(kv, row + C, j, dst + C + j);
     return;
   }
-  normed(dq, (size_t)t * dq.ld, Q, qw, [&](int j, float v) { cq[(size_t)t * Q + j] = from_f32<T>(v); });
+  normed(dq, (size_t)t * dq.ld, Q, qw, [&](int j, const Out& o) { *reinterpret_cast<Out*>(cq + (size_t)t * Q + j) = o; });
 }
 
 // q: the query rows, or nullptr; x: the rows that hold, from kv_col on (kv_col < 0: nothing is kept), a token's latent and shared
@@ -279,14 +331,21 @@ extern "C" int ms_latent_prepare(const float* q, int q_ld, int q_splits, long lo
   const LatentSource ks{keeps ? x + kv_col : nullptr, ld, splits, (size_t)stride};
   const LatentSource ds{makes ? x + dq_col : nullptr, ld, splits, (size_t)stride};
   const dim3 grid(tokens, q_blocks + keeps + makes);
-#define LP(T, TW)                                                                                                             \
-  latent_prepare_kernel<T, TW><<<grid, 256, 0, st>>>(qs, ks, ds, Q, rope, rot, pairing, (const TW*)cw, (const TW*)qw, eps,      \
+  auto fours = [](const float* p, int row, int n, long long apart) { return (size_t)p % 16 == 0 && row % 4 == 0 && (n <= 1 || apart % 4 == 0); };
+  const bool vec = Dn % 4 == 0 && R % 4 == 0 && C % 4 == 0 && rot % (pairing == MS_ROPE_HALVES ? 8 : 4) == 0 &&
+                   (q == nullptr || fours(q, q_ld, q_splits, q_stride)) &&
+                   (!keeps || (fours(x + kv_col, ld, splits, stride) && (size_t)kc % 16 == 0)) &&
+                   (!makes || (fours(x + dq_col, ld, splits, stride) && Q % 4 == 0));
+#define LP(T, TW) do { if (vec) LPV(T, TW, 4); else LPV(T, TW, 1); } while (0)
+#define LPV(T, TW, V)                                                                                                         \
+  latent_prepare_kernel<T, TW, V><<<grid, 256, 0, st>>>(qs, ks, ds, Q, rope, rot, pairing, (const TW*)cw, (const TW*)qw, eps,      \
                                                      (T*)q_plain, (T*)q_full, (T*)cq, slots, (T*)kc, (T*)vc, page_size, H, Dn, R, C, q_blocks)
   if (out_is_bf16) {
     if (w_is_bf16) LP(bf16, bf16); else LP(bf16, float);
   } else {
     if (w_is_bf16) LP(float, bf16); else LP(float, float);
   }
+#undef LPV
 #undef LP
   return launch_status();
 }

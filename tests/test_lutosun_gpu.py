@@ -213,11 +213,13 @@ def test_bounded_experts_beside_a_gated_shared_one(width, ff, shared, experts, t
         close(stream[torch.tensor(clear)], want[clear], dtype, f"{T} tokens", tol=3e-5 if dtype == torch.float32 else 8e-3)
 
 
+LATENTS = [(3, 16, 8, 8, 12, 24, 40), (5, 6, 6, 4, 14, 23, 22), (8, 64, 32, 32, 64, 64, 96), (4, 32, 32, 16, 48, 1100, 288), (1, 8, 2, 2, 8, 1, 8),
+           (16, 24, 16, 16, 32, 100, 112), (2, 128, 64, 64, 128, 384, 512), (7, 40, 16, 16, 24, 64, 48)]
+
+
 @pytest.mark.parametrize("dtype", DTYPES)
-@pytest.mark.parametrize("heads,dim,rot_dim,dims,value_dim,q_rank,rank", [
-    (3, 16, 8, 8, 12, 24, 40), (5, 6, 6, 4, 14, 23, 22), (8, 64, 32, 32, 64, 64, 96), (4, 32, 32, 16, 48, 1100, 288), (1, 8, 2, 2, 8, 1, 8),
-    (16, 24, 16, 16, 32, 100, 112), (2, 128, 64, 64, 128, 384, 512), (7, 40, 16, 16, 24, 64, 48)])
-@pytest.mark.parametrize("far", [0, 15, 16, 170])
+@pytest.mark.parametrize("heads,dim,rot_dim,dims,value_dim,q_rank,rank,far", [(*s, far) for s in LATENTS for far in (0, 16)] + [
+    (*s, far) for s in (LATENTS[0], LATENTS[2]) for far in (15, 170)])  # two places for every shape, four for two of them
 def test_latent_attention_with_queries_from_a_latent(heads, dim, rot_dim, dims, value_dim, q_rank, rank, far, dtype):
     """The mixer over scattered pages in cuts of every kind: both norms, the second query product, rotation, store, attention over
     every earlier token. The latent of one token (the first, the last of a page, the first of a page, one in the middle) is made
@@ -228,8 +230,6 @@ def test_latent_attention_with_queries_from_a_latent(heads, dim, rot_dim, dims, 
     from miniserve_amd.loading import runtime
     from miniserve_amd.parts.registry import part_class
 
-    if far not in (0, 16) and (heads, dtype) not in ((3, torch.float32), (8, torch.bfloat16)):
-        pytest.skip("two places for every shape, four for two of them")
     rng = np.random.default_rng(heads * dim + rank)
     T, W, eps, scale = 330, 64, 1e-4, 4.0 / np.sqrt(dim + rot_dim)
     m = {"heads": heads, "dim": dim, "rot_dim": rot_dim, "vdim": value_dim, "q_rank": q_rank, "kv_rank": rank, "scale": scale,
